@@ -225,8 +225,8 @@ class ModelRunner:
         else:
             raise ValueError(f"unknown kv_cache_dtype {kv_cache_dtype!r}")
         # per-layer cache shapes: (kv heads, key dim, value dim[, value heads
-        # when fewer than the key heads]), or None for a layer that keeps no
-        # paged keys/values
+        # when fewer than the key heads[, fp32 numbers kept beside every
+        # token]]), or None for a layer that keeps no paged keys/values
         if hasattr(self.model, "kv_cache_specs"):
             self.kv_specs = list(self.model.kv_cache_specs())
         else:
@@ -249,6 +249,15 @@ class ModelRunner:
                      spec[2]),
                     dtype=self.kv_dtype, device=self.device,
                 ),
+            ) + (
+                ()
+                if len(spec) < 5
+                else (
+                    torch.zeros(
+                        (num_gpu_blocks, block_size, spec[4]),
+                        dtype=torch.float32, device=self.device,
+                    ),
+                )
             )
             for spec in self.kv_specs
         ]
@@ -273,8 +282,9 @@ class ModelRunner:
 
     def _profile_num_blocks(self, gpu_memory_utilization: float) -> int:
         per_block_bytes = sum(
-            self.block_size * (spec[0] * spec[1] + (spec[3] if len(spec) > 3 else spec[0])
-                               * spec[2]) * self.kv_dtype.itemsize
+            self.block_size * ((spec[0] * spec[1] + (spec[3] if len(spec) > 3 else spec[0])
+                                * spec[2]) * self.kv_dtype.itemsize
+                               + (4 * spec[4] if len(spec) > 4 else 0))
             for spec in self.kv_specs
             if spec is not None
         )

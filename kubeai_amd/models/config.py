@@ -85,6 +85,8 @@ class ModelArchConfig:
             return vekusun_arch_config(cfg)
         if cfg.get("architecture") == "Vigonex":
             return vigonex_arch_config(cfg)
+        if cfg.get("architecture") == "Pubopel":
+            return pubopel_arch_config(cfg)
         hidden = cfg["hidden_size"]
         n_heads = cfg["num_attention_heads"]
         arch = (cfg.get("architectures") or ["LlamaForCausalLM"])[0]
@@ -347,6 +349,38 @@ def vigonex_arch_config(cfg: dict) -> ModelArchConfig:
             canon_taps=0,
             streams=streams,
             logit_scale=float(cfg.get("logit_scale", 1.0)),
+        ),
+    )
+
+
+def pubopel_arch_config(cfg: dict) -> ModelArchConfig:
+    """Pubopel config.json -> arch config: the list of layers (mixer type, the
+    mixer's sizes and constants, the feed-forward), the taps of the input
+    convolutions and the norm epsilon, all as the file gives them."""
+    layers = [
+        HybridLayerSpec(type=L["type"], mixer=L["mixer"], mlp=L.get("mlp"), weights_of=i)
+        for i, L in enumerate(cfg["layers"])
+    ]
+    taps = int(cfg["canon"]["taps"])
+    if taps < 1:
+        raise ValueError("canon.taps must be at least 1")
+    return ModelArchConfig(
+        architecture="pubopel",
+        vocab_size=int(cfg["vocab"]),
+        hidden_size=int(cfg["width"]),
+        num_hidden_layers=len(layers),
+        intermediate_size=0,
+        num_attention_heads=0,
+        num_key_value_heads=0,
+        head_dim=0,
+        max_position_embeddings=1 << 30,  # positions enter as score biases
+        bos_token_id=-1,
+        eos_token_id=-1,  # the design defines no end token
+        hybrid=HybridSpec(
+            layers=layers,
+            norm_eps=float(cfg["norm"]["eps"]),
+            embedding_scale=1.0,
+            canon_taps=taps,
         ),
     )
 
@@ -899,6 +933,34 @@ def vigonex_preset(width: int, layers: int, vocab: int = 32000, head_dim: int = 
     })
 
 
+def pubopel_preset(width: int, layers: int, vocab: int = 32000, head_dim: int = 128,
+                   window: int = 1024, keep_first: int = 8, experts: int = 8,
+                   top: int = 2, ff_scale: float = 1.0) -> ModelArchConfig:
+    """A Pubopel stack of the given size with random-init weights. Odd layers
+    attend over a sliding window (with the first tokens kept), even layers
+    over everything; width/head_dim query heads over a quarter as many
+    key/value heads; every layer has a routed feed-forward with a shared
+    expert, whose work per token (chosen experts + shared) is that of a dense
+    3.5 x width gated layer (times ff_scale, for matching another model's
+    size)."""
+    heads = max(1, width // head_dim)
+    ff = max(16, int(3.5 * ff_scale * width / (top + 1)) // 16 * 16)
+    mlp = {"kind": "moe", "expert": {"ff": ff},
+           "router": {"experts": experts, "top": top}, "shared": {"ff": ff}}
+    att = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": head_dim,
+           "vdim": head_dim, "scale": head_dim ** -0.5, "softcap": 30.0}
+    out = []
+    for i in range(layers):
+        mixer = dict(att)
+        if i % 2:
+            mixer["mask"] = {"size": window, "keep_first": keep_first}
+        out.append({"type": "attention", "mixer": mixer, "mlp": mlp})
+    return pubopel_arch_config({
+        "architecture": "Pubopel", "vocab": vocab, "width": width,
+        "norm": {"eps": 1e-5}, "canon": {"taps": 3}, "layers": out,
+    })
+
+
 def dulotar_preset(width: int, layers: int, vocab: int = 32000, head_dim: int = 128,
                    chunk: int = 1024, ff_mult: int = 4) -> ModelArchConfig:
     """A Dulotar stack of the given size with random-init weights: the
@@ -945,6 +1007,11 @@ PRESETS.update({
     "vigonex-1k": vigonex_preset(1024, 12),
     "vigonex-2k": vigonex_preset(2048, 12),
     "vigonex-4k": vigonex_preset(4096, 6),
+    "pubopel-tiny": pubopel_preset(128, 4, vocab=512, head_dim=32, window=40,
+                                   keep_first=3, experts=4, top=2),
+    "pubopel-1k": pubopel_preset(1024, 12),
+    "pubopel-2k": pubopel_preset(2048, 12),
+    "pubopel-4k": pubopel_preset(4096, 6),
     "dulotar-tiny": dulotar_preset(128, 3, vocab=512, head_dim=32, chunk=64),
     "dulotar-1k": dulotar_preset(1024, 12),
     "dulotar-2k": dulotar_preset(2048, 12),

@@ -469,6 +469,70 @@ class LatentAttention(nn.Module):
         return self.o_proj(o.view(T, H * Dv))
 
 
+class TiedValueAttention(nn.Module):
+    """Causal softmax attention whose values are its keys as projected (before
+    their norm), so that the cache keeps one row per token and key/value head.
+    An RMS norm runs over the whole q and the whole k projection (all heads at
+    once). No rotation: positions enter as a bias -slope_h * (i - j) taken off
+    after the tanh cap. Options, each a constructor argument: the cap, a
+    sliding window, first tokens that stay visible behind it, the slopes
+    (None: no bias), a learned score per head in the softmax denominator.
+
+    With r_j = 1 / rms(k_j) the normed key is r_j w_k * k_j, so a score is
+    r_j ((q_hat * w_q * w_k) . k_j): the cache holds the projected k_j, which
+    is the value as well, and r_j beside it (fp32), and q's weight carries
+    w_k and the heads' score multipliers (fold_query_weight)."""
+
+    def __init__(self, width, heads, kv_heads, dim, scale, softcap=0.0, window=0,
+                 keep_first=0, slopes=None, sink=True, eps=1e-6):
+        super().__init__()
+        if heads % kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        self.heads, self.kv_heads, self.dim, self.eps = heads, kv_heads, dim, eps
+        self.scale, self.softcap = float(scale), float(softcap or 0.0)
+        self.window, self.keep_first = int(window or 0), int(keep_first or 0)
+        self.sizes = (heads * dim, kv_heads * dim)
+        self.in_proj = Proj(width, sum(self.sizes))  # q | k
+        self.o_proj = Proj(heads * dim, width)
+        self.q_weight = _f32(heads * dim)
+        nn.init.ones_(self.q_weight)
+        self.sink_scores = _f32(heads) if sink else None
+        self.register_buffer(
+            "slopes",
+            None if slopes is None else torch.tensor(list(slopes), dtype=torch.float32),
+            persistent=False)
+
+    def fold_query_weight(self, q_norm, k_norm, temp):
+        """fp32 [H * D]: q's norm weight times the head's score multiplier
+        times the norm weight of the key head it meets."""
+        H, G, D = self.heads, self.kv_heads, self.dim
+        kw = k_norm.float().view(G, 1, D).expand(G, H // G, D).reshape(H, D)
+        return (q_norm.float().view(H, D) * temp.float().view(H, 1) * kw).reshape(-1)
+
+    def state_spec(self):
+        return {}
+
+    def kv_spec(self):
+        # rows that are key and value, and one fp32 number per token
+        return (self.kv_heads, self.dim, 0, self.kv_heads, 1)
+
+    def forward(self, h, fb, state, kv_cache):
+        T = h.shape[0]
+        nq, _ = self.sizes
+        qk = self.in_proj(h)
+        q = qk[:, :nq].unflatten(-1, (self.heads, self.dim))
+        k = qk[:, nq:].unflatten(-1, (self.kv_heads, self.dim))
+        rows, _, key_scale = kv_cache
+        sops.qnorm_rows_to_cache(q, k, self.q_weight, self.eps, rows, key_scale,
+                                 fb.slot_mapping)
+        out = torch.empty((T, self.heads, self.dim), dtype=h.dtype, device=h.device)
+        sops.masked_paged_attention(
+            q, rows, rows, fb.seq, self.scale, out, softcap=self.softcap,
+            window=self.window, keep_first=self.keep_first, slopes=self.slopes,
+            key_scale=key_scale, sink=self.sink_scores)
+        return self.o_proj(out.view(T, self.heads * self.dim))
+
+
 class GatedDeltaMixer(nn.Module):
     """Gated delta rule: a matrix state per head that decays by a
     data-dependent factor and is corrected towards the current value along
@@ -589,10 +653,11 @@ class RoutedSquaredReluMoE(nn.Module):
 
 class RoutedGatedMoE(nn.Module):
     """Mixture of gated experts (down(act(gate h) * (up h)), no biases).
-    Routing: fp32 logits, scores = softmax over all experts; the `top`
-    experts with the largest score + correction (a per-expert bias that only
+    Routing: fp32 logits, scores = softmax over all experts, or every logit's
+    sigmoid (score="sigmoid"); the `top` experts with the largest score + correction (a per-expert bias that only
     steers the choice) are used, weighted by their scores as they are (times
-    weight_scale).
+    weight_scale). weight_on="input": the weight multiplies what the expert
+    reads instead of what it returns.
 
     The activation is g * sigmoid(act_alpha * g) * (u + up_shift), with
     g = min(gate, act_limit) and u = clamp(up, +-act_limit) when act_limit > 0
@@ -617,8 +682,12 @@ class RoutedGatedMoE(nn.Module):
 
     def __init__(self, width, experts, top, ff, correction=True, act_alpha=1.0,
                  act_limit=0.0, up_shift=0.0, weight_scale=1.0, shared_ff=0,
-                 shared_limit=0.0, shared_gate=False, extra_out=0):
+                 shared_limit=0.0, shared_gate=False, extra_out=0, score="softmax",
+                 weight_on="output"):
         super().__init__()
+        if score not in ("softmax", "sigmoid") or weight_on not in ("input", "output"):
+            raise ValueError(f"unknown routing {score!r} / {weight_on!r}")
+        self.score, self.w_input = score, weight_on == "input"
         self.experts, self.top, self.ff = experts, top, ff
         self.act = dict(alpha=float(act_alpha), limit=float(act_limit or 0.0),
                         up_shift=float(up_shift))
@@ -644,13 +713,13 @@ class RoutedGatedMoE(nn.Module):
         sg = logits[:, E:] if self.shared_gate else None
         dense, w, idx = sops.router_scores_topk(
             logits[:, :E] if self.shared_gate else logits, self.top, self.correction,
-            self.weight_scale)
+            self.weight_scale, self.score)
         at = E * 2 * ff + 2 * sff  # where the caller's extra projection starts
         if T <= self.DENSE_MAX_TOKENS:
             gu = self.gate_up(h)
             a = torch.empty((T, E * ff + sff), dtype=h.dtype, device=h.device)
             sops.glu_weighted(gu[:, : E * 2 * ff], dense, ff, out=a[:, : E * ff],
-                              **self.act)
+                              w_input=self.w_input, **self.act)
             if sff:
                 sops.glu_weighted(gu[:, E * 2 * ff : at], sg, sff, w_sigmoid=True,
                                   out=a[:, E * ff :], **self.shared_act)
@@ -670,7 +739,7 @@ class RoutedGatedMoE(nn.Module):
             rows = tok[s : s + n]
             gu = F.linear(h.index_select(0, rows),
                           self.gate_up.weight[e * 2 * ff : (e + 1) * 2 * ff])
-            a = sops.glu_weighted(gu, wrow[s : s + n], ff, **self.act)
+            a = sops.glu_weighted(gu, wrow[s : s + n], ff, w_input=self.w_input, **self.act)
             y = F.linear(a, self.down.weight[:, e * ff : (e + 1) * ff])
             out.index_add_(0, rows, y.float())
             s += n

@@ -33,6 +33,12 @@ def _vigonex():
     return VigonexForCausalLM
 
 
+def _pubopel():
+    from .pubopel import PubopelForCausalLM
+
+    return PubopelForCausalLM
+
+
 MODEL_REGISTRY = {
     "llama": _llama,
     "mixtral": _llama,
@@ -40,6 +46,7 @@ MODEL_REGISTRY = {
     "nugopel": _nugopel,
     "vekusun": _vekusun,
     "vigonex": _vigonex,
+    "pubopel": _pubopel,
 }
 
 
@@ -61,6 +68,7 @@ MODEL_EXTENSIONS = {
     "nugopel": ("_C_seq",),
     "vekusun": ("_C_seq",),
     "vigonex": ("_C_seq",),
+    "pubopel": ("_C_seq",),
 }
 
 

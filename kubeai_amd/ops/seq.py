@@ -206,6 +206,36 @@ def scaled_add_rmsnorm(residual, a, a_scale, b, b_scale, mult: float, extra,
     return (residual * r * weight).to(out_dtype)
 
 
+def add_dyt_conv(branch, post, residual, pre, conv_w, tails, meta: SeqMeta, out_dtype):
+    """A sublayer's output joins the residual and the next sublayer's input is
+    formed, where the norms are dynamic tanh, dyt(x) = tanh(alpha x) * w + b
+    (elementwise, no statistics), and the input passes a causal convolution:
+
+        residual' = residual + dyt_post(branch)
+        h = dyt_pre(residual')
+        out_t = h_t + sum_j conv_w[:, j] * h_(t - taps + 1 + j)     (out_dtype)
+
+    post, pre: (alpha fp32 [1], w fp32 [C], b fp32 [C]); branch [T, C]
+    (serving dtype or fp32) may be None (residual' = residual). conv_w fp32
+    [C, taps], tails fp32 [slots, taps - 1, C] with the conventions of
+    causal_conv; conv_w None: out = h. h enters the convolution and the tails
+    in fp32. Returns (out, residual'); residual itself is left as it was."""
+    if residual.is_cuda:
+        _require_ext()
+        out = torch.empty(residual.shape, dtype=out_dtype, device=residual.device)
+        new = residual if branch is None else torch.empty_like(residual)
+        _C.add_dyt_conv(out, new, branch, *(post if branch is not None else (None,) * 3),
+                        residual, *pre, conv_w, tails, meta.start_loc, meta.slots,
+                        meta.positions, meta.max_len)
+        return out, new
+    if branch is not None:
+        residual = residual + torch.tanh(post[0] * branch.float()) * post[1] + post[2]
+    h = torch.tanh(pre[0] * residual) * pre[1] + pre[2]
+    if conv_w is not None:
+        h = causal_conv(h, conv_w, tails, meta, residual=True)
+    return h.to(out_dtype), residual
+
+
 def tanh_cap(x, cap: float):
     """cap * tanh(x / cap) on an fp32 tensor, in place."""
     if x.is_cuda:
@@ -570,6 +600,32 @@ def latent_rope_to_cache(x, weight, eps: float, q_rot, q_out, positions,
     flat[slot_mapping[ok].long()] = y[ok].to(cache.dtype)
 
 
+def qnorm_rows_to_cache(q, k, q_weight, eps: float, cache, key_scale, slot_mapping):
+    """Whole-row RMS norms of q and k (all heads at once) when the cached row
+    is to serve as key and value: q <- q / rms(q) * q_weight in place, k's row
+    goes to the cache as it is, and 1 / rms(k), the number that turns it into
+    the normed key (up to a per-channel weight, which the caller folds into
+    q_weight), goes to key_scale. rms(x) = sqrt(mean(x^2) + eps), fp32.
+    q [T, H, D], k [T, G, D] may be strided views, q_weight fp32 [H * D], cache
+    [blocks, G, block, D], key_scale fp32 [blocks, block, 1]; slot < 0: no
+    write."""
+    if q.is_cuda:
+        _require_ext()
+        _C.qnorm_rows_to_cache(q, k, q_weight, eps, cache, key_scale, slot_mapping)
+        return q
+    T = q.shape[0]
+    qf, kf = q.float().reshape(T, -1), k.float().reshape(T, -1)
+    qf = qf * torch.rsqrt((qf * qf).mean(-1, keepdim=True) + eps) * q_weight
+    q.copy_(qf.view(q.shape).to(q.dtype))
+    bs = cache.shape[2]
+    ok = slot_mapping >= 0
+    blk = (slot_mapping[ok] // bs).long()
+    off = (slot_mapping[ok] % bs).long()
+    cache[blk, :, off] = k[ok].to(cache.dtype)
+    key_scale[blk, off, 0] = torch.rsqrt((kf * kf).mean(-1) + eps)[ok]
+    return q
+
+
 def sigmoid_gate(x, gate, out=None):
     """x * sigmoid(gate), elementwise; gate may be a strided column view."""
     if out is None:
@@ -645,8 +701,10 @@ def relu_squared_weighted(u, w, group: int):
     return r.to(u.dtype)
 
 
-def router_scores_topk(logits, top: int, bias=None, scale: float = 1.0):
-    """Routing by scores: s = softmax(logits) over all experts (fp32); the
+def router_scores_topk(logits, top: int, bias=None, scale: float = 1.0,
+                       score: str = "softmax"):
+    """Routing by scores: s = softmax(logits) over all experts, or every
+    logit's sigmoid (score), in fp32; the
     `top` experts with the largest s + bias are chosen (equal values: lower
     index first; bias fp32 [E] or None), and their weights are their scores
     s themselves times `scale`, not renormalised. Returns (dense [T, E] with the weights at
@@ -657,9 +715,10 @@ def router_scores_topk(logits, top: int, bias=None, scale: float = 1.0):
         dense = torch.empty((T, E), dtype=torch.float32, device=logits.device)
         w = torch.empty((T, top), dtype=torch.float32, device=logits.device)
         idx = torch.empty((T, top), dtype=torch.int32, device=logits.device)
-        _C.router_scores_topk(logits.contiguous(), bias, dense, w, idx, scale)
+        _C.router_scores_topk(logits.contiguous(), bias, dense, w, idx, scale,
+                              {"softmax": 0, "sigmoid": 1}[score])
         return dense, w, idx
-    s = torch.softmax(logits.float(), dim=-1)
+    s = torch.softmax(logits.float(), -1) if score == "softmax" else torch.sigmoid(logits.float())
     choice = s if bias is None else s + bias
     idx = torch.sort(choice, dim=-1, descending=True, stable=True).indices[:, :top]
     w = torch.gather(s, 1, idx) * scale
@@ -677,7 +736,8 @@ def silu_mul_weighted(gu, w, group: int):
 
 
 def glu_weighted(gu, w, group: int, *, alpha: float = 1.0, limit: float = 0.0,
-                 up_shift: float = 0.0, w_sigmoid: bool = False, out=None):
+                 up_shift: float = 0.0, w_sigmoid: bool = False,
+                 w_input: bool = False, out=None):
     """Gated activation over blocks of `group` gate columns followed by
     `group` up columns (gu [T, n * 2 * group], rows may be strided):
 
@@ -685,25 +745,31 @@ def glu_weighted(gu, w, group: int, *, alpha: float = 1.0, limit: float = 0.0,
         out[t, e * group + c] = g * sigmoid(alpha * g) * (u + up_shift) * w[t, e]
 
     alpha = 1 is silu. w fp32 [T, n] (strided columns view fine) or None (no
-    weight); with w_sigmoid the weight is sigmoid(w). out [T, n * group] may
-    be a strided column view of a wider buffer. fp32 inside."""
+    weight); with w_sigmoid the weight is sigmoid(w). w_input: the weight
+    belongs to the expert's input instead of its output, so it multiplies gate
+    and up (both linear in the input) before anything else. out [T, n * group]
+    may be a strided column view of a wider buffer. fp32 inside."""
     T, C2 = gu.shape
     n = C2 // (2 * group)
     if out is None:
         out = torch.empty((T, n * group), dtype=gu.dtype, device=gu.device)
     if gu.is_cuda:
         _require_ext()
-        _C.glu_weighted(out, gu, w, group, alpha, limit, up_shift, w_sigmoid)
+        _C.glu_weighted(out, gu, w, group, alpha, limit, up_shift, w_sigmoid, w_input)
         return out
     g = gu.float().reshape(T, n, 2, group)
     gate, up = g[:, :, 0], g[:, :, 1]
+    wf = None
+    if w is not None:
+        wf = (torch.sigmoid(w.float()) if w_sigmoid else w.float()).unsqueeze(-1)
+        if w_input:
+            gate, up, wf = gate * wf, up * wf, None
     if limit > 0:
         gate = gate.clamp(max=limit)
         up = up.clamp(-limit, limit)
     a = gate * torch.sigmoid(alpha * gate) * (up + up_shift)
-    if w is not None:
-        wf = torch.sigmoid(w.float()) if w_sigmoid else w.float()
-        a = a * wf.unsqueeze(-1)
+    if wf is not None:
+        a = a * wf
     out.copy_(a.reshape(T, n * group).to(out.dtype))
     return out
 
@@ -715,12 +781,18 @@ def glu_weighted(gu, w, group: int, *, alpha: float = 1.0, limit: float = 0.0,
 def masked_paged_attention(q, k_cache, v_cache, meta: SeqMeta, scale: float,
                            out, *, softcap: float = 0.0, chunk: int = 0,
                            window: int = 0, out_scale: float = 1.0,
-                           sink: Optional[torch.Tensor] = None):
+                           sink: Optional[torch.Tensor] = None,
+                           keep_first: int = 0,
+                           slopes: Optional[torch.Tensor] = None,
+                           key_scale: Optional[torch.Tensor] = None):
     """Softmax attention of every packed token over its own sequence's cached
     keys. The token at position i sees j <= i with, when chunk > 0,
     floor(j / chunk) == floor(i / chunk) (position-aligned chunks) and, when
-    window > 0, j > i - window. Scores are (q . k) * scale, then
-    softcap * tanh(score / softcap) if softcap > 0; all in fp32. With sink
+    window > 0, j > i - window or j < keep_first (the first tokens stay
+    visible; no chunks then). Scores are (q . k) * scale, times the key
+    token's key_scale (fp32 [blocks, block, 1], paged as the keys are) if one
+    is given, then softcap * tanh(score / softcap) if softcap > 0, then minus
+    slopes[h] * (i - j) (fp32 [H]) if slopes are given; all in fp32. With sink
     (fp32 [H]), the softmax of head h has one more key whose score is
     sink[h] as it stands (not scaled, not capped) and that carries no value:
     the denominator grows by exp(sink[h]).
@@ -731,6 +803,10 @@ def masked_paged_attention(q, k_cache, v_cache, meta: SeqMeta, scale: float,
     one value head);
     out [T, H, Dv] may be a strided view; out = attention * out_scale.
     sink=True stands for a score of 0 on every head."""
+    if keep_first and chunk:
+        raise ValueError("kept first tokens and chunks do not combine")
+    if not window:
+        keep_first = 0  # nothing is hidden behind a window
     if sink is True:
         sink = torch.zeros(q.shape[1], dtype=torch.float32, device=q.device)
     elif sink is False:
@@ -740,7 +816,7 @@ def masked_paged_attention(q, k_cache, v_cache, meta: SeqMeta, scale: float,
         _C.masked_paged_attention(out, q, k_cache, v_cache, meta.block_tables,
                                   meta.start_loc, meta.token_seq, meta.positions,
                                   meta.max_len, scale, softcap, chunk, window,
-                                  out_scale, sink)
+                                  out_scale, sink, keep_first, slopes, key_scale)
         return out
     T, H, D = q.shape
     G, bs = k_cache.shape[1], k_cache.shape[2]
@@ -758,20 +834,24 @@ def masked_paged_attention(q, k_cache, v_cache, meta: SeqMeta, scale: float,
             lo = (int(pos.min()) // chunk) * chunk
         if window > 0:
             lo = max(lo, int(pos.min()) - window + 1)
-        j = torch.arange(lo, L)
+        j = torch.cat([torch.arange(0, min(keep_first, lo)), torch.arange(lo, L)])
         blk = bt[si][(j // bs)].long()
         ks = k_cache[blk, :, j % bs].float()  # [L', G, D]
         vs = v_cache[blk, :, j % bs].float()
         ks = ks.repeat_interleave(rep, dim=1)
         vs = vs.repeat_interleave(rep_v, dim=1)
         s = torch.einsum("thd,lhd->htl", q[s0 : s0 + n].float(), ks) * scale
+        if key_scale is not None:
+            s = s * key_scale[blk, j % bs, 0]
         if softcap > 0:
             s = softcap * torch.tanh(s / softcap)
+        if slopes is not None:
+            s = s - slopes.view(H, 1, 1) * (pos.view(-1, 1) - j.view(1, -1)).float()
         vis = j.view(1, -1) <= pos.view(-1, 1)
         if chunk > 0:
             vis &= (j.view(1, -1) // chunk) == (pos.view(-1, 1) // chunk)
         if window > 0:
-            vis &= j.view(1, -1) > pos.view(-1, 1) - window
+            vis &= (j.view(1, -1) > pos.view(-1, 1) - window) | (j.view(1, -1) < keep_first)
         s = s.masked_fill(~vis.unsqueeze(0), float("-inf"))
         if sink is not None:
             s = torch.cat(
