@@ -1,9 +1,12 @@
 // Rotary (interleaved pairs, or split halves after a whole-row RMS norm of q
 // and k) fused with the paged cache write, and softmax attention of every
 // packed token over its own sequence's cached keys under a chunk / window
-// mask, with separate key and value sizes and an optional sink (a key of
-// score 0 without a value: one more term in the denominator).
+// mask, with separate key and value sizes. Options: first tokens that stay
+// visible behind a window, a tanh cap, a bias per position, a scale per cached
+// key, and a sink (a score without a value: one more term in the denominator).
 #include "seq_common.h"
+
+#include <type_traits>
 
 namespace {
 
@@ -132,7 +135,89 @@ __global__ __launch_bounds__(256) void qknorm_rope_half_cache_kernel(
   }
 }
 
+// grid (T). Whole-row RMS norms of q and k when a cached row is key and value:
+// q <- q / rms(q) * w in place; k's row goes to the cache as it is and
+// 1 / rms(k) to key_scale. kVec: 16-byte accesses (rows and heads of whole,
+// aligned vectors).
+template <typename T, bool kVec>
+__global__ __launch_bounds__(256) void qnorm_rows_cache_kernel(
+    T* __restrict__ q, int64_t q_stride, const T* __restrict__ k, int64_t k_stride,
+    const float* __restrict__ w, float eps, T* __restrict__ cache,
+    float* __restrict__ key_scale, const int64_t* __restrict__ slot_mapping, int H,
+    int G, int D, int bs) {
+  constexpr int N = kVec ? Vec16<T>::N : 1;
+  __shared__ float red0[16], red1[16];
+  const int t = blockIdx.x;
+  const int64_t slot = slot_mapping[t];
+  T* qr = q + (size_t)t * q_stride;
+  const T* kr = k + (size_t)t * k_stride;
+  const int nq = H * D, nk = G * D;
+  auto load = [](const T* p, float* x) {
+    if constexpr (kVec) Vec16<T>::load(p, x);
+    else x[0] = ldf(p);
+  };
+  float sq = 0.f, sk = 0.f;
+  for (int i = threadIdx.x * N; i < nq; i += blockDim.x * N) {
+    float x[N];
+    load(qr + i, x);
+#pragma unroll
+    for (int e = 0; e < N; ++e) sq += x[e] * x[e];
+  }
+  const int64_t blk = slot >= 0 ? slot / bs : 0;
+  const int off = slot >= 0 ? (int)(slot % bs) : 0;
+  for (int i = threadIdx.x * N; i < nk; i += blockDim.x * N) {
+    float x[N];
+    load(kr + i, x);
+#pragma unroll
+    for (int e = 0; e < N; ++e) sk += x[e] * x[e];
+    if (slot >= 0) {
+      const int g = i / D, d = i % D;
+      T* dst = cache + (((size_t)blk * G + g) * bs + off) * D + d;
+      if constexpr (kVec) *(uint4*)dst = *(const uint4*)(kr + i);
+      else *dst = kr[i];
+    }
+  }
+  const float rq = 1.0f / sqrtf(block_sum(sq, red0) / (float)nq + eps);
+  const float rk = 1.0f / sqrtf(block_sum(sk, red1) / (float)nk + eps);
+  if (slot >= 0 && threadIdx.x == 0) key_scale[slot] = rk;
+  for (int i = threadIdx.x * N; i < nq; i += blockDim.x * N) {
+    float x[N];
+    load(qr + i, x);
+#pragma unroll
+    for (int e = 0; e < N; ++e) x[e] *= rq * w[i + e];
+    if constexpr (kVec) Vec16<T>::store(qr + i, x);
+    else stf(qr + i, x[0]);
+  }
+}
+
 constexpr int kMaxDvPerLane = 16;  // value size <= 1024
+constexpr float kLog2e = 1.4426950408889634f;
+
+// What every attention kernel below needs to know about scores and rows.
+// Visible keys of position p: [0, kept(p)) and [lower(p), p].
+struct AttnArgs {
+  float scale, softcap, out_scale;
+  int chunk, window, keep;
+  const float* sink;    // [H] or null: score of a key without a value
+  const float* slopes;  // [H] or null: slopes[h] * (i - j) comes off a score
+  const float* kscale;  // [blocks, bs] or null: factor of a cached key's scores
+  int64_t v_rs;         // elements between value rows
+  int H, G, D, Dv, bs, kvs;
+
+  DEV_INLINE int lower(int p) const {
+    int lo = 0;
+    if (chunk > 0) lo = (p / chunk) * chunk;
+    if (window > 0) lo = max(lo, p - window + 1);
+    return lo;
+  }
+  DEV_INLINE int kept(int lo) const { return min(keep, lo); }
+};
+
+// softcap * tanh(x / softcap) times log2 e as cap2 - 2 cap2 / (e^(2x/cap) + 1):
+// absolute error below 1e-6 of the cap. x comes multiplied by 2 log2(e) / cap.
+DEV_INLINE float cap_base2(float x, float cap2) {
+  return cap2 - 2.f * cap2 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(x) + 1.f);
+}
 
 constexpr int kDecWaves = 4;
 
@@ -154,9 +239,8 @@ __global__ __launch_bounds__(kDecWaves * WAVE) void masked_paged_attention_kerne
     int64_t q_stride, const T* __restrict__ k_cache,
     const T* __restrict__ v_cache, const int* __restrict__ block_tables,
     int max_blocks, const int* __restrict__ token_seq,
-    const int* __restrict__ positions, float scale, float softcap, int chunk,
-    int window, float out_scale, const float* __restrict__ sink, int64_t v_rs, int H, int G, int D, int Dv, int bs,
-    int kvs) {
+    const int* __restrict__ positions, AttnArgs a) {
+  const int H = a.H, G = a.G, D = a.D, Dv = a.Dv, bs = a.bs;
   constexpr int N = Vec16<T>::N;
   const int lpr = kVec ? Dv / N : 1;          // lanes per value row
   const int ngrp = kVec ? WAVE / lpr : 1;     // key groups of a wave
@@ -172,9 +256,9 @@ __global__ __launch_bounds__(kDecWaves * WAVE) void masked_paged_attention_kerne
   const int g = h / (H / G);
   const int pos = positions[t];
   const int* bt = block_tables + (size_t)token_seq[t] * max_blocks;
-  int lo = 0;
-  if (chunk > 0) lo = (pos / chunk) * chunk;
-  if (window > 0) lo = max(lo, pos - window + 1);
+  // the visible keys are numbered 0 .. n_keys - 1: kept first tokens, then lo .. pos
+  const int lo = a.lower(pos), kept = a.kept(lo), n_keys = kept + pos - lo + 1;
+  const float slope = a.slopes != nullptr ? a.slopes[h] : 0.f;
   for (int i = threadIdx.x; i < D; i += blockDim.x)
     qs[i] = ldf(q + (size_t)t * q_stride + h * D + i);
   __syncthreads();
@@ -186,11 +270,12 @@ __global__ __launch_bounds__(kDecWaves * WAVE) void masked_paged_attention_kerne
   for (int i = 0; i < kMaxDvPerLane; ++i) acc[i] = 0.f;
   // the wave's own LDS rows are touched by this wave only, so the tile loop
   // needs no block barrier (a wave's LDS accesses complete in order)
-  for (int j0 = lo + wave * WAVE; j0 <= pos; j0 += kDecWaves * WAVE) {
-    const int j = j0 + lane;
+  for (int v0 = wave * WAVE; v0 < n_keys; v0 += kDecWaves * WAVE) {
+    const int vk = v0 + lane;
     float sc = -INFINITY;
     int64_t vb = 0;
-    if (j <= pos) {
+    if (vk < n_keys) {
+      const int j = vk < kept ? vk : lo + vk - kept;
       const int64_t blk = bt[j / bs];
       const int64_t rowi = (blk * G + g) * bs + (j % bs);
       const T* kp = k_cache + rowi * D;
@@ -205,12 +290,14 @@ __global__ __launch_bounds__(kDecWaves * WAVE) void masked_paged_attention_kerne
       } else {
         for (int i = 0; i < D; ++i) dot += qs[i] * ldf(kp + i);
       }
-      sc = dot * scale;
-      if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);
-      vb = ((blk * (G / kvs) + g / kvs) * bs + (j % bs)) * v_rs;
+      sc = dot * a.scale;
+      if (a.kscale != nullptr) sc *= a.kscale[blk * bs + j % bs];
+      if (a.softcap > 0.f) sc = a.softcap * tanhf(sc / a.softcap);
+      sc -= slope * (float)(pos - j);
+      vb = ((blk * (G / a.kvs) + g / a.kvs) * bs + (j % bs)) * a.v_rs;
     }
     const float m_new = fmaxf(m, wave_max(sc));  // finite: lane 0's key is visible
-    const float p = j <= pos ? expf(sc - m_new) : 0.f;
+    const float p = vk < n_keys ? expf(sc - m_new) : 0.f;
     const float corr = expf(m - m_new);  // m = -inf on the wave's first tile -> 0
     l = l * corr + wave_sum(p);
     m = m_new;
@@ -218,7 +305,7 @@ __global__ __launch_bounds__(kDecWaves * WAVE) void masked_paged_attention_kerne
     vbase[lane] = vb;
     __builtin_amdgcn_s_waitcnt(0xc07f);  // lgkmcnt(0): the wave's LDS writes landed
     __builtin_amdgcn_wave_barrier();
-    const int nk = min(WAVE, pos - j0 + 1);
+    const int nk = min(WAVE, n_keys - v0);
     if (kVec) {
 #pragma unroll
       for (int e = 0; e < N; ++e) acc[e] *= corr;
@@ -236,9 +323,9 @@ __global__ __launch_bounds__(kDecWaves * WAVE) void masked_paged_attention_kerne
       for (int c = 0; c < kMaxDvPerLane; ++c) {
         const int d = c * WAVE + lane;
         if (d < Dv) {
-          float a = acc[c] * corr;
-          for (int jj = 0; jj < nk; ++jj) a += ps[jj] * ldf(v_cache + vbase[jj] + d);
-          acc[c] = a;
+          float x = acc[c] * corr;
+          for (int jj = 0; jj < nk; ++jj) x += ps[jj] * ldf(v_cache + vbase[jj] + d);
+          acc[c] = x;
         }
       }
     }
@@ -270,17 +357,17 @@ __global__ __launch_bounds__(kDecWaves * WAVE) void masked_paged_attention_kerne
     wsc[w] = mw == -INFINITY ? 0.f : expf(mw - mx);  // a wave may have had no tile
     lsum += stat[2 * w + 1] * wsc[w];
   }
-  if (sink != nullptr) lsum += expf(sink[h] - mx);
-  const float inv = out_scale / lsum;
+  if (a.sink != nullptr) lsum += expf(a.sink[h] - mx);
+  const float inv = a.out_scale / lsum;
   for (int d = threadIdx.x; d < Dv; d += blockDim.x) {
-    float a = 0.f;
+    float x = 0.f;
     for (int w = 0; w < kDecWaves; ++w) {
       const float* rw = red_all + (size_t)w * ngrp * Dv;
       float part = 0.f;
       for (int gi = 0; gi < ngrp; ++gi) part += rw[gi * Dv + d];
-      a += part * wsc[w];
+      x += part * wsc[w];
     }
-    stf(out + (size_t)t * out_stride + h * Dv + d, a * inv);
+    stf(out + (size_t)t * out_stride + h * Dv + d, x * inv);
   }
 }
 
@@ -303,9 +390,8 @@ __global__ __launch_bounds__(WAVE) void masked_prefill_mfma_kernel(
     int64_t q_stride, const bf16raw* __restrict__ k_cache,
     const bf16raw* __restrict__ v_cache, const int* __restrict__ block_tables,
     int max_blocks, const int* __restrict__ start_loc,
-    const int* __restrict__ positions, int tiles_per_run, float scale,
-    float softcap, int chunk, int window, float out_scale, const float* __restrict__ sink, int64_t v_rs, int H, int G,
-    int D, int Dv, int bs, int kvs) {
+    const int* __restrict__ positions, int tiles_per_run, AttnArgs a) {
+  const int H = a.H, G = a.G, D = a.D, Dv = a.Dv, bs = a.bs;
   const int s = blockIdx.x / tiles_per_run, tile = blockIdx.x % tiles_per_run;
   const int h = blockIdx.y, g = h / (H / G);
   const int s0 = start_loc[s], s1 = start_loc[s + 1];
@@ -317,14 +403,13 @@ __global__ __launch_bounds__(WAVE) void masked_prefill_mfma_kernel(
   const int tq = q0 + min(col, nq - 1);
   const int pos_q = q_ok ? positions[tq] : -1;
   const int pos_min = positions[q0], pos_max = pos_min + nq - 1;
-  auto lower = [&](int p) {
-    int lo = 0;
-    if (chunk > 0) lo = (p / chunk) * chunk;
-    if (window > 0) lo = max(lo, p - window + 1);
-    return lo;
-  };
-  const int lo_q = q_ok ? lower(pos_q) : 0;
-  const int lo_tile = lower(pos_min);
+  const int lo_q = q_ok ? a.lower(pos_q) : 0;
+  const int lo_tile = a.lower(pos_min);
+  // key tiles: those of the kept first tokens, then from the first query's
+  // window to the last query
+  const int kept = a.kept(lo_tile), n_kept = (kept + 15) / 16;
+  const int n_tiles = n_kept + (pos_max - lo_tile) / 16 + 1;
+  const float slope = a.slopes != nullptr ? a.slopes[h] : 0.f;
   const int* bt = block_tables + (size_t)s * max_blocks;
   const int nks = D / 16, ndt = Dv / 16;
   bf16x4 qf[kMaxDSteps];
@@ -336,9 +421,11 @@ __global__ __launch_bounds__(WAVE) void masked_prefill_mfma_kernel(
 #pragma unroll
   for (int dt = 0; dt < kMaxDvTiles; ++dt) oacc[dt] = (f32x4){0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;
-  for (int j0 = lo_tile; j0 <= pos_max; j0 += 16) {
+  for (int it = 0; it < n_tiles; ++it) {
+    const int j0 = it < n_kept ? it * 16 : lo_tile + (it - n_kept) * 16;
+    const int j_end = it < n_kept ? kept - 1 : pos_max;
     // K operand: row = key j0 + col, 4 consecutive dims per step
-    const int jk = min(j0 + col, pos_max);
+    const int jk = min(j0 + col, j_end);
     const bf16raw* kp = k_cache + (((int64_t)bt[jk / bs] * G + g) * bs + jk % bs) * D + grp * 4;
     f32x4 sacc = (f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -354,13 +441,16 @@ __global__ __launch_bounds__(WAVE) void masked_prefill_mfma_kernel(
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int j = j0 + grp * 4 + i;
-      float x = sacc[i] * scale;
-      if (softcap > 0.f) x = softcap * tanhf(x / softcap);
-      vis[i] = j <= pos_q && j >= lo_q;
+      const int jv = min(j, j_end);
+      const int64_t blk = bt[jv / bs];
+      float x = sacc[i] * a.scale;
+      if (a.kscale != nullptr) x *= a.kscale[blk * bs + jv % bs];
+      if (a.softcap > 0.f) x = a.softcap * tanhf(x / a.softcap);
+      x -= slope * (float)(pos_q - j);
+      vis[i] = j <= j_end && j <= pos_q && (j >= lo_q || j < a.keep);
       sc[i] = vis[i] ? x : -INFINITY;
       mt = fmaxf(mt, sc[i]);
-      const int jv = min(j, pos_max);
-      vrow[i] = (((int64_t)bt[jv / bs] * (G / kvs) + g / kvs) * bs + jv % bs) * v_rs;
+      vrow[i] = ((blk * (G / a.kvs) + g / a.kvs) * bs + jv % bs) * a.v_rs;
     }
     mt = fmaxf(mt, __shfl_xor(mt, 16, WAVE));
     mt = fmaxf(mt, __shfl_xor(mt, 32, WAVE));
@@ -382,17 +472,17 @@ __global__ __launch_bounds__(WAVE) void masked_prefill_mfma_kernel(
         bf16x4 vf;  // V^T operand: row = value dim dt*16 + col, keys grp*4 + i
 #pragma unroll
         for (int i = 0; i < 4; ++i) vf[i] = (short)v_cache[vrow[i] + dt * 16 + col];
-        f32x4 a = oacc[dt];
-        a[0] *= corr; a[1] *= corr; a[2] *= corr; a[3] *= corr;
-        oacc[dt] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(vf, pb, a, 0, 0, 0);
+        f32x4 o = oacc[dt];
+        o[0] *= corr; o[1] *= corr; o[2] *= corr; o[3] *= corr;
+        oacc[dt] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(vf, pb, o, 0, 0, 0);
       }
     }
   }
   l += __shfl_xor(l, 16, WAVE);
   l += __shfl_xor(l, 32, WAVE);
-  if (sink != nullptr) l += expf(sink[h] - m);
+  if (a.sink != nullptr) l += expf(a.sink[h] - m);
   if (q_ok) {
-    const float inv = out_scale / l;
+    const float inv = a.out_scale / l;
     bf16raw* op = out + (size_t)tq * out_stride + h * Dv + grp * 4;
 #pragma unroll
     for (int dt = 0; dt < kMaxDvTiles; ++dt) {
@@ -408,65 +498,125 @@ __global__ __launch_bounds__(WAVE) void masked_prefill_mfma_kernel(
   }
 }
 
-constexpr float kLog2e = 1.4426950408889634f;
-
-// two fp32 -> packed bf16 pair (round to nearest even), low half first
+// two fp32 -> packed bf16 pair (round to nearest even), low half first; a
+// conversion the compiler knows, so that it keeps the wait states between an
+// exponential and its reader
+typedef __attribute__((ext_vector_type(2))) float f32x2;
+typedef __attribute__((ext_vector_type(2))) __bf16 bf16x2;
 DEV_INLINE uint32_t cvt_pk_bf16(float a, float b) {
-  uint32_t r;
-  asm volatile("v_cvt_pk_bf16_f32 %0, %1, %2" : "=v"(r) : "v"(a), "v"(b));
-  return r;
+  return __builtin_bit_cast(uint32_t, __builtin_convertvector((f32x2){a, b}, bf16x2));
 }
 
-constexpr int kKT = 32;      // keys staged per iteration
-constexpr int kKPad = 8;     // padding of a staged key row (elements)
-constexpr int kVPad = 4;     // padding of a staged transposed value row
+// max over the four lanes 16 apart that share a lane column
+DEV_INLINE float column_max(float x, int lane) {
+  auto from = [&](float v, int src) {
+    return __builtin_bit_cast(
+        float, __builtin_amdgcn_ds_bpermute(src * 4, __builtin_bit_cast(int, v)));
+  };
+  x = fmaxf(x, from(x, lane ^ 16));
+  return fmaxf(x, from(x, lane ^ 32));
+}
+
+constexpr int kKT = 32;    // keys of a tile
+constexpr int kRPad = 8;   // padding of a staged row (elements)
+
+typedef __attribute__((ext_vector_type(8))) short bf16x8;
+
+// A 16 x 16 piece of a row-major LDS tile, transposed on the way to the
+// registers: p points at (row r0 + (lane & 15) / 4 + 4 * (lane >> 4), column
+// c0 + 4 * (lane & 3)); the lane receives rows r0 + 4 * (lane >> 4) + 0..3 of
+// column c0 + (lane & 15).
+DEV_INLINE bf16x4 lds_read_transposed(const bf16raw* p) {
+  return __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+      (__attribute__((address_space(3))) bf16x4*)p);
+}
+
+// K Q^T over 16 (four slots a lane) or 32 (eight slots) key dims
+DEV_INLINE f32x4 mfma_qk(bf16x4 k, bf16x4 q, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(k, q, c, 0, 0, 0);
+}
+DEV_INLINE f32x4 mfma_qk(bf16x8 k, bf16x8 q, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, q, c, 0, 0, 0);
+}
+
+template <bool kWide> struct QkFrag {  // one lane's share of a row step
+  typedef bf16x4 type;
+  static constexpr int kDims = 16, kElems = 4;
+};
+template <> struct QkFrag<true> {
+  typedef bf16x8 type;
+  static constexpr int kDims = 32, kElems = 8;
+};
+
+// Scores of a lane's eight keys of a 32-key tile (keys sub * 16 + grp * 4 + i,
+// e = sub * 4 + i) in the base-2 domain, so that every exponential is one
+// v_exp_f32: scale and key scale, cap, bias. rel0 = (first key - query) of the
+// lane: sub 0, i 0. kcv: the tile's key scales in LDS at the lane's keys, or
+// null.
+DEV_INLINE void base2_scores(const f32x4* sacc, const AttnArgs& a, float slope2,
+                             float cap2, float rel0, const float* kcv, float* sc) {
+  const float c = cap2 > 0.f ? a.scale * (2.f * kLog2e) / a.softcap : a.scale * kLog2e;
+  if (kcv != nullptr) {
+    const float4 k0 = *(const float4*)kcv, k1 = *(const float4*)(kcv + 16);
+    sc[0] = sacc[0][0] * (c * k0.x); sc[1] = sacc[0][1] * (c * k0.y);
+    sc[2] = sacc[0][2] * (c * k0.z); sc[3] = sacc[0][3] * (c * k0.w);
+    sc[4] = sacc[1][0] * (c * k1.x); sc[5] = sacc[1][1] * (c * k1.y);
+    sc[6] = sacc[1][2] * (c * k1.z); sc[7] = sacc[1][3] * (c * k1.w);
+  } else {
+#pragma unroll
+    for (int e = 0; e < 8; ++e) sc[e] = sacc[e >> 2][e & 3] * c;
+  }
+  if (cap2 > 0.f) {
+#pragma unroll
+    for (int e = 0; e < 8; ++e) sc[e] = cap_base2(sc[e], cap2);
+  }
+  if (slope2 != 0.f) {
+    const float b = slope2 * rel0;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) sc[e] += b + slope2 * (float)((e >> 2) * 16 + (e & 3));
+  }
+}
 
 // Prompt portions on the matrix cores with the key / value tiles shared
 // through LDS. A block of HW * QW waves covers QW * 16 consecutive queries of
 // a run for HW query heads of one key/value head (for latent attention all
 // heads share the one cached row, for grouped heads the group does). Per
-// iteration the block stages 32 keys: K rows as they lie in the cache
-// (16-byte loads, padded rows) and V transposed ([value dim][key]), so both
-// MFMA operands are 8-byte LDS reads. Two LDS buffers: the next tile is loaded
-// into registers before the products of the current one and written to the
-// other buffer after them, one barrier per iteration. Masking and the fp32
-// softmax statistics are those of masked_prefill_mfma_kernel; P V contracts
-// all 32 keys of a tile in one v_mfma_f32_16x16x32_bf16 per 16 value dims (a
-// lane's eight contraction slots are keys grp*4 + 0..3 and 16 + grp*4 + 0..3,
-// for P and V alike), and so does K Q^T over 32 key dims when the key size
-// allows (kWideQK).
-typedef __attribute__((ext_vector_type(8))) short bf16x8;
-
-template <int kMaxDSteps, int kMaxDvTiles, bool kWideQK>
+// iteration the block stages 32 keys as they lie in the cache (16-byte loads,
+// padded rows): K rows are read back as MFMA operands in 8 or 16-byte pieces,
+// V rows through the transposing LDS read. kTied: the value is the leading
+// part of the key row, so one staged tile serves both. Two LDS buffers: the
+// next tile is loaded into registers before the products of the current one
+// and written to the other buffer after them, one barrier per iteration. P V
+// contracts all 32 keys of a tile in one v_mfma_f32_16x16x32_bf16 per 16 value
+// dims (a lane's eight contraction slots are keys grp*4 + 0..3 and
+// 16 + grp*4 + 0..3, for P and V alike), and so does K Q^T over 32 key dims
+// when the key size allows (kWideQK). Statistics are fp32, base 2.
+template <int kMaxDSteps, int kMaxDvTiles, bool kWideQK, bool kTied>
 __global__ __launch_bounds__(512) void masked_prefill_mfma_shared_kernel(
     bf16raw* __restrict__ out, int64_t out_stride, const bf16raw* __restrict__ q,
     int64_t q_stride, const bf16raw* __restrict__ k_cache,
     const bf16raw* __restrict__ v_cache, const int* __restrict__ block_tables,
     int max_blocks, const int* __restrict__ start_loc,
-    const int* __restrict__ positions, int tiles_per_run, float scale,
-    float softcap, int chunk, int window, float out_scale, const float* __restrict__ sink, int64_t v_rs, int H, int G,
-    int D, int Dv, int bs, int HW, int QW, int kvs) {
+    const int* __restrict__ positions, int tiles_per_run, int HW, int QW, AttnArgs a) {
   extern __shared__ __attribute__((aligned(16))) bf16raw lds[];
+  typedef QkFrag<kWideQK> Frag;
+  typedef typename Frag::type frag_t;
+  constexpr int kNF = kMaxDSteps * 16 / Frag::kDims;
   constexpr int kKVec = kKT * kMaxDSteps * 16 / 8 / 256;   // per thread, 256 threads
-  constexpr int kVVec = kKT * kMaxDvTiles * 16 / 8 / 256;
+  constexpr int kVVec = kTied ? 1 : kKT * kMaxDvTiles * 16 / 8 / 256;
+  const int G = a.G, D = a.D, Dv = a.Dv, bs = a.bs;
   const int nthr = blockDim.x;
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int col = lane & 15, grp = lane >> 4;
   const int hw = wave % HW, qw = wave / HW;
   const int s = blockIdx.x / tiles_per_run, tile = blockIdx.x % tiles_per_run;
-  const int g = blockIdx.y, rep = H / G;
+  const int g = blockIdx.y, rep = a.H / G;
   const int hz = blockIdx.z * HW + hw;
   const int s0 = start_loc[s], s1 = start_loc[s + 1];
   const int bq0 = s0 + tile * QW * 16;
   if (bq0 >= s1) return;  // the whole block: no barrier is skipped
   const int bnq = min(QW * 16, s1 - bq0);
   const int bpos_min = positions[bq0], bpos_max = bpos_min + bnq - 1;
-  auto lower = [&](int p) {
-    int lo = 0;
-    if (chunk > 0) lo = (p / chunk) * chunk;
-    if (window > 0) lo = max(lo, p - window + 1);
-    return lo;
-  };
   const int q0 = bq0 + qw * 16;
   const bool wave_on = q0 < s1 && hz < rep;
   const int nq = wave_on ? min(16, s1 - q0) : 0;
@@ -475,134 +625,144 @@ __global__ __launch_bounds__(512) void masked_prefill_mfma_shared_kernel(
   const int tq = wave_on ? q0 + min(col, nq - 1) : bq0;
   const int pos_q = q_ok ? positions[tq] : -1;
   const int wpos_min = wave_on ? positions[q0] : 0, wpos_max = wpos_min + nq - 1;
-  const int lo_q = q_ok ? lower(pos_q) : 0;
-  const int wlo = lower(wpos_min);
-  const int blo = lower(bpos_min);
+  const int lo_q = q_ok ? a.lower(pos_q) : 0;
+  const int wlo = a.lower(wpos_min), wlo_max = a.lower(max(wpos_max, 0));
+  const int blo = a.lower(bpos_min);
+  // tiles of the kept first tokens, then from the first query's window on
+  const int kept = a.kept(blo), n_kept = (kept + kKT - 1) / kKT;
+  const int n_tiles = n_kept + (bpos_max - blo) / kKT + 1;
   const int* bt = block_tables + (size_t)s * max_blocks;
-  const int nks = D / 16, ndt = Dv / 16;
-  const int krow = D + kKPad, vrow = kKT + kVPad;  // LDS row lengths (elements)
-  const int buf_elems = kKT * krow + Dv * vrow;
+  const int nf = D / Frag::kDims, ndt = Dv / 16;
+  const int krow = D + kRPad, vrow = kTied ? krow : Dv + kRPad;
+  const int k_elems = kKT * krow, v_elems = kTied ? 0 : kKT * vrow;
+  const int buf_elems = k_elems + v_elems + 2 * kKT;  // + key scales (fp32)
   const int kcpr = D / 8, vcpr = Dv / 8;  // 16-byte chunks per cached row
+  const float slope2 = a.slopes != nullptr ? a.slopes[h] * kLog2e : 0.f;
+  const float cap2 = a.softcap * kLog2e;
 
-  // query fragments: [ks] 4 dims at ks*16 + grp*4, or (wide) [kc] 8 dims at
-  // kc*32 + grp*8
-  bf16x4 qf[kWideQK ? 1 : kMaxDSteps];
-  bf16x8 qf8[kWideQK ? kMaxDSteps / 2 : 1];
+  frag_t qf[kNF];
   const bf16raw* qrow = q + (size_t)tq * q_stride + h * D;
-  if (kWideQK) {
 #pragma unroll
-    for (int kc = 0; kc < kMaxDSteps / 2; ++kc)
-      if (kc < D / 32) {
-        const bf16x4 a = *(const bf16x4*)(qrow + kc * 32 + grp * 8);
-        const bf16x4 b = *(const bf16x4*)(qrow + kc * 32 + grp * 8 + 4);
-        qf8[kc] = (bf16x8){a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+  for (int f = 0; f < kNF; ++f)
+    if (f < nf) {
+      const bf16raw* p = qrow + f * Frag::kDims + grp * Frag::kElems;
+      if constexpr (kWideQK) {
+        const bf16x4 x = *(const bf16x4*)p, y = *(const bf16x4*)(p + 4);
+        qf[f] = (bf16x8){x[0], x[1], x[2], x[3], y[0], y[1], y[2], y[3]};
+      } else {
+        qf[f] = *(const bf16x4*)p;
       }
-  } else {
-#pragma unroll
-    for (int ks = 0; ks < kMaxDSteps; ++ks)
-      if (ks < nks) qf[ks] = *(const bf16x4*)(qrow + ks * 16 + grp * 4);
-  }
+    }
   f32x4 oacc[kMaxDvTiles];
 #pragma unroll
   for (int dt = 0; dt < kMaxDvTiles; ++dt) oacc[dt] = (f32x4){0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;
 
   uint4 kreg[kKVec], vreg[kVVec];
-  // K: consecutive threads take consecutive chunks of a row (coalesced);
-  // V: consecutive threads take consecutive keys at one chunk, so that the
-  // transposed 2-byte LDS writes of a wave fall into consecutive addresses
-  auto load_tile = [&](int j0) {
+  float kscr = 0.f;
+  auto first_key = [&](int it) {
+    return it < n_kept ? it * kKT : blo + (it - n_kept) * kKT;
+  };
+  auto last_key = [&](int it) { return it < n_kept ? kept - 1 : bpos_max; };
+  auto load_tile = [&](int it) {
+    const int j0 = first_key(it), j_end = last_key(it);
 #pragma unroll
     for (int i = 0; i < kKVec; ++i) {
       const int v = i * nthr + threadIdx.x;
       const int row = v / kcpr, c = v % kcpr;
       if (row < kKT) {
-        const int j = min(j0 + row, bpos_max);
+        const int j = min(j0 + row, j_end);
         kreg[i] = *(const uint4*)(k_cache +
             (((int64_t)bt[j / bs] * G + g) * bs + j % bs) * D + c * 8);
       }
     }
+    if constexpr (!kTied) {
 #pragma unroll
-    for (int i = 0; i < kVVec; ++i) {
-      const int v = i * nthr + threadIdx.x;
-      const int row = v % kKT, c = v / kKT;
-      if (c < vcpr) {
-        const int j = min(j0 + row, bpos_max);
-        vreg[i] = *(const uint4*)(v_cache +
-            (((int64_t)bt[j / bs] * (G / kvs) + g / kvs) * bs + j % bs) * v_rs + c * 8);
+      for (int i = 0; i < kVVec; ++i) {
+        const int v = i * nthr + threadIdx.x;
+        const int row = v / vcpr, c = v % vcpr;
+        if (row < kKT) {
+          const int j = min(j0 + row, j_end);
+          vreg[i] = *(const uint4*)(v_cache +
+              (((int64_t)bt[j / bs] * (G / a.kvs) + g / a.kvs) * bs + j % bs) * a.v_rs +
+              c * 8);
+        }
       }
+    }
+    if (a.kscale != nullptr && threadIdx.x < kKT) {
+      const int j = min(j0 + (int)threadIdx.x, j_end);
+      kscr = a.kscale[(int64_t)bt[j / bs] * bs + j % bs];
     }
   };
   auto store_tile = [&](int buf) {
     bf16raw* ks_ = lds + buf * buf_elems;
-    bf16raw* vs_ = ks_ + kKT * krow;
 #pragma unroll
     for (int i = 0; i < kKVec; ++i) {
       const int v = i * nthr + threadIdx.x;
       const int row = v / kcpr, c = v % kcpr;
       if (row < kKT) *(uint4*)(ks_ + row * krow + c * 8) = kreg[i];
     }
+    if constexpr (!kTied) {
+      bf16raw* vs_ = ks_ + k_elems;
 #pragma unroll
-    for (int i = 0; i < kVVec; ++i) {
-      const int v = i * nthr + threadIdx.x;
-      const int row = v % kKT, c = v / kKT;
-      if (c < vcpr) {
-        const uint32_t wv[4] = {vreg[i].x, vreg[i].y, vreg[i].z, vreg[i].w};
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          vs_[(c * 8 + 2 * e) * vrow + row] = (bf16raw)(wv[e] & 0xffffu);
-          vs_[(c * 8 + 2 * e + 1) * vrow + row] = (bf16raw)(wv[e] >> 16);
-        }
+      for (int i = 0; i < kVVec; ++i) {
+        const int v = i * nthr + threadIdx.x;
+        const int row = v / vcpr, c = v % vcpr;
+        if (row < kKT) *(uint4*)(vs_ + row * vrow + c * 8) = vreg[i];
       }
     }
+    if (a.kscale != nullptr && threadIdx.x < kKT)
+      ((float*)(ks_ + k_elems + v_elems))[threadIdx.x] = kscr;
   };
 
-  load_tile(blo);
+  load_tile(0);
   store_tile(0);
   __syncthreads();
   int buf = 0;
-  for (int j0 = blo; j0 <= bpos_max; j0 += kKT, buf ^= 1) {
-    const bool more = j0 + kKT <= bpos_max;
-    if (more) load_tile(j0 + kKT);
+  for (int it = 0; it < n_tiles; ++it, buf ^= 1) {
+    const bool more = it + 1 < n_tiles;
+    if (more) load_tile(it + 1);
+    const int j0 = first_key(it);
     const bf16raw* ks_ = lds + buf * buf_elems;
-    const bf16raw* vs_ = ks_ + kKT * krow;
+    const bf16raw* vs_ = ks_ + (kTied ? 0 : k_elems);
+    const float* kc_ = (const float*)(ks_ + k_elems + v_elems);
     // wave-uniform: something of this tile is visible to the wave's queries
-    if (wave_on && j0 <= wpos_max && j0 + kKT - 1 >= wlo) {
+    if (wave_on && j0 <= wpos_max && (j0 + kKT - 1 >= wlo || j0 < a.keep)) {
       f32x4 sacc[2];
 #pragma unroll
       for (int sub = 0; sub < 2; ++sub) {
         sacc[sub] = (f32x4){0.f, 0.f, 0.f, 0.f};
-        const bf16raw* kp = ks_ + (sub * 16 + col) * krow;
-        if (kWideQK) {
+        const bf16raw* kp = ks_ + (sub * 16 + col) * krow + grp * Frag::kElems;
 #pragma unroll
-          for (int kc = 0; kc < kMaxDSteps / 2; ++kc)
-            if (kc < D / 32)
-              sacc[sub] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                  *(const bf16x8*)(kp + kc * 32 + grp * 8), qf8[kc], sacc[sub], 0, 0, 0);
-        } else {
+        for (int f = 0; f < kNF; ++f)
+          if (f < nf)
+            sacc[sub] = mfma_qk(*(const frag_t*)(kp + f * Frag::kDims), qf[f], sacc[sub]);
+      }
+      // this lane: query `col`, keys j0 + sub * 16 + grp * 4 + i
+      float sc[8];
+      base2_scores(sacc, a, slope2, cap2, (float)(j0 + grp * 4 - pos_q),
+                   a.kscale != nullptr ? kc_ + grp * 4 : nullptr, sc);
+      // wave-uniform: a tile whose keys all queries see needs no mask. (Masks
+      // are selects: hipcc 7.2 has lost such an assignment from under a branch.)
+      const int jl = j0 + grp * 4;
+      if (it < n_kept) {
+        if (j0 + kKT > kept) {
 #pragma unroll
-          for (int ks = 0; ks < kMaxDSteps; ++ks)
-            if (ks < nks)
-              sacc[sub] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(
-                  *(const bf16x4*)(kp + ks * 16 + grp * 4), qf[ks], sacc[sub], 0, 0, 0);
+          for (int e = 0; e < 8; ++e)
+            sc[e] = jl + (e >> 2) * 16 + (e & 3) < kept ? sc[e] : -INFINITY;
+        }
+      } else if (nq < 16 || j0 + kKT - 1 > wpos_min || j0 < wlo_max) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          const int j = jl + (e >> 2) * 16 + (e & 3);
+          const bool vis = (j <= pos_q) & ((j >= lo_q) | (j < a.keep));
+          sc[e] = vis ? sc[e] : -INFINITY;
         }
       }
-      // this lane: query `col`, keys j0 + sub * 16 + grp * 4 + i. Scores and
-      // the running max are kept in the base-2 domain (score * log2 e), so
-      // every exponential is one v_exp_f32.
-      float sc[8];
-      float mt = -INFINITY;
+      float mt = sc[0];
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        const int j = j0 + (e >> 2) * 16 + grp * 4 + (e & 3);
-        float x = sacc[e >> 2][e & 3] * scale;
-        if (softcap > 0.f) x = softcap * tanhf(x / softcap);
-        const bool vis = j <= pos_q && j >= lo_q;
-        sc[e] = vis ? x * kLog2e : -INFINITY;
-        mt = fmaxf(mt, sc[e]);
-      }
-      mt = fmaxf(mt, __shfl_xor(mt, 16, WAVE));
-      mt = fmaxf(mt, __shfl_xor(mt, 32, WAVE));
+      for (int e = 1; e < 8; ++e) mt = fmaxf(mt, sc[e]);
+      mt = column_max(mt, lane);
       const float m_new = fmaxf(m, mt);
       // no visible key so far: keep everything at zero without forming inf - inf
       const float m_use = m_new == -INFINITY ? 0.f : m_new;
@@ -620,16 +780,16 @@ __global__ __launch_bounds__(512) void masked_prefill_mfma_shared_kernel(
       const bf16x8 pb = pk.v;
       l = l * corr + ps;
       m = m_new;
-      const bf16raw* vp = vs_ + col * vrow + grp * 4;
+      const bf16raw* vp = vs_ + (grp * 4 + (col >> 2)) * vrow + (col & 3) * 4;
 #pragma unroll
       for (int dt = 0; dt < kMaxDvTiles; ++dt) {
         if (dt < ndt) {
-          const bf16x4 v0 = *(const bf16x4*)(vp + dt * 16 * vrow);
-          const bf16x4 v1 = *(const bf16x4*)(vp + dt * 16 * vrow + 16);
+          const bf16x4 v0 = lds_read_transposed(vp + dt * 16);
+          const bf16x4 v1 = lds_read_transposed(vp + dt * 16 + 16 * vrow);
           const bf16x8 vf = (bf16x8){v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
-          f32x4 a = oacc[dt];
-          a[0] *= corr; a[1] *= corr; a[2] *= corr; a[3] *= corr;
-          oacc[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pb, a, 0, 0, 0);
+          f32x4 o = oacc[dt];
+          o[0] *= corr; o[1] *= corr; o[2] *= corr; o[3] *= corr;
+          oacc[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pb, o, 0, 0, 0);
         }
       }
     }
@@ -638,9 +798,9 @@ __global__ __launch_bounds__(512) void masked_prefill_mfma_shared_kernel(
   }
   l += __shfl_xor(l, 16, WAVE);
   l += __shfl_xor(l, 32, WAVE);
-  if (sink != nullptr) l += __builtin_amdgcn_exp2f(sink[h] * kLog2e - m);
+  if (a.sink != nullptr) l += __builtin_amdgcn_exp2f(a.sink[h] * kLog2e - m);
   if (q_ok) {
-    const float inv = out_scale / l;
+    const float inv = a.out_scale / l;
     bf16raw* op = out + (size_t)tq * out_stride + h * Dv + grp * 4;
 #pragma unroll
     for (int dt = 0; dt < kMaxDvTiles; ++dt) {
@@ -658,23 +818,35 @@ __global__ __launch_bounds__(512) void masked_prefill_mfma_shared_kernel(
 
 constexpr int kDW = 4;  // waves of a decode block; each takes every fourth key tile
 
-// Single decode tokens on the matrix cores, bf16. grid (T, G, ceil(rep / 16)):
-// the 16 rows of an MFMA tile are the query heads that share one key/value
-// head (all heads of a latent layer, the group of a grouped layer), so a key
-// or value row is loaded once for all of them. The four waves walk disjoint
-// 32-key tiles: K rows come straight from the cache as A operands, the V tile
-// is transposed through a wave-private LDS region, statistics are fp32 in the
-// base-2 domain, and the waves' partial results are joined through LDS.
-template <int kMaxDSteps, int kMaxDvTiles>
+// bytes of a decode wave's staging region: a 32-row value tile + key scales
+static inline __host__ __device__ int decode_stage_bytes(int Dv) {
+  return kKT * (Dv + kRPad) * (int)sizeof(bf16raw) + kKT * (int)sizeof(float);
+}
+
+// Single decode tokens on the matrix cores, bf16. grid (T, G, ceil(rep / 16) *
+// splits): the 16 rows of an MFMA tile are the query heads that share one
+// key/value head (all heads of a latent layer, the group of a grouped layer),
+// so a key or value row is loaded once for all of them. The visible keys are
+// numbered through (kept first tokens, then the window) and cut into 32-key
+// tiles; the four waves walk disjoint tiles. A lane loads its pieces of two
+// rows per tile straight as MFMA operands, one tile ahead; the value part
+// (kTied: the same registers) is written to a wave-private LDS tile and comes
+// back through the transposing LDS read. Statistics are fp32 in the base-2
+// domain, and the waves' partial results are joined through LDS.
+template <int kMaxDSteps, int kMaxDvTiles, bool kWide, bool kTied>
 __global__ __launch_bounds__(kDW * WAVE) void masked_decode_mfma_kernel(
     bf16raw* __restrict__ out, int64_t out_stride, const bf16raw* __restrict__ q,
     int64_t q_stride, const bf16raw* __restrict__ k_cache,
     const bf16raw* __restrict__ v_cache, const int* __restrict__ block_tables,
     int max_blocks, const int* __restrict__ token_seq,
-    const int* __restrict__ positions, float scale, float softcap, int chunk,
-    int window, float out_scale, const float* __restrict__ sink, int64_t v_rs, int H, int G, int D, int Dv, int bs,
-    int n_split, float* __restrict__ part_o, float* __restrict__ part_ml, int kvs) {
+    const int* __restrict__ positions, int n_split, float* __restrict__ part_o,
+    float* __restrict__ part_ml, AttnArgs a) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
+  typedef QkFrag<kWide> Frag;
+  typedef typename Frag::type frag_t;
+  constexpr int kNF = kMaxDSteps * 16 / Frag::kDims;
+  constexpr int kNV = kMaxDvTiles * 16 / Frag::kDims;
+  const int H = a.H, G = a.G, D = a.D, Dv = a.Dv, bs = a.bs;
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int col = lane & 15, grp = lane >> 4;
   const int t = blockIdx.x, g = blockIdx.y, rep = H / G;
@@ -683,68 +855,117 @@ __global__ __launch_bounds__(kDW * WAVE) void masked_decode_mfma_kernel(
   const int nh = min(16, (g + 1) * rep - h0);
   const int pos = positions[t];
   const int* bt = block_tables + (size_t)token_seq[t] * max_blocks;
-  int lo = 0;
-  if (chunk > 0) lo = (pos / chunk) * chunk;
-  if (window > 0) lo = max(lo, pos - window + 1);
-  const int nks = D / 16, ndt = Dv / 16;
-  constexpr int vrow = kKT + kVPad;
-  bf16raw* vt = (bf16raw*)smem + (size_t)wave * Dv * vrow;
-  bf16x4 qf[kMaxDSteps];
+  const int lo = a.lower(pos), kept = a.kept(lo), n_keys = kept + pos - lo + 1;
+  const int nf = D / Frag::kDims, nv = Dv / Frag::kDims, ndt = Dv / 16;
+  const int vrow = Dv + kRPad;
+  bf16raw* vt = (bf16raw*)(smem + (size_t)wave * decode_stage_bytes(Dv));
+  float* kc = (float*)(vt + kKT * vrow);
+  const int hq = h0 + min(col, nh - 1);
+  const float slope2 = a.slopes != nullptr ? a.slopes[hq] * kLog2e : 0.f;
+  const float cap2 = a.softcap * kLog2e;
+  frag_t qf[kNF];
 #pragma unroll
-  for (int ks = 0; ks < kMaxDSteps; ++ks)
-    if (ks < nks)
-      qf[ks] = col < nh ? *(const bf16x4*)(q + (size_t)t * q_stride + (h0 + col) * D +
-                                           ks * 16 + grp * 4)
-                        : (bf16x4){0, 0, 0, 0};
+  for (int f = 0; f < kNF; ++f)
+    if (f < nf) {
+      const bf16raw* p =
+          q + (size_t)t * q_stride + (size_t)hq * D + f * Frag::kDims + grp * Frag::kElems;
+      if constexpr (kWide) {
+        const bf16x4 x = *(const bf16x4*)p, y = *(const bf16x4*)(p + 4);
+        qf[f] = (bf16x8){x[0], x[1], x[2], x[3], y[0], y[1], y[2], y[3]};
+      } else {
+        qf[f] = *(const bf16x4*)p;
+      }
+    }
   f32x4 oacc[kMaxDvTiles];
 #pragma unroll
   for (int dt = 0; dt < kMaxDvTiles; ++dt) oacc[dt] = (f32x4){0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;
-  // the visible keys in 32-key tiles, dealt to the splits in contiguous shares
-  const int n_tiles = (pos - lo) / kKT + 1;
+  // the tiles dealt to the splits in contiguous shares
+  const int n_tiles = (n_keys + kKT - 1) / kKT;
   const int per_split = (n_tiles + n_split - 1) / n_split;
   const int tile_end = min(n_tiles, (sp + 1) * per_split);
-  for (int tile = sp * per_split + wave; tile < tile_end; tile += kDW) {
-    const int j0 = lo + tile * kKT;
-    // V tile, transposed: lane takes key (v % 32), 16-byte chunk (v / 32)
-    for (int v = lane; v < kKT * (Dv / 8); v += WAVE) {
-      const int row = v % kKT, c = v / kKT;
-      const int j = min(j0 + row, pos);
-      const uint4 x = *(const uint4*)(v_cache +
-          (((int64_t)bt[j / bs] * (G / kvs) + g / kvs) * bs + j % bs) * v_rs + c * 8);
-      const uint32_t wv[4] = {x.x, x.y, x.z, x.w};
+  int jn[2], bn[2];  // the lane's two keys of the tile to load, and their blocks
+  frag_t kf[2][kNF], vf[2][kTied ? 1 : kNV];
+  float ksr[2] = {0.f, 0.f};
+  auto find_rows = [&](int tile) {
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        vt[(c * 8 + 2 * e) * vrow + row] = (bf16raw)(wv[e] & 0xffffu);
-        vt[(c * 8 + 2 * e + 1) * vrow + row] = (bf16raw)(wv[e] >> 16);
-      }
+    for (int sub = 0; sub < 2; ++sub) {
+      const int v = min(tile * kKT + sub * 16 + col, n_keys - 1);
+      jn[sub] = v < kept ? v : lo + v - kept;
+      bn[sub] = bt[jn[sub] / bs];
     }
+  };
+  auto load_rows = [&]() {
+#pragma unroll
+    for (int sub = 0; sub < 2; ++sub) {
+      const int off = jn[sub] % bs;
+      const bf16raw* kp =
+          k_cache + (((int64_t)bn[sub] * G + g) * bs + off) * D + grp * Frag::kElems;
+#pragma unroll
+      for (int f = 0; f < kNF; ++f)
+        if (f < nf) kf[sub][f] = *(const frag_t*)(kp + f * Frag::kDims);
+      if constexpr (!kTied) {
+        const bf16raw* vp = v_cache +
+            (((int64_t)bn[sub] * (G / a.kvs) + g / a.kvs) * bs + off) * a.v_rs +
+            grp * Frag::kElems;
+#pragma unroll
+        for (int f = 0; f < kNV; ++f)
+          if (f < nv) vf[sub][f] = *(const frag_t*)(vp + f * Frag::kDims);
+      }
+      if (a.kscale != nullptr) ksr[sub] = a.kscale[(int64_t)bn[sub] * bs + off];
+    }
+  };
+  int tile = sp * per_split + wave;
+  if (tile < tile_end) {
+    find_rows(tile);
+    load_rows();
+    if (tile + kDW < tile_end) find_rows(tile + kDW);
+  }
+  for (; tile < tile_end; tile += kDW) {
     f32x4 sacc[2];
 #pragma unroll
     for (int sub = 0; sub < 2; ++sub) {
+      bf16raw* vw = vt + (sub * 16 + col) * vrow + grp * Frag::kElems;
+#pragma unroll
+      for (int f = 0; f < kNV; ++f)
+        if (f < nv) *(frag_t*)(vw + f * Frag::kDims) = kTied ? kf[sub][f] : vf[sub][kTied ? 0 : f];
+      if (a.kscale != nullptr && grp == 0) kc[sub * 16 + col] = ksr[sub];
       sacc[sub] = (f32x4){0.f, 0.f, 0.f, 0.f};
-      const int jk = min(j0 + sub * 16 + col, pos);
-      const bf16raw* kp =
-          k_cache + (((int64_t)bt[jk / bs] * G + g) * bs + jk % bs) * D + grp * 4;
 #pragma unroll
-      for (int ks = 0; ks < kMaxDSteps; ++ks)
-        if (ks < nks)
-          sacc[sub] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(
-              *(const bf16x4*)(kp + ks * 16), qf[ks], sacc[sub], 0, 0, 0);
+      for (int f = 0; f < kNF; ++f)
+        if (f < nf) sacc[sub] = mfma_qk(kf[sub][f], qf[f], sacc[sub]);
     }
-    // this lane: head `col`, keys j0 + sub * 16 + grp * 4 + i
+    if (tile + kDW < tile_end) {
+      load_rows();
+      if (tile + 2 * kDW < tile_end) find_rows(tile + 2 * kDW);
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    // this lane: head `col`, keys v0 + sub * 16 + grp * 4 + i of the numbering
+    const int v0 = tile * kKT;
     float sc[8];
-    float mt = -INFINITY;
+    if (v0 >= kept || v0 + kKT <= kept) {  // one stretch of positions
+      const int j0 = v0 < kept ? v0 : lo + v0 - kept;
+      base2_scores(sacc, a, slope2, cap2, (float)(j0 + grp * 4 - pos),
+                   a.kscale != nullptr ? kc + grp * 4 : nullptr, sc);
+    } else {
+      base2_scores(sacc, a, 0.f, cap2, 0.f,
+                   a.kscale != nullptr ? kc + grp * 4 : nullptr, sc);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      const int j = j0 + (e >> 2) * 16 + grp * 4 + (e & 3);
-      float x = sacc[e >> 2][e & 3] * scale;
-      if (softcap > 0.f) x = softcap * tanhf(x / softcap);
-      sc[e] = j <= pos ? x * kLog2e : -INFINITY;  // j >= lo holds for every tile
-      mt = fmaxf(mt, sc[e]);
+      for (int e = 0; e < 8; ++e) {
+        const int v = v0 + (e >> 2) * 16 + grp * 4 + (e & 3);
+        sc[e] += slope2 * (float)((v < kept ? v : lo + v - kept) - pos);
+      }
     }
-    mt = fmaxf(mt, __shfl_xor(mt, 16, WAVE));
-    mt = fmaxf(mt, __shfl_xor(mt, 32, WAVE));
+    if (v0 + kKT > n_keys) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e)
+        sc[e] = v0 + (e >> 2) * 16 + grp * 4 + (e & 3) < n_keys ? sc[e] : -INFINITY;
+    }
+    float mt = sc[0];
+#pragma unroll
+    for (int e = 1; e < 8; ++e) mt = fmaxf(mt, sc[e]);
+    mt = column_max(mt, lane);
     const float m_new = fmaxf(m, mt);  // finite: the tile's first key is visible
     const float corr = __builtin_amdgcn_exp2f(m - m_new);
     float pv[8];
@@ -759,21 +980,22 @@ __global__ __launch_bounds__(kDW * WAVE) void masked_decode_mfma_kernel(
     for (int e = 0; e < 4; ++e) pk.u[e] = cvt_pk_bf16(pv[2 * e], pv[2 * e + 1]);
     l = l * corr + ps;
     m = m_new;
-    __builtin_amdgcn_s_waitcnt(0xc07f);  // lgkmcnt(0): the wave's LDS writes landed
-    __builtin_amdgcn_wave_barrier();
-    const bf16raw* vp = vt + col * vrow + grp * 4;
+    const bf16raw* vp = vt + (grp * 4 + (col >> 2)) * vrow + (col & 3) * 4;
 #pragma unroll
     for (int dt = 0; dt < kMaxDvTiles; ++dt) {
       if (dt < ndt) {
-        const bf16x4 v0 = *(const bf16x4*)(vp + dt * 16 * vrow);
-        const bf16x4 v1 = *(const bf16x4*)(vp + dt * 16 * vrow + 16);
-        const bf16x8 vf = (bf16x8){v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
-        f32x4 a = oacc[dt];
-        a[0] *= corr; a[1] *= corr; a[2] *= corr; a[3] *= corr;
-        oacc[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pk.v, a, 0, 0, 0);
+        const bf16x4 v0t = lds_read_transposed(vp + dt * 16);
+        const bf16x4 v1t = lds_read_transposed(vp + dt * 16 + 16 * vrow);
+        const bf16x8 vfr = (bf16x8){v0t[0], v0t[1], v0t[2], v0t[3],
+                                    v1t[0], v1t[1], v1t[2], v1t[3]};
+        f32x4 o = oacc[dt];
+        o[0] *= corr; o[1] *= corr; o[2] *= corr; o[3] *= corr;
+        oacc[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vfr, pk.v, o, 0, 0, 0);
       }
     }
-    __builtin_amdgcn_wave_barrier();  // all lanes read the tile before it is rewritten
+    // all lanes read the tile before it is rewritten
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
   }
   l += __shfl_xor(l, 16, WAVE);
   l += __shfl_xor(l, 32, WAVE);
@@ -787,30 +1009,27 @@ __global__ __launch_bounds__(kDW * WAVE) void masked_decode_mfma_kernel(
   }
 #pragma unroll
   for (int dt = 0; dt < kMaxDvTiles; ++dt)
-    if (dt < ndt) {
-#pragma unroll
-      for (int i = 0; i < 4; ++i)
-        co[((size_t)wave * 16 + col) * Dv + dt * 16 + grp * 4 + i] = oacc[dt][i];
-    }
+    if (dt < ndt)
+      *(f32x4*)(co + ((size_t)wave * 16 + col) * Dv + dt * 16 + grp * 4) = oacc[dt];
   __syncthreads();
   for (int idx = threadIdx.x; idx < nh * Dv; idx += blockDim.x) {
     const int hh = idx / Dv, d = idx % Dv;
     float mx = -INFINITY;
     for (int w = 0; w < kDW; ++w) mx = fmaxf(mx, cm[w * 16 + hh]);
-    float lsum = 0.f, a = 0.f;
+    float lsum = 0.f, x = 0.f;
     for (int w = 0; w < kDW; ++w) {
       const float mw = cm[w * 16 + hh];
       const float wsc = mw == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(mw - mx);
       lsum += cl[w * 16 + hh] * wsc;
-      a += co[((size_t)w * 16 + hh) * Dv + d] * wsc;
+      x += co[((size_t)w * 16 + hh) * Dv + d] * wsc;
     }
     if (n_split == 1) {
-      if (sink != nullptr) lsum += __builtin_amdgcn_exp2f(sink[h0 + hh] * kLog2e - mx);
-      stf(out + (size_t)t * out_stride + (h0 + hh) * Dv + d, a * out_scale / lsum);
+      if (a.sink != nullptr) lsum += __builtin_amdgcn_exp2f(a.sink[h0 + hh] * kLog2e - mx);
+      stf(out + (size_t)t * out_stride + (h0 + hh) * Dv + d, x * a.out_scale / lsum);
     } else {
       // partial result of this split: [t][head][split] -> (max, sum), values
       const size_t row = ((size_t)t * H + h0 + hh) * n_split + sp;
-      part_o[row * Dv + d] = a;
+      part_o[row * Dv + d] = x;
       if (d == 0) {
         part_ml[row * 2] = mx;
         part_ml[row * 2 + 1] = lsum;
@@ -935,13 +1154,51 @@ void qknorm_rope_half_and_cache(torch::Tensor q, torch::Tensor k, torch::Tensor 
   SEQ_CHECK_LAUNCH();
 }
 
+void qnorm_rows_to_cache(torch::Tensor q, torch::Tensor k, torch::Tensor q_weight,
+                         double eps, torch::Tensor cache, torch::Tensor key_scale,
+                         torch::Tensor slot_mapping) {
+  check_f32(q_weight, "q_weight");
+  check_f32(key_scale, "key_scale");
+  TORCH_CHECK(q.dim() == 3 && k.dim() == 3 && dense_heads3(q) && dense_heads3(k));
+  TORCH_CHECK(slot_mapping.scalar_type() == torch::kInt64 &&
+              slot_mapping.is_contiguous() && slot_mapping.is_cuda());
+  const int T = q.size(0), H = q.size(1), D = q.size(2), G = k.size(1);
+  TORCH_CHECK(k.size(0) == T && k.size(2) == D && slot_mapping.numel() == T &&
+              q_weight.numel() == (int64_t)H * D);
+  TORCH_CHECK(cache.is_cuda() && cache.is_contiguous() && cache.dim() == 4 &&
+              cache.size(1) == G && cache.size(3) == D &&
+              key_scale.numel() == cache.size(0) * cache.size(2));
+  TORCH_CHECK(k.scalar_type() == q.scalar_type() && cache.scalar_type() == q.scalar_type());
+  if (T == 0) return;
+  const int n = 16 / q.element_size();
+  auto al = [&](const torch::Tensor& x) {
+    return ((size_t)x.data_ptr()) % 16 == 0 && x.stride(0) % n == 0;
+  };
+  const bool vec = D % n == 0 && al(q) && al(k) && ((size_t)cache.data_ptr()) % 16 == 0;
+  SEQ_DISPATCH_ACT(q, {
+    auto launch = [&](auto kern) {
+      hipLaunchKernelGGL(kern, dim3(T), dim3(256), 0, SEQ_STREAM(), (act_t*)q.data_ptr(),
+                         q.stride(0), (const act_t*)k.data_ptr(), k.stride(0),
+                         (const float*)q_weight.data_ptr(), (float)eps,
+                         (act_t*)cache.data_ptr(), (float*)key_scale.data_ptr(),
+                         (const int64_t*)slot_mapping.data_ptr(), H, G, D,
+                         (int)cache.size(2));
+    };
+    if (vec) launch(qnorm_rows_cache_kernel<act_t, true>);
+    else launch(qnorm_rows_cache_kernel<act_t, false>);
+  });
+  SEQ_CHECK_LAUNCH();
+}
+
 void masked_paged_attention(torch::Tensor out, torch::Tensor q,
                             torch::Tensor k_cache, torch::Tensor v_cache,
                             torch::Tensor block_tables, torch::Tensor start_loc,
                             torch::Tensor token_seq, torch::Tensor positions,
                             int64_t max_len, double scale, double softcap,
                             int64_t chunk, int64_t window, double out_scale,
-                            c10::optional<torch::Tensor> sink_scores) {
+                            c10::optional<torch::Tensor> sink_scores,
+                            int64_t keep_first, c10::optional<torch::Tensor> slopes,
+                            c10::optional<torch::Tensor> key_scale) {
   check_i32(start_loc, "start_loc");
   check_i32(block_tables, "block_tables");
   check_i32(token_seq, "token_seq");
@@ -962,12 +1219,35 @@ void masked_paged_attention(torch::Tensor out, torch::Tensor q,
               v_cache.stride(1) == (int64_t)bs * v_rs &&
               v_cache.stride(0) == (int64_t)Gv * bs * v_rs,
               "value cache rows must be evenly spaced");
-  const float* sink = nullptr;
+  AttnArgs args{};
   if (sink_scores.has_value()) {
     check_f32(*sink_scores, "sink_scores");
     TORCH_CHECK(sink_scores->numel() == H, "one sink score per head");
-    sink = (const float*)sink_scores->data_ptr();
+    args.sink = (const float*)sink_scores->data_ptr();
   }
+  if (slopes.has_value()) {
+    check_f32(*slopes, "slopes");
+    TORCH_CHECK(slopes->numel() == H, "one slope per head");
+    args.slopes = (const float*)slopes->data_ptr();
+  }
+  if (key_scale.has_value()) {
+    check_f32(*key_scale, "key_scale");
+    TORCH_CHECK(key_scale->numel() == k_cache.size(0) * bs, "one scale per cached key");
+    args.kscale = (const float*)key_scale->data_ptr();
+  }
+  TORCH_CHECK(keep_first >= 0 && (keep_first == 0 || (chunk == 0 && window > 0)),
+              "kept first tokens belong to a window");
+  args.scale = (float)scale;
+  args.softcap = (float)softcap;
+  args.out_scale = (float)out_scale;
+  args.chunk = (int)chunk;
+  args.window = (int)window;
+  args.keep = (int)keep_first;
+  args.v_rs = v_rs;
+  args.H = H; args.G = G; args.D = D; args.Dv = Dv; args.bs = bs; args.kvs = kvs;
+  // one row per token and head that is key and (its leading part) value
+  const bool tied = v_cache.data_ptr() == k_cache.data_ptr() && kvs == 1 && v_rs == D &&
+                    Dv <= D;
   TORCH_CHECK(G > 0 && H % G == 0 && H <= 65535);
   TORCH_CHECK(out.size(0) == T && out.size(1) == H && out.size(2) == Dv);
   TORCH_CHECK(Dv <= kMaxDvPerLane * WAVE, "value size too large");
@@ -994,12 +1274,11 @@ void masked_paged_attention(torch::Tensor out, torch::Tensor q,
                          (const bf16raw*)v_cache.data_ptr(),
                          (const int*)block_tables.data_ptr(),
                          (int)block_tables.size(1), (const int*)start_loc.data_ptr(),
-                         (const int*)positions.data_ptr(), tiles, (float)scale,
-                         (float)softcap, (int)chunk, (int)window, (float)out_scale,
-                         sink, v_rs, H, G, D, Dv, bs, kvs);
+                         (const int*)positions.data_ptr(), tiles, args);
     };
     const size_t lds_shared =
-        (size_t)2 * (kKT * (D + kKPad) + Dv * (kKT + kVPad)) * sizeof(bf16raw);
+        (size_t)2 * (kKT * (D + kRPad) + (tied ? 0 : kKT * (Dv + kRPad)) + 2 * kKT) *
+        sizeof(bf16raw);
     const bool cache_al16 = ((size_t)k_cache.data_ptr()) % 16 == 0 &&
                             ((size_t)v_cache.data_ptr()) % 16 == 0;
     if (D <= 256 && Dv <= 256 && lds_shared <= 64 * 1024 && cache_al16) {
@@ -1022,18 +1301,21 @@ void masked_paged_attention(torch::Tensor out, torch::Tensor q,
                          (const bf16raw*)v_cache.data_ptr(),
                          (const int*)block_tables.data_ptr(),
                          (int)block_tables.size(1), (const int*)start_loc.data_ptr(),
-                         (const int*)positions.data_ptr(), btiles, (float)scale,
-                         (float)softcap, (int)chunk, (int)window, (float)out_scale,
-                         sink, v_rs, H, G, D, Dv, bs, HW, QW, kvs);
+                         (const int*)positions.data_ptr(), btiles, HW, QW, args);
       };
       // key sizes above 128 (a latent with a rotated part behind it) keep
       // twice as many query fragments in registers
-      if (D <= 128) {
-        if (D % 32 == 0) launch_shared(masked_prefill_mfma_shared_kernel<8, 16, true>);
-        else launch_shared(masked_prefill_mfma_shared_kernel<8, 16, false>);
+      auto pick = [&](auto wide, auto is_tied) {
+        constexpr bool kW = decltype(wide)::value, kT = decltype(is_tied)::value;
+        if (D <= 128) launch_shared(masked_prefill_mfma_shared_kernel<8, kT ? 8 : 16, kW, kT>);
+        else launch_shared(masked_prefill_mfma_shared_kernel<16, 16, kW, kT>);
+      };
+      if (D % 32 == 0) {
+        if (tied) pick(std::true_type{}, std::true_type{});
+        else pick(std::true_type{}, std::false_type{});
       } else {
-        if (D % 32 == 0) launch_shared(masked_prefill_mfma_shared_kernel<16, 16, true>);
-        else launch_shared(masked_prefill_mfma_shared_kernel<16, 16, false>);
+        if (tied) pick(std::false_type{}, std::true_type{});
+        else pick(std::false_type{}, std::false_type{});
       }
     } else if (D <= 128 && Dv <= 256) {
       launch(masked_prefill_mfma_kernel<8, 16>);
@@ -1052,12 +1334,14 @@ void masked_paged_attention(torch::Tensor out, torch::Tensor q,
       ((size_t)k_cache.data_ptr()) % 16 == 0 && ((size_t)v_cache.data_ptr()) % 16 == 0) {
     // decode tokens: the heads of a key/value group are the rows of a tile
     const int rep = H / G, zb = (rep + 15) / 16;
-    const size_t stage = (size_t)kDW * Dv * (kKT + kVPad) * sizeof(bf16raw);
+    const size_t stage = (size_t)kDW * decode_stage_bytes(Dv);
     const size_t join = (size_t)kDW * (32 + 16 * Dv) * sizeof(float);
     // split the keys over blocks so that a wave walks about two tiles at the
     // longest context the block tables can describe; splits beyond a
     // sequence's keys exit at once
-    const int64_t cap = (int64_t)block_tables.size(1) * bs;
+    int64_t cap = (int64_t)block_tables.size(1) * bs;
+    if (window > 0) cap = std::min(cap, window + keep_first);
+    if (chunk > 0) cap = std::min(cap, chunk);
     int n_split = (int)std::min<int64_t>(16, std::max<int64_t>(1, (cap + 255) / 256));
     // past about eight blocks a CU more splits only add joins (64 sequences of
     // 1536 tokens on 8 key heads: 144 us with 16 splits, 91 us with 4)
@@ -1069,27 +1353,38 @@ void masked_paged_attention(torch::Tensor out, torch::Tensor q,
       part_o = torch::empty({(int64_t)T * H * n_split, Dv}, f32);
       part_ml = torch::empty({(int64_t)T * H * n_split, 2}, f32);
     }
-    auto decode_kern = D <= 128 ? masked_decode_mfma_kernel<8, 8>
-                                : masked_decode_mfma_kernel<16, 8>;
-    hipLaunchKernelGGL(decode_kern, dim3(T, G, zb * n_split),
-                       dim3(kDW * WAVE), stage > join ? stage : join, SEQ_STREAM(),
-                       (bf16raw*)out.data_ptr(), out.stride(0),
-                       (const bf16raw*)q.data_ptr(), q.stride(0),
-                       (const bf16raw*)k_cache.data_ptr(),
-                       (const bf16raw*)v_cache.data_ptr(),
-                       (const int*)block_tables.data_ptr(), (int)block_tables.size(1),
-                       (const int*)token_seq.data_ptr(), (const int*)positions.data_ptr(),
-                       (float)scale, (float)softcap, (int)chunk, (int)window,
-                       (float)out_scale, sink, v_rs, H, G, D, Dv, bs, n_split,
-                       n_split > 1 ? (float*)part_o.data_ptr() : nullptr,
-                       n_split > 1 ? (float*)part_ml.data_ptr() : nullptr, kvs);
+    auto launch = [&](auto kern) {
+      hipLaunchKernelGGL(kern, dim3(T, G, zb * n_split), dim3(kDW * WAVE),
+                         stage > join ? stage : join, SEQ_STREAM(),
+                         (bf16raw*)out.data_ptr(), out.stride(0),
+                         (const bf16raw*)q.data_ptr(), q.stride(0),
+                         (const bf16raw*)k_cache.data_ptr(),
+                         (const bf16raw*)v_cache.data_ptr(),
+                         (const int*)block_tables.data_ptr(), (int)block_tables.size(1),
+                         (const int*)token_seq.data_ptr(),
+                         (const int*)positions.data_ptr(), n_split,
+                         n_split > 1 ? (float*)part_o.data_ptr() : nullptr,
+                         n_split > 1 ? (float*)part_ml.data_ptr() : nullptr, args);
+    };
+    auto pick = [&](auto wide, auto is_tied) {
+      constexpr bool kW = decltype(wide)::value, kT = decltype(is_tied)::value;
+      if (D <= 128) launch(masked_decode_mfma_kernel<8, 8, kW, kT>);
+      else launch(masked_decode_mfma_kernel<16, 8, kW, kT>);
+    };
+    if (D % 32 == 0 && Dv % 32 == 0) {
+      if (tied) pick(std::true_type{}, std::true_type{});
+      else pick(std::true_type{}, std::false_type{});
+    } else {
+      if (tied) pick(std::false_type{}, std::true_type{});
+      else pick(std::false_type{}, std::false_type{});
+    }
     if (n_split > 1) {
       SEQ_CHECK_LAUNCH();
       hipLaunchKernelGGL(decode_split_join_kernel, dim3(T, H), dim3(64), 0, SEQ_STREAM(),
                          (bf16raw*)out.data_ptr(), out.stride(0),
                          (const float*)part_o.data_ptr(),
                          (const float*)part_ml.data_ptr(), H, (int)Dv, n_split,
-                         (float)out_scale, sink);
+                         (float)out_scale, args.sink);
     }
     SEQ_CHECK_LAUNCH();
     return;
@@ -1113,9 +1408,7 @@ void masked_paged_attention(torch::Tensor out, torch::Tensor q,
                          (const act_t*)v_cache.data_ptr(),
                          (const int*)block_tables.data_ptr(),
                          (int)block_tables.size(1), (const int*)token_seq.data_ptr(),
-                         (const int*)positions.data_ptr(), (float)scale,
-                         (float)softcap, (int)chunk, (int)window, (float)out_scale,
-                         sink, v_rs, H, G, D, Dv, bs, kvs);
+                         (const int*)positions.data_ptr(), args);
     };
     if (vec) launch(masked_paged_attention_kernel<act_t, true>);
     else launch(masked_paged_attention_kernel<act_t, false>);

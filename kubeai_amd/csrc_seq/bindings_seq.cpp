@@ -35,7 +35,21 @@ void masked_paged_attention(torch::Tensor out, torch::Tensor q,
                             torch::Tensor token_seq, torch::Tensor positions,
                             int64_t max_len, double scale, double softcap,
                             int64_t chunk, int64_t window, double out_scale,
-                            c10::optional<torch::Tensor> sink_scores);
+                            c10::optional<torch::Tensor> sink_scores,
+                            int64_t keep_first, c10::optional<torch::Tensor> slopes,
+                            c10::optional<torch::Tensor> key_scale);
+void qnorm_rows_to_cache(torch::Tensor q, torch::Tensor k, torch::Tensor q_weight,
+                         double eps, torch::Tensor cache, torch::Tensor key_scale,
+                         torch::Tensor slot_mapping);
+void add_dyt_conv(torch::Tensor out, torch::Tensor new_residual,
+                  c10::optional<torch::Tensor> branch,
+                  c10::optional<torch::Tensor> post_alpha,
+                  c10::optional<torch::Tensor> post_w,
+                  c10::optional<torch::Tensor> post_b, torch::Tensor residual,
+                  torch::Tensor alpha, torch::Tensor w, torch::Tensor b,
+                  c10::optional<torch::Tensor> conv_w,
+                  c10::optional<torch::Tensor> tails, torch::Tensor start_loc,
+                  torch::Tensor slots, torch::Tensor positions, int64_t max_len);
 void qknorm_rope_half_and_cache(torch::Tensor q, torch::Tensor k, torch::Tensor v,
                                 c10::optional<torch::Tensor> q_weight,
                                 c10::optional<torch::Tensor> k_weight, double eps,
@@ -72,10 +86,10 @@ void latent_rope_to_cache(torch::Tensor cache, torch::Tensor x, torch::Tensor we
                           torch::Tensor slot_mapping);
 void router_scores_topk(torch::Tensor logits, c10::optional<torch::Tensor> bias,
                         torch::Tensor dense, torch::Tensor weights,
-                        torch::Tensor index, double scale);
+                        torch::Tensor index, double scale, int64_t score);
 void glu_weighted(torch::Tensor out, torch::Tensor gu, c10::optional<torch::Tensor> w,
                   int64_t group, double alpha, double limit, double up_shift,
-                  bool w_sigmoid);
+                  bool w_sigmoid, bool w_input);
 void embed_sinusoid(torch::Tensor out, torch::Tensor ids, torch::Tensor table,
                     double scale, torch::Tensor positions, torch::Tensor freqs);
 void hyper_mix_rmsnorm(torch::Tensor out, torch::Tensor streams,
@@ -114,6 +128,10 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "chunk/window-masked paged softmax attention, optional sink");
   m.def("qknorm_rope_half_and_cache", &qknorm_rope_half_and_cache,
         "whole-row q/k RMS norm + split-half rotary + paged cache write");
+  m.def("qnorm_rows_to_cache", &qnorm_rows_to_cache,
+        "whole-row q norm; k rows and their 1/rms into a paged cache");
+  m.def("add_dyt_conv", &add_dyt_conv,
+        "dynamic tanh of a branch + fp32 residual add + dynamic tanh + causal conv");
   m.def("sandwich_rmsnorm", &sandwich_rmsnorm,
         "post-norm of a branch + fp32 residual add + next pre-norm");
   m.def("rmsnorm_to_cache", &rmsnorm_to_cache, "RMS norm written into a paged cache");

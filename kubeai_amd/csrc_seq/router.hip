@@ -66,7 +66,8 @@ __global__ void relu_squared_weighted_kernel(T* __restrict__ out,
   stf(out + i, r * r * s);
 }
 
-// One thread per token: scores s = softmax(logits) over all experts; the
+// One thread per token: scores s = softmax(logits) over all experts, or the
+// logits' sigmoids (sigmoid != 0); the
 // `top` experts with the largest s + bias are chosen in the order (value
 // descending, index ascending); their weights are their scores s as they
 // are, times wscale. dense[t, e] holds the weight at a chosen expert's column, else 0.
@@ -76,20 +77,24 @@ __global__ void router_scores_topk_kernel(const float* __restrict__ logits,
                                           float* __restrict__ dense,
                                           float* __restrict__ weights,
                                           int* __restrict__ index, int T, int E,
-                                          int top, float wscale) {
+                                          int top, float wscale, int sigmoid) {
   const int t = blockIdx.x * blockDim.x + threadIdx.x;
   if (t >= T) return;
   const float* z = logits + (size_t)t * E;
   float* s = dense + (size_t)t * E;
-  float zmax = -INFINITY;
-  for (int e = 0; e < E; ++e) zmax = fmaxf(zmax, z[e]);
-  float sum = 0.f;
-  for (int e = 0; e < E; ++e) {
-    const float p = expf(z[e] - zmax);
-    s[e] = p;
-    sum += p;
+  if (sigmoid) {
+    for (int e = 0; e < E; ++e) s[e] = sigmoid_f(z[e]);
+  } else {
+    float zmax = -INFINITY;
+    for (int e = 0; e < E; ++e) zmax = fmaxf(zmax, z[e]);
+    float sum = 0.f;
+    for (int e = 0; e < E; ++e) {
+      const float p = expf(z[e] - zmax);
+      s[e] = p;
+      sum += p;
+    }
+    for (int e = 0; e < E; ++e) s[e] = s[e] / sum;
   }
-  for (int e = 0; e < E; ++e) s[e] = s[e] / sum;
   float last_v = INFINITY;
   int last_i = -1;
   for (int k = 0; k < top; ++k) {
@@ -118,11 +123,12 @@ __global__ void router_scores_topk_kernel(const float* __restrict__ logits,
 // up columns (gu [T, n * 2 * group], strided rows):
 //   g = gate, u = up; limit > 0: g = min(g, limit), u = clamp(u, -limit, limit)
 //   out[t, e * group + c] = g * sigmoid(alpha * g) * (u + shift) * weight[t, e]
-// weight: absent (1), w itself, or sigmoid(w). One thread per N consecutive
+// weight: absent (1), w itself, or sigmoid(w); w_input: it multiplies gate and
+// up (the expert's input) instead of the product. One thread per N consecutive
 // channels (N = 1, or the elements of a 16-byte access).
 struct GluParams {
   float alpha, limit, shift;
-  int w_sigmoid;
+  int w_sigmoid, w_input;
 };
 
 DEV_INLINE float glu_f(float g, float u, const GluParams& p) {
@@ -151,15 +157,16 @@ __global__ void glu_weighted_kernel(T* __restrict__ out, int64_t out_stride,
     wt = w[t * w_stride + e];
     if (p.w_sigmoid) wt = sigmoid_f(wt);
   }
+  const float wi = p.w_input ? wt : 1.f, wo = p.w_input ? 1.f : wt;
   if constexpr (kVec) {
     float g[N], u[N];
     Vec16<T>::load(row + j, g);
     Vec16<T>::load(row + group + j, u);
 #pragma unroll
-    for (int x = 0; x < N; ++x) g[x] = glu_f(g[x], u[x], p) * wt;
+    for (int x = 0; x < N; ++x) g[x] = glu_f(g[x] * wi, u[x] * wi, p) * wo;
     Vec16<T>::store(out + t * out_stride + c, g);
   } else {
-    stf(out + t * out_stride + c, glu_f(ldf(row + j), ldf(row + group + j), p) * wt);
+    stf(out + t * out_stride + c, glu_f(ldf(row + j) * wi, ldf(row + group + j) * wi, p) * wo);
   }
 }
 
@@ -167,13 +174,14 @@ __global__ void glu_weighted_kernel(T* __restrict__ out, int64_t out_stride,
 
 void router_scores_topk(torch::Tensor logits, c10::optional<torch::Tensor> bias,
                         torch::Tensor dense, torch::Tensor weights,
-                        torch::Tensor index, double scale) {
+                        torch::Tensor index, double scale, int64_t score) {
   check_f32(logits, "logits");
   check_f32(dense, "dense");
   check_f32(weights, "weights");
   check_i32(index, "index");
   TORCH_CHECK(logits.dim() == 2 && weights.dim() == 2);
   const int T = logits.size(0), E = logits.size(1), top = weights.size(1);
+  TORCH_CHECK(score == 0 || score == 1, "score: 0 softmax, 1 sigmoid");
   TORCH_CHECK(top >= 1 && top <= E, "top must be within the number of experts");
   TORCH_CHECK(dense.numel() == (int64_t)T * E && weights.size(0) == T &&
               index.numel() == (int64_t)T * top);
@@ -187,13 +195,13 @@ void router_scores_topk(torch::Tensor logits, c10::optional<torch::Tensor> bias,
   hipLaunchKernelGGL(router_scores_topk_kernel, dim3((T + 63) / 64), dim3(64), 0,
                      SEQ_STREAM(), (const float*)logits.data_ptr(), bp,
                      (float*)dense.data_ptr(), (float*)weights.data_ptr(),
-                     (int*)index.data_ptr(), T, E, top, (float)scale);
+                     (int*)index.data_ptr(), T, E, top, (float)scale, (int)score);
   SEQ_CHECK_LAUNCH();
 }
 
 void glu_weighted(torch::Tensor out, torch::Tensor gu, c10::optional<torch::Tensor> w,
                   int64_t group, double alpha, double limit, double up_shift,
-                  bool w_sigmoid) {
+                  bool w_sigmoid, bool w_input) {
   check_rows(gu, "gu");
   check_rows(out, "out");
   TORCH_CHECK(out.scalar_type() == gu.scalar_type());
@@ -211,7 +219,8 @@ void glu_weighted(torch::Tensor out, torch::Tensor gu, c10::optional<torch::Tens
     ws = w->stride(0);
   }
   if (T == 0 || C == 0) return;
-  const GluParams p{(float)alpha, (float)limit, (float)up_shift, w_sigmoid ? 1 : 0};
+  const GluParams p{(float)alpha, (float)limit, (float)up_shift, w_sigmoid ? 1 : 0,
+                    w_input ? 1 : 0};
   const int vn = 16 / gu.element_size();
   const bool vec = group % vn == 0 && gu.stride(0) % vn == 0 && out.stride(0) % vn == 0 &&
                    ((size_t)gu.data_ptr()) % 16 == 0 && ((size_t)out.data_ptr()) % 16 == 0;

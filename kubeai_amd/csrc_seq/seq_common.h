@@ -79,6 +79,18 @@ template <> struct Vec16<bf16raw> {
 DEV_INLINE float sigmoid_f(float x) { return 1.0f / (1.0f + expf(-x)); }
 DEV_INLINE float silu_f(float x) { return x / (1.0f + expf(-x)); }
 
+// tanh to about 3e-7 relative: (1 - t) / (1 + t) with t = e^(-2|x|), and near
+// zero, where that cancels, the Taylor polynomial up to x^9
+DEV_INLINE float tanh_f(float x) {
+  const float ax = fabsf(x), s = x * x;
+  const float t = __builtin_amdgcn_exp2f(-2.8853900817779268f * ax);
+  const float big = copysignf((1.f - t) * __builtin_amdgcn_rcpf(1.f + t), x);
+  float p = fmaf(s, 62.f / 2835.f, -17.f / 315.f);
+  p = fmaf(s, p, 2.f / 15.f);
+  p = fmaf(s, p, -1.f / 3.f);
+  return ax < 0.25f ? fmaf(x * s, p, x) : big;
+}
+
 DEV_INLINE float wave_sum(float v) {
 #pragma unroll
   for (int off = 32; off > 0; off >>= 1) v += __shfl_xor(v, off, WAVE);
