@@ -1,13 +1,15 @@
 """Prefill and decode throughput of a layer-list design (Dulotar, Nugopel,
-Vekusun, Vigonex) beside the closest existing stack of equal width, depth and
+Vekusun, Vigonex, Pubopel) beside the closest existing stack of equal width, depth and
 (about) parameter count, random weights, one GPU: a dense Llama for Dulotar,
 a Mixtral-style routed Llama (same number of experts and choices) for
-Nugopel, Nugopel itself (latent attention, routed experts) for Vekusun, and
+Nugopel, Nugopel itself (latent attention, routed experts) for Vekusun,
 Vekusun (full causal attention, a delta rule, dense and routed gated
-feed-forwards, sequence state) for Vigonex; the feed-forward sizes of the
-last two are scaled so that the parameter counts agree.
+feed-forwards, sequence state) for Vigonex, and Nugopel (window attention with
+a sink and whole-projection norms, norms on both sides of a sublayer, routed
+experts with a shared one) for Pubopel; the feed-forward sizes of the last
+three are scaled so that the parameter counts agree.
 
-    python bench.py --compare-hybrid [--compare-design dulotar|nugopel|vekusun|vigonex]
+    python bench.py --compare-hybrid [--compare-design dulotar|nugopel|vekusun|vigonex|pubopel]
                     [--compare-sizes 1k,2k,4k]
 
 Prefill: one sequence's whole prompt as a single fixed step (both families
@@ -24,8 +26,11 @@ import time
 
 import torch
 
+from kubeai_amd.models import config as configs
 from kubeai_amd.models.config import PRESETS, ModelArchConfig
 
+# design -> the layer-list design it is compared with at equal parameter count
+SIZED_LIKE = {"vekusun": "nugopel", "vigonex": "vekusun", "pubopel": "nugopel"}
 SIZES = {"1k": (1024, 12), "2k": (2048, 12), "4k": (4096, 6)}
 
 
@@ -75,12 +80,6 @@ def _sized_like(preset, width: int, layers: int, target_params: int) -> ModelArc
     p2 = _meta_params(preset(width, layers, ff_scale=2.0))
     scale = 1.0 + (target_params - p1) / max(p2 - p1, 1)
     return preset(width, layers, ff_scale=max(scale, 0.1))
-
-
-def _vekusun_sized_like(width: int, layers: int, target_params: int) -> ModelArchConfig:
-    from kubeai_amd.models.config import vekusun_preset
-
-    return _sized_like(vekusun_preset, width, layers, target_params)
 
 
 def _engine(name: str, device: str, blocks: int, seqs: int, max_len: int):
@@ -146,21 +145,16 @@ def main(args) -> None:
     prefill_lens = [2048, 8192] if device == "cuda" else [64]
     batches = [(64, 1536), (8, 3584)] if device == "cuda" else [(2, 32)]
     design = getattr(args, "compare_design", None) or "dulotar"
-    if design not in ("dulotar", "nugopel", "vekusun", "vigonex"):
+    if design not in ("dulotar", "nugopel", "vekusun", "vigonex", "pubopel"):
         raise SystemExit(f"unknown design {design!r}")
     for key in sizes:
         width, layers = SIZES[key]
         name = f"{design}-{key}" if device == "cuda" else f"{design}-tiny"
-        if design == "vekusun" and device == "cuda":
-            name = f"vekusun-like-nugopel-{key}"
-            PRESETS[name] = _vekusun_sized_like(
-                width, layers, _meta_params(PRESETS[f"nugopel-{key}"]))
-        if design == "vigonex" and device == "cuda":
-            from kubeai_amd.models.config import vigonex_preset
-
-            name = f"vigonex-like-vekusun-{key}"
-            PRESETS[name] = _sized_like(vigonex_preset, width, layers,
-                                        _meta_params(PRESETS[f"vekusun-{key}"]))
+        if design in SIZED_LIKE and device == "cuda":
+            other = SIZED_LIKE[design]
+            name = f"{design}-like-{other}-{key}"
+            PRESETS[name] = _sized_like(getattr(configs, f"{design}_preset"), width, layers,
+                                        _meta_params(PRESETS[f"{other}-{key}"]))
         arch = PRESETS[name]
         max_len = 8192 + 256
         blocks = (max(b * (c + 128) for b, c in batches) + max_len) // 16 + 64
@@ -170,12 +164,9 @@ def main(args) -> None:
         ref_name = f"llama-like-{key}"
         ref_fam = "llama"
         moe = arch.hybrid.layers[0].mlp if design == "nugopel" else None
-        if design == "vekusun":
-            ref_fam = "nugopel"
-            ref_name = f"nugopel-{key}" if device == "cuda" else "nugopel-tiny"
-        elif design == "vigonex":
-            ref_fam = "vekusun"
-            ref_name = f"vekusun-{key}" if device == "cuda" else "vekusun-tiny"
+        if design in SIZED_LIKE:
+            ref_fam = SIZED_LIKE[design]
+            ref_name = f"{ref_fam}-{key}" if device == "cuda" else f"{ref_fam}-tiny"
         elif moe:
             ref_fam = "mixtral"
             PRESETS[ref_name] = _llama_like(
