@@ -213,6 +213,21 @@ struct AttnArgs {
   DEV_INLINE int kept(int lo) const { return min(keep, lo); }
 };
 
+// Query tiles of a packed step: with `size` queries a tile, run s owns tile
+// numbers start_loc[s] / size + s and on (never fewer than it needs), so T /
+// size + n_seq blocks cover every batch, whatever its mix of lengths. Returns
+// the run of tile number b and b's place in the run.
+DEV_INLINE int find_tile(const int* start_loc, int n_seq, int size, int b, int* tile) {
+  int lo = 0, hi = n_seq - 1;  // the last run whose first number is <= b
+  while (lo < hi) {
+    const int mid = (lo + hi + 1) >> 1;
+    if (start_loc[mid] / size + mid <= b) lo = mid;
+    else hi = mid - 1;
+  }
+  *tile = b - (start_loc[lo] / size + lo);
+  return lo;
+}
+
 // softcap * tanh(x / softcap) times log2 e as cap2 - 2 cap2 / (e^(2x/cap) + 1):
 // absolute error below 1e-6 of the cap. x comes multiplied by 2 log2(e) / cap.
 DEV_INLINE float cap_base2(float x, float cap2) {
@@ -376,7 +391,7 @@ typedef __attribute__((ext_vector_type(4))) float f32x4;
 
 
 // Prompt portions on the matrix cores (bf16, key and value sizes multiples
-// of 16). grid (n_seq * tiles_per_run, H), one wave per 16 consecutive
+// of 16). grid (query tiles, H), one wave per 16 consecutive
 // queries of a run and one query head. Per 16-key tile:
 //   S^T = K Q^T   (v_mfma_f32_16x16x16_bf16, K rows straight from the cache)
 //   fp32 scale, cap, mask, running max / sum per query (a query is a lane
@@ -390,9 +405,10 @@ __global__ __launch_bounds__(WAVE) void masked_prefill_mfma_kernel(
     int64_t q_stride, const bf16raw* __restrict__ k_cache,
     const bf16raw* __restrict__ v_cache, const int* __restrict__ block_tables,
     int max_blocks, const int* __restrict__ start_loc,
-    const int* __restrict__ positions, int tiles_per_run, AttnArgs a) {
+    const int* __restrict__ positions, int n_seq, AttnArgs a) {
   const int H = a.H, G = a.G, D = a.D, Dv = a.Dv, bs = a.bs;
-  const int s = blockIdx.x / tiles_per_run, tile = blockIdx.x % tiles_per_run;
+  int tile;
+  const int s = find_tile(start_loc, n_seq, 16, blockIdx.x, &tile);
   const int h = blockIdx.y, g = h / (H / G);
   const int s0 = start_loc[s], s1 = start_loc[s + 1];
   const int q0 = s0 + tile * 16;
@@ -597,7 +613,7 @@ __global__ __launch_bounds__(512) void masked_prefill_mfma_shared_kernel(
     int64_t q_stride, const bf16raw* __restrict__ k_cache,
     const bf16raw* __restrict__ v_cache, const int* __restrict__ block_tables,
     int max_blocks, const int* __restrict__ start_loc,
-    const int* __restrict__ positions, int tiles_per_run, int HW, int QW, AttnArgs a) {
+    const int* __restrict__ positions, int n_seq, int HW, int QW, AttnArgs a) {
   extern __shared__ __attribute__((aligned(16))) bf16raw lds[];
   typedef QkFrag<kWideQK> Frag;
   typedef typename Frag::type frag_t;
@@ -609,7 +625,8 @@ __global__ __launch_bounds__(512) void masked_prefill_mfma_shared_kernel(
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int col = lane & 15, grp = lane >> 4;
   const int hw = wave % HW, qw = wave / HW;
-  const int s = blockIdx.x / tiles_per_run, tile = blockIdx.x % tiles_per_run;
+  int tile;
+  const int s = find_tile(start_loc, n_seq, QW * 16, blockIdx.x, &tile);
   const int g = blockIdx.y, rep = a.H / G;
   const int hz = blockIdx.z * HW + hw;
   const int s0 = start_loc[s], s1 = start_loc[s + 1];
@@ -1265,16 +1282,16 @@ void masked_paged_attention(torch::Tensor out, torch::Tensor q,
   if (q.scalar_type() == torch::kBFloat16 && max_len > 1 && D % 16 == 0 &&
       Dv % 16 == 0 && D <= 512 && Dv <= 512 && al8(q) && al8(out) && v_rs % 8 == 0) {
     // prompt portions: matrix-core kernel over 16-query tiles of every run
-    const int tiles = (int)((max_len + 15) / 16);
+    const int tiles = T / 16 + n_seq;
     auto launch = [&](auto kern) {
-      hipLaunchKernelGGL(kern, dim3(n_seq * tiles, H), dim3(WAVE), 0, SEQ_STREAM(),
+      hipLaunchKernelGGL(kern, dim3(tiles, H), dim3(WAVE), 0, SEQ_STREAM(),
                          (bf16raw*)out.data_ptr(), out.stride(0),
                          (const bf16raw*)q.data_ptr(), q.stride(0),
                          (const bf16raw*)k_cache.data_ptr(),
                          (const bf16raw*)v_cache.data_ptr(),
                          (const int*)block_tables.data_ptr(),
                          (int)block_tables.size(1), (const int*)start_loc.data_ptr(),
-                         (const int*)positions.data_ptr(), tiles, args);
+                         (const int*)positions.data_ptr(), n_seq, args);
     };
     const size_t lds_shared =
         (size_t)2 * (kKT * (D + kRPad) + (tied ? 0 : kKT * (Dv + kRPad)) + 2 * kKT) *
@@ -1287,27 +1304,30 @@ void masked_paged_attention(torch::Tensor out, torch::Tensor q,
       const int rep = H / G;
       int HW = 1;
       while (HW * 2 <= rep && HW < 8) HW *= 2;
-      const int WPB = HW < 4 ? 4 : HW;
+      const int WPB = 8;
       const int QW = WPB / HW;
-      const int btiles = (int)((max_len + QW * 16 - 1) / (QW * 16));
+      const int btiles = T / (QW * 16) + n_seq;
       const int zb = (rep + HW - 1) / HW;
       TORCH_CHECK(G <= 65535 && zb <= 65535);
       auto launch_shared = [&](auto kern) {
       hipLaunchKernelGGL(kern,
-                         dim3(n_seq * btiles, G, zb), dim3(WPB * WAVE), lds_shared,
+                         dim3(btiles, G, zb), dim3(WPB * WAVE), lds_shared,
                          SEQ_STREAM(), (bf16raw*)out.data_ptr(), out.stride(0),
                          (const bf16raw*)q.data_ptr(), q.stride(0),
                          (const bf16raw*)k_cache.data_ptr(),
                          (const bf16raw*)v_cache.data_ptr(),
                          (const int*)block_tables.data_ptr(),
                          (int)block_tables.size(1), (const int*)start_loc.data_ptr(),
-                         (const int*)positions.data_ptr(), btiles, HW, QW, args);
+                         (const int*)positions.data_ptr(), n_seq, HW, QW, args);
       };
       // key sizes above 128 (a latent with a rotated part behind it) keep
       // twice as many query fragments in registers
       auto pick = [&](auto wide, auto is_tied) {
         constexpr bool kW = decltype(wide)::value, kT = decltype(is_tied)::value;
-        if (D <= 128) launch_shared(masked_prefill_mfma_shared_kernel<8, kT ? 8 : 16, kW, kT>);
+        if (D <= 128 && Dv <= 128)
+          launch_shared(masked_prefill_mfma_shared_kernel<8, 8, kW, kT>);
+        else if (D <= 128)
+          launch_shared(masked_prefill_mfma_shared_kernel<8, 16, kW, kT>);
         else launch_shared(masked_prefill_mfma_shared_kernel<16, 16, kW, kT>);
       };
       if (D % 32 == 0) {

@@ -49,7 +49,8 @@ void add_dyt_conv(torch::Tensor out, torch::Tensor new_residual,
                   torch::Tensor alpha, torch::Tensor w, torch::Tensor b,
                   c10::optional<torch::Tensor> conv_w,
                   c10::optional<torch::Tensor> tails, torch::Tensor start_loc,
-                  torch::Tensor slots, torch::Tensor positions, int64_t max_len);
+                  torch::Tensor slots, torch::Tensor token_seq,
+                  torch::Tensor positions, int64_t max_len);
 void qknorm_rope_half_and_cache(torch::Tensor q, torch::Tensor k, torch::Tensor v,
                                 c10::optional<torch::Tensor> q_weight,
                                 c10::optional<torch::Tensor> k_weight, double eps,

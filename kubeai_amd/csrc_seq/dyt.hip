@@ -39,26 +39,26 @@ template <int V> DEV_INLINE void store_act(bf16raw* p, const float* x) {
   }
 }
 
-// grid (n_seq * spans, channel blocks); a thread owns V channels of `span`
-// consecutive tokens of one run:
+// grid (token spans, channel blocks); a thread owns V channels of `span`
+// consecutive tokens of the packed stream:
 //   r' = r + dyt_post(branch),  h = dyt_pre(r'),  out = h + sum_j conv[j] h_(t-K1+j)
-// TAIL bounds taps - 1; the window is kept zero-padded to TAIL entries. The
-// inputs ahead of a span come from the run's own tokens (formed again: r is
-// read, not updated in place) or from the carried tail; positions < 0 are 0.
-// A run that is one span advances its tail here; longer ones leave that to
-// dyt_tail_kernel, since their first span may still be reading it.
+// TAIL bounds taps - 1; the window is kept zero-padded to TAIL entries. Inputs
+// ahead of a span come from their run's own tokens (formed again: r is read,
+// not updated in place), inputs ahead of a run from its carried tail;
+// positions < 0 are 0. A run inside one span advances its tail here; the
+// others leave that to dyt_tail_kernel, since their first span may still be
+// reading it.
 template <typename T, typename B, int V, int TAIL>
 __global__ __launch_bounds__(128) void add_dyt_conv_kernel(
     T* __restrict__ out, float* __restrict__ r_out, const B* __restrict__ branch,
     DytParams post, const float* __restrict__ r_in, DytParams pre,
     const float* __restrict__ conv_w, float* __restrict__ tails,
     const int* __restrict__ start_loc, const int* __restrict__ slots,
-    const int* __restrict__ positions, int C, int K1, int spans, int span) {
-  const int s = blockIdx.x / spans, sp = blockIdx.x % spans;
+    const int* __restrict__ token_seq, const int* __restrict__ positions, int T_all,
+    int C, int K1, int span) {
   const int c = (blockIdx.y * blockDim.x + threadIdx.x) * V;
-  const int s0 = start_loc[s], s1 = start_loc[s + 1];
-  const int t0 = s0 + sp * span, t1 = min(s1, t0 + span);
-  if (c >= C || t0 >= s1) return;
+  const int t0 = blockIdx.x * span, t1 = min(T_all, t0 + span);
+  if (c >= C) return;
   const float al = pre.alpha[0], alp = branch != nullptr ? post.alpha[0] : 0.f;
   float w[V], b[V], pw[V], pb[V];
   load_f<V>(pre.w + c, w);
@@ -90,24 +90,31 @@ __global__ __launch_bounds__(128) void add_dyt_conv_kernel(
       cw[j][e] = conv_w != nullptr && tap >= 0
                      ? conv_w[(size_t)(c + e) * (K1 + 1) + tap] : 0.f;
     }
-  const int slot = conv_w != nullptr ? slots[s] : -1;
-  const int p0 = positions[s0];
+  int s0 = 0, s1 = 0, slot = -1;  // the run that token t lies in
+  auto enter_run = [&](int t) {
+    const int s = token_seq[t];
+    s0 = start_loc[s];
+    s1 = start_loc[s + 1];
+    slot = slots[s];
+    const int p0 = positions[s0];
 #pragma unroll
-  for (int i = 0; i < TAIL; ++i) {
-    const int d = TAIL - i;  // steps back from t0
-    const int t = t0 - d;
+    for (int i = 0; i < TAIL; ++i) {
+      const int d = TAIL - i;  // steps back from t
+      const int tb = t - d;
 #pragma unroll
-    for (int e = 0; e < V; ++e) hist[i][e] = 0.f;
-    if (d > K1) continue;
-    if (t >= s0) {
-      float x[V];
-      residual(t, x);
-      squash(x, hist[i]);
-    } else if (slot >= 0 && p0 + (t - s0) >= 0) {
-      load_f<V>(tails + ((size_t)slot * K1 + (t - s0 + K1)) * C + c, hist[i]);
+      for (int e = 0; e < V; ++e) hist[i][e] = 0.f;
+      if (d > K1) continue;
+      if (tb >= s0) {
+        float x[V];
+        residual(tb, x);
+        squash(x, hist[i]);
+      } else if (slot >= 0 && p0 + (tb - s0) >= 0) {
+        load_f<V>(tails + ((size_t)slot * K1 + (tb - s0 + K1)) * C + c, hist[i]);
+      }
     }
-  }
+  };
   for (int t = t0; t < t1; ++t) {
+    if (TAIL > 0 && t >= s1) enter_run(t);
     float x[V], h[V], y[V];
     residual(t, x);
     if (branch != nullptr) store_act<V>(r_out + (size_t)t * C + c, x);
@@ -126,28 +133,37 @@ __global__ __launch_bounds__(128) void add_dyt_conv_kernel(
       for (int i = 0; i + 1 < TAIL; ++i) hist[i][e] = hist[i + 1][e];
       if (TAIL > 0) hist[TAIL > 0 ? TAIL - 1 : 0][e] = h[e];
     }
-  }
-  if (slot >= 0 && s1 - s0 <= span) {
+    if (TAIL > 0 && t == s1 - 1 && slot >= 0 && s0 >= t0) {
 #pragma unroll
-    for (int i = 0; i < TAIL; ++i)
-      if (i >= TAIL - K1)
-        store_act<V>(tails + ((size_t)slot * K1 + (i - (TAIL - K1))) * C + c, hist[i]);
+      for (int i = 0; i < TAIL; ++i)
+        if (i >= TAIL - K1)
+          store_act<V>(tails + ((size_t)slot * K1 + (i - (TAIL - K1))) * C + c, hist[i]);
+    }
   }
 }
 
-// grid (n_seq, channel blocks): tails of runs longer than one span (and so
-// longer than the tail), formed from the updated residual.
+// grid (n_seq, channel blocks): tails of runs that cross a span's border, from
+// the updated residual. One thread owns a channel's tail and moves it towards
+// the front, so a run shorter than the tail shifts it safely.
 __global__ void dyt_tail_kernel(float* __restrict__ tails, const float* __restrict__ r,
                                 DytParams pre, const int* __restrict__ start_loc,
-                                const int* __restrict__ slots, int C, int K1, int span) {
+                                const int* __restrict__ slots,
+                                const int* __restrict__ positions, int C, int K1,
+                                int span) {
   const int s = blockIdx.x;
   const int c = blockIdx.y * blockDim.x + threadIdx.x;
-  const int slot = slots[s], s0 = start_loc[s], s1 = start_loc[s + 1];
-  if (c >= C || slot < 0 || s1 - s0 <= span) return;
+  const int slot = slots[s], s0 = start_loc[s], n = start_loc[s + 1] - s0;
+  if (c >= C || slot < 0 || n <= 0 || s0 / span == (s0 + n - 1) / span) return;
+  const int p0 = positions[s0];
   const float al = pre.alpha[0], w = pre.w[c], b = pre.b[c];
-  for (int i = 0; i < K1; ++i)
-    tails[((size_t)slot * K1 + i) * C + c] =
-        fmaf(tanh_f(al * r[(size_t)(s1 - K1 + i) * C + c]), w, b);
+  float* tail = tails + (size_t)slot * K1 * C + c;
+  for (int i = 0; i < K1; ++i) {
+    const int u = n - K1 + i;  // place in the run; negative: carried
+    float v = 0.f;
+    if (u >= 0) v = fmaf(tanh_f(al * r[(size_t)(s0 + u) * C + c]), w, b);
+    else if (p0 + u >= 0) v = tail[(size_t)(i + n) * C];
+    tail[(size_t)i * C] = v;
+  }
 }
 
 }  // namespace
@@ -160,7 +176,8 @@ void add_dyt_conv(torch::Tensor out, torch::Tensor new_residual,
                   torch::Tensor alpha, torch::Tensor w, torch::Tensor b,
                   c10::optional<torch::Tensor> conv_w,
                   c10::optional<torch::Tensor> tails, torch::Tensor start_loc,
-                  torch::Tensor slots, torch::Tensor positions, int64_t max_len) {
+                  torch::Tensor slots, torch::Tensor token_seq,
+                  torch::Tensor positions, int64_t max_len) {
   check_f32(residual, "residual");
   check_f32(new_residual, "new_residual");
   check_f32(alpha, "alpha");
@@ -168,12 +185,14 @@ void add_dyt_conv(torch::Tensor out, torch::Tensor new_residual,
   check_f32(b, "b");
   check_i32(start_loc, "start_loc");
   check_i32(slots, "slots");
+  check_i32(token_seq, "token_seq");
   check_i32(positions, "positions");
   TORCH_CHECK(residual.dim() == 2 && out.is_cuda() && out.is_contiguous() &&
               out.sizes() == residual.sizes() && new_residual.sizes() == residual.sizes());
   const int T = residual.size(0), C = residual.size(1), n_seq = slots.numel();
   TORCH_CHECK(alpha.numel() == 1 && w.numel() == C && b.numel() == C);
-  TORCH_CHECK(start_loc.numel() == n_seq + 1 && positions.numel() == T && max_len >= 1);
+  TORCH_CHECK(start_loc.numel() == n_seq + 1 && token_seq.numel() == T &&
+              positions.numel() == T && max_len >= 1);
   TORCH_CHECK(branch.has_value() == post_alpha.has_value() &&
               branch.has_value() == post_w.has_value() &&
               branch.has_value() == post_b.has_value());
@@ -214,14 +233,15 @@ void add_dyt_conv(torch::Tensor out, torch::Tensor new_residual,
   if (T == 0 || n_seq == 0) return;
   const DytParams pre{(const float*)alpha.data_ptr(), (const float*)w.data_ptr(),
                       (const float*)b.data_ptr()};
-  const int span = 16;  // at least the largest tail
-  const int spans = (int)((max_len + span - 1) / span);
+  // decode: one token a thread; prompts: long spans repeat fewer inputs, short
+  // ones make more blocks
+  const int span = max_len == 1 ? 1 : T >= 4096 ? 16 : T >= 512 ? 8 : 4;
   auto al16 = [](const void* p) { return ((size_t)p) % 16 == 0; };
   const bool vec = C % 4 == 0 && al16(out.data_ptr()) && al16(residual.data_ptr()) &&
                    al16(new_residual.data_ptr()) && al16(bp) && al16(pre.w) &&
                    al16(pre.b) && al16(post.w) && al16(post.b) && al16(tp);
   const int V = vec ? 4 : 1;
-  const dim3 grid(n_seq * spans, (C + 128 * V - 1) / (128 * V));
+  const dim3 grid((T + span - 1) / span, (C + 128 * V - 1) / (128 * V));
   TORCH_CHECK(grid.y <= 65535);
   SEQ_DISPATCH_ACT(out, {
     auto go = [&](auto kern, auto* branch_ptr) {
@@ -229,7 +249,8 @@ void add_dyt_conv(torch::Tensor out, torch::Tensor new_residual,
                          (float*)new_residual.data_ptr(), branch_ptr, post,
                          (const float*)residual.data_ptr(), pre, cwp, tp,
                          (const int*)start_loc.data_ptr(), (const int*)slots.data_ptr(),
-                         (const int*)positions.data_ptr(), C, K1, spans, span);
+                         (const int*)token_seq.data_ptr(),
+                         (const int*)positions.data_ptr(), T, C, K1, span);
     };
     auto by_tail = [&](auto* branch_ptr) {
       using B = std::remove_const_t<std::remove_pointer_t<decltype(branch_ptr)>>;
@@ -244,11 +265,11 @@ void add_dyt_conv(torch::Tensor out, torch::Tensor new_residual,
     else by_tail((const act_t*)bp);
   });
   SEQ_CHECK_LAUNCH();
-  if (K1 > 0 && max_len > span) {
+  if (K1 > 0 && max_len > 1) {
     hipLaunchKernelGGL(dyt_tail_kernel, dim3(n_seq, (C + 255) / 256), dim3(256), 0,
                        SEQ_STREAM(), tp, (const float*)new_residual.data_ptr(), pre,
-                       (const int*)start_loc.data_ptr(), (const int*)slots.data_ptr(), C,
-                       K1, span);
+                       (const int*)start_loc.data_ptr(), (const int*)slots.data_ptr(),
+                       (const int*)positions.data_ptr(), C, K1, span);
     SEQ_CHECK_LAUNCH();
   }
 }

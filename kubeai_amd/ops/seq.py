@@ -226,7 +226,7 @@ def add_dyt_conv(branch, post, residual, pre, conv_w, tails, meta: SeqMeta, out_
         new = residual if branch is None else torch.empty_like(residual)
         _C.add_dyt_conv(out, new, branch, *(post if branch is not None else (None,) * 3),
                         residual, *pre, conv_w, tails, meta.start_loc, meta.slots,
-                        meta.positions, meta.max_len)
+                        meta.token_seq, meta.positions, meta.max_len)
         return out, new
     if branch is not None:
         residual = residual + torch.tanh(post[0] * branch.float()) * post[1] + post[2]
