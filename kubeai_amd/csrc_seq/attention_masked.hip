@@ -4,9 +4,16 @@
 // mask, with separate key and value sizes. Options: first tokens that stay
 // visible behind a window, a tanh cap, a bias per position, a scale per cached
 // key, and a sink (a score without a value: one more term in the denominator).
-#include "seq_common.h"
+#include "attn_masked.h"
 
 #include <type_traits>
+
+// Single decode tokens on the matrix cores (attention_masked_decode.hip); false
+// when the sizes are not its.
+bool masked_decode_mfma(const torch::Tensor& out, const torch::Tensor& q,
+                        const torch::Tensor& k_cache, const torch::Tensor& v_cache,
+                        const torch::Tensor& block_tables, const torch::Tensor& token_seq,
+                        const torch::Tensor& positions, const AttnArgs& args, bool tied);
 
 namespace {
 
@@ -191,49 +198,6 @@ __global__ __launch_bounds__(256) void qnorm_rows_cache_kernel(
 }
 
 constexpr int kMaxDvPerLane = 16;  // value size <= 1024
-constexpr float kLog2e = 1.4426950408889634f;
-
-// What every attention kernel below needs to know about scores and rows.
-// Visible keys of position p: [0, kept(p)) and [lower(p), p].
-struct AttnArgs {
-  float scale, softcap, out_scale;
-  int chunk, window, keep;
-  const float* sink;    // [H] or null: score of a key without a value
-  const float* slopes;  // [H] or null: slopes[h] * (i - j) comes off a score
-  const float* kscale;  // [blocks, bs] or null: factor of a cached key's scores
-  int64_t v_rs;         // elements between value rows
-  int H, G, D, Dv, bs, kvs;
-
-  DEV_INLINE int lower(int p) const {
-    int lo = 0;
-    if (chunk > 0) lo = (p / chunk) * chunk;
-    if (window > 0) lo = max(lo, p - window + 1);
-    return lo;
-  }
-  DEV_INLINE int kept(int lo) const { return min(keep, lo); }
-};
-
-// Query tiles of a packed step: with `size` queries a tile, run s owns tile
-// numbers start_loc[s] / size + s and on (never fewer than it needs), so T /
-// size + n_seq blocks cover every batch, whatever its mix of lengths. Returns
-// the run of tile number b and b's place in the run.
-DEV_INLINE int find_tile(const int* start_loc, int n_seq, int size, int b, int* tile) {
-  int lo = 0, hi = n_seq - 1;  // the last run whose first number is <= b
-  while (lo < hi) {
-    const int mid = (lo + hi + 1) >> 1;
-    if (start_loc[mid] / size + mid <= b) lo = mid;
-    else hi = mid - 1;
-  }
-  *tile = b - (start_loc[lo] / size + lo);
-  return lo;
-}
-
-// softcap * tanh(x / softcap) times log2 e as cap2 - 2 cap2 / (e^(2x/cap) + 1):
-// absolute error below 1e-6 of the cap. x comes multiplied by 2 log2(e) / cap.
-DEV_INLINE float cap_base2(float x, float cap2) {
-  return cap2 - 2.f * cap2 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(x) + 1.f);
-}
-
 constexpr int kDecWaves = 4;
 
 // grid (T, H), kDecWaves waves per (token, query head). Keys are walked in
@@ -386,10 +350,6 @@ __global__ __launch_bounds__(kDecWaves * WAVE) void masked_paged_attention_kerne
   }
 }
 
-typedef __attribute__((ext_vector_type(4))) short bf16x4;
-typedef __attribute__((ext_vector_type(4))) float f32x4;
-
-
 // Prompt portions on the matrix cores (bf16, key and value sizes multiples
 // of 16). grid (query tiles, H), one wave per 16 consecutive
 // queries of a run and one query head. Per 16-key tile:
@@ -514,84 +474,7 @@ __global__ __launch_bounds__(WAVE) void masked_prefill_mfma_kernel(
   }
 }
 
-// two fp32 -> packed bf16 pair (round to nearest even), low half first; a
-// conversion the compiler knows, so that it keeps the wait states between an
-// exponential and its reader
-typedef __attribute__((ext_vector_type(2))) float f32x2;
-typedef __attribute__((ext_vector_type(2))) __bf16 bf16x2;
-DEV_INLINE uint32_t cvt_pk_bf16(float a, float b) {
-  return __builtin_bit_cast(uint32_t, __builtin_convertvector((f32x2){a, b}, bf16x2));
-}
-
-// max over the four lanes 16 apart that share a lane column
-DEV_INLINE float column_max(float x, int lane) {
-  auto from = [&](float v, int src) {
-    return __builtin_bit_cast(
-        float, __builtin_amdgcn_ds_bpermute(src * 4, __builtin_bit_cast(int, v)));
-  };
-  x = fmaxf(x, from(x, lane ^ 16));
-  return fmaxf(x, from(x, lane ^ 32));
-}
-
-constexpr int kKT = 32;    // keys of a tile
-constexpr int kRPad = 8;   // padding of a staged row (elements)
-
-typedef __attribute__((ext_vector_type(8))) short bf16x8;
-
-// A 16 x 16 piece of a row-major LDS tile, transposed on the way to the
-// registers: p points at (row r0 + (lane & 15) / 4 + 4 * (lane >> 4), column
-// c0 + 4 * (lane & 3)); the lane receives rows r0 + 4 * (lane >> 4) + 0..3 of
-// column c0 + (lane & 15).
-DEV_INLINE bf16x4 lds_read_transposed(const bf16raw* p) {
-  return __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-      (__attribute__((address_space(3))) bf16x4*)p);
-}
-
-// K Q^T over 16 (four slots a lane) or 32 (eight slots) key dims
-DEV_INLINE f32x4 mfma_qk(bf16x4 k, bf16x4 q, f32x4 c) {
-  return __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(k, q, c, 0, 0, 0);
-}
-DEV_INLINE f32x4 mfma_qk(bf16x8 k, bf16x8 q, f32x4 c) {
-  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, q, c, 0, 0, 0);
-}
-
-template <bool kWide> struct QkFrag {  // one lane's share of a row step
-  typedef bf16x4 type;
-  static constexpr int kDims = 16, kElems = 4;
-};
-template <> struct QkFrag<true> {
-  typedef bf16x8 type;
-  static constexpr int kDims = 32, kElems = 8;
-};
-
-// Scores of a lane's eight keys of a 32-key tile (keys sub * 16 + grp * 4 + i,
-// e = sub * 4 + i) in the base-2 domain, so that every exponential is one
-// v_exp_f32: scale and key scale, cap, bias. rel0 = (first key - query) of the
-// lane: sub 0, i 0. kcv: the tile's key scales in LDS at the lane's keys, or
-// null.
-DEV_INLINE void base2_scores(const f32x4* sacc, const AttnArgs& a, float slope2,
-                             float cap2, float rel0, const float* kcv, float* sc) {
-  const float c = cap2 > 0.f ? a.scale * (2.f * kLog2e) / a.softcap : a.scale * kLog2e;
-  if (kcv != nullptr) {
-    const float4 k0 = *(const float4*)kcv, k1 = *(const float4*)(kcv + 16);
-    sc[0] = sacc[0][0] * (c * k0.x); sc[1] = sacc[0][1] * (c * k0.y);
-    sc[2] = sacc[0][2] * (c * k0.z); sc[3] = sacc[0][3] * (c * k0.w);
-    sc[4] = sacc[1][0] * (c * k1.x); sc[5] = sacc[1][1] * (c * k1.y);
-    sc[6] = sacc[1][2] * (c * k1.z); sc[7] = sacc[1][3] * (c * k1.w);
-  } else {
-#pragma unroll
-    for (int e = 0; e < 8; ++e) sc[e] = sacc[e >> 2][e & 3] * c;
-  }
-  if (cap2 > 0.f) {
-#pragma unroll
-    for (int e = 0; e < 8; ++e) sc[e] = cap_base2(sc[e], cap2);
-  }
-  if (slope2 != 0.f) {
-    const float b = slope2 * rel0;
-#pragma unroll
-    for (int e = 0; e < 8; ++e) sc[e] += b + slope2 * (float)((e >> 2) * 16 + (e & 3));
-  }
-}
+constexpr int kPrefillThreads = 512;
 
 // Prompt portions on the matrix cores with the key / value tiles shared
 // through LDS. A block of HW * QW waves covers QW * 16 consecutive queries of
@@ -606,9 +489,11 @@ DEV_INLINE void base2_scores(const f32x4* sacc, const AttnArgs& a, float slope2,
 // contracts all 32 keys of a tile in one v_mfma_f32_16x16x32_bf16 per 16 value
 // dims (a lane's eight contraction slots are keys grp*4 + 0..3 and
 // 16 + grp*4 + 0..3, for P and V alike), and so does K Q^T over 32 key dims
-// when the key size allows (kWideQK). Statistics are fp32, base 2.
-template <int kMaxDSteps, int kMaxDvTiles, bool kWideQK, bool kTied>
-__global__ __launch_bounds__(512) void masked_prefill_mfma_shared_kernel(
+// when the key size allows (kWideQK). Statistics are fp32, base 2. kExact: the
+// sizes are D = 16 kMaxDSteps, Dv = 16 kMaxDvTiles and the block size is a
+// power of two; otherwise the template sizes are bounds and steps are guarded.
+template <int kMaxDSteps, int kMaxDvTiles, bool kWideQK, bool kTied, bool kExact>
+__global__ __launch_bounds__(kPrefillThreads) void masked_prefill_mfma_shared_kernel(
     bf16raw* __restrict__ out, int64_t out_stride, const bf16raw* __restrict__ q,
     int64_t q_stride, const bf16raw* __restrict__ k_cache,
     const bf16raw* __restrict__ v_cache, const int* __restrict__ block_tables,
@@ -618,10 +503,12 @@ __global__ __launch_bounds__(512) void masked_prefill_mfma_shared_kernel(
   typedef QkFrag<kWideQK> Frag;
   typedef typename Frag::type frag_t;
   constexpr int kNF = kMaxDSteps * 16 / Frag::kDims;
-  constexpr int kKVec = kKT * kMaxDSteps * 16 / 8 / 256;   // per thread, 256 threads
-  constexpr int kVVec = kTied ? 1 : kKT * kMaxDvTiles * 16 / 8 / 256;
-  const int G = a.G, D = a.D, Dv = a.Dv, bs = a.bs;
-  const int nthr = blockDim.x;
+  // 16-byte pieces of a tile per thread
+  constexpr int nthr = kPrefillThreads;
+  constexpr int kKVec = (kKT * kMaxDSteps * 2 + nthr - 1) / nthr;
+  constexpr int kVVec = kTied ? 1 : (kKT * kMaxDvTiles * 2 + nthr - 1) / nthr;
+  const int G = a.G;
+  const int D = kExact ? kMaxDSteps * 16 : a.D, Dv = kExact ? kMaxDvTiles * 16 : a.Dv;
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int col = lane & 15, grp = lane >> 4;
   const int hw = wave % HW, qw = wave / HW;
@@ -654,14 +541,13 @@ __global__ __launch_bounds__(512) void masked_prefill_mfma_shared_kernel(
   const int k_elems = kKT * krow, v_elems = kTied ? 0 : kKT * vrow;
   const int buf_elems = k_elems + v_elems + 2 * kKT;  // + key scales (fp32)
   const int kcpr = D / 8, vcpr = Dv / 8;  // 16-byte chunks per cached row
-  const float slope2 = a.slopes != nullptr ? a.slopes[h] * kLog2e : 0.f;
-  const float cap2 = a.softcap * kLog2e;
+  const ScoreConsts consts(a, h);
 
   frag_t qf[kNF];
   const bf16raw* qrow = q + (size_t)tq * q_stride + h * D;
 #pragma unroll
   for (int f = 0; f < kNF; ++f)
-    if (f < nf) {
+    if (kExact || f < nf) {
       const bf16raw* p = qrow + f * Frag::kDims + grp * Frag::kElems;
       if constexpr (kWideQK) {
         const bf16x4 x = *(const bf16x4*)p, y = *(const bf16x4*)(p + 4);
@@ -681,16 +567,25 @@ __global__ __launch_bounds__(512) void masked_prefill_mfma_shared_kernel(
     return it < n_kept ? it * kKT : blo + (it - n_kept) * kKT;
   };
   auto last_key = [&](int it) { return it < n_kept ? kept - 1 : bpos_max; };
+  auto cached_at = [&](int j, int64_t* blk, int* off) {
+    *blk = bt[kExact ? j >> a.bs_shift : j / a.bs];
+    *off = kExact ? j & (a.bs - 1) : j % a.bs;
+  };
   auto load_tile = [&](int it) {
     const int j0 = first_key(it), j_end = last_key(it);
+    int64_t blk;
+    int off;
+    if (a.kscale != nullptr && threadIdx.x < kKT) {
+      cached_at(min(j0 + (int)threadIdx.x, j_end), &blk, &off);
+      kscr = a.kscale[blk * a.bs + off];
+    }
 #pragma unroll
     for (int i = 0; i < kKVec; ++i) {
       const int v = i * nthr + threadIdx.x;
       const int row = v / kcpr, c = v % kcpr;
       if (row < kKT) {
-        const int j = min(j0 + row, j_end);
-        kreg[i] = *(const uint4*)(k_cache +
-            (((int64_t)bt[j / bs] * G + g) * bs + j % bs) * D + c * 8);
+        cached_at(min(j0 + row, j_end), &blk, &off);
+        kreg[i] = *(const uint4*)(k_cache + ((blk * G + g) * a.bs + off) * D + c * 8);
       }
     }
     if constexpr (!kTied) {
@@ -699,16 +594,11 @@ __global__ __launch_bounds__(512) void masked_prefill_mfma_shared_kernel(
         const int v = i * nthr + threadIdx.x;
         const int row = v / vcpr, c = v % vcpr;
         if (row < kKT) {
-          const int j = min(j0 + row, j_end);
+          cached_at(min(j0 + row, j_end), &blk, &off);
           vreg[i] = *(const uint4*)(v_cache +
-              (((int64_t)bt[j / bs] * (G / a.kvs) + g / a.kvs) * bs + j % bs) * a.v_rs +
-              c * 8);
+              ((blk * (G / a.kvs) + g / a.kvs) * a.bs + off) * a.v_rs + c * 8);
         }
       }
-    }
-    if (a.kscale != nullptr && threadIdx.x < kKT) {
-      const int j = min(j0 + (int)threadIdx.x, j_end);
-      kscr = a.kscale[(int64_t)bt[j / bs] * bs + j % bs];
     }
   };
   auto store_tile = [&](int buf) {
@@ -746,19 +636,19 @@ __global__ __launch_bounds__(512) void masked_prefill_mfma_shared_kernel(
     // wave-uniform: something of this tile is visible to the wave's queries
     if (wave_on && j0 <= wpos_max && (j0 + kKT - 1 >= wlo || j0 < a.keep)) {
       f32x4 sacc[2];
+      sacc[0] = sacc[1] = (f32x4){0.f, 0.f, 0.f, 0.f};
+      const bf16raw* kp = ks_ + col * krow + grp * Frag::kElems;
 #pragma unroll
-      for (int sub = 0; sub < 2; ++sub) {
-        sacc[sub] = (f32x4){0.f, 0.f, 0.f, 0.f};
-        const bf16raw* kp = ks_ + (sub * 16 + col) * krow + grp * Frag::kElems;
-#pragma unroll
-        for (int f = 0; f < kNF; ++f)
-          if (f < nf)
-            sacc[sub] = mfma_qk(*(const frag_t*)(kp + f * Frag::kDims), qf[f], sacc[sub]);
-      }
+      for (int f = 0; f < kNF; ++f)
+        if (kExact || f < nf) {
+          sacc[0] = mfma_qk(*(const frag_t*)(kp + f * Frag::kDims), qf[f], sacc[0]);
+          sacc[1] = mfma_qk(*(const frag_t*)(kp + 16 * krow + f * Frag::kDims), qf[f],
+                            sacc[1]);
+        }
       // this lane: query `col`, keys j0 + sub * 16 + grp * 4 + i
       float sc[8];
-      base2_scores(sacc, a, slope2, cap2, (float)(j0 + grp * 4 - pos_q),
-                   a.kscale != nullptr ? kc_ + grp * 4 : nullptr, sc);
+      base2_scores<true>(sacc, consts, (float)(j0 + grp * 4 - pos_q),
+                         a.kscale != nullptr ? kc_ + grp * 4 : nullptr, sc);
       // wave-uniform: a tile whose keys all queries see needs no mask. (Masks
       // are selects: hipcc 7.2 has lost such an assignment from under a branch.)
       const int jl = j0 + grp * 4;
@@ -800,7 +690,7 @@ __global__ __launch_bounds__(512) void masked_prefill_mfma_shared_kernel(
       const bf16raw* vp = vs_ + (grp * 4 + (col >> 2)) * vrow + (col & 3) * 4;
 #pragma unroll
       for (int dt = 0; dt < kMaxDvTiles; ++dt) {
-        if (dt < ndt) {
+        if (kExact || dt < ndt) {
           const bf16x4 v0 = lds_read_transposed(vp + dt * 16);
           const bf16x4 v1 = lds_read_transposed(vp + dt * 16 + 16 * vrow);
           const bf16x8 vf = (bf16x8){v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
@@ -821,7 +711,7 @@ __global__ __launch_bounds__(512) void masked_prefill_mfma_shared_kernel(
     bf16raw* op = out + (size_t)tq * out_stride + h * Dv + grp * 4;
 #pragma unroll
     for (int dt = 0; dt < kMaxDvTiles; ++dt) {
-      if (dt < ndt) {
+      if (kExact || dt < ndt) {
         ushort4 o4;
         o4.x = f32_to_bf16(oacc[dt][0] * inv);
         o4.y = f32_to_bf16(oacc[dt][1] * inv);
@@ -830,252 +720,6 @@ __global__ __launch_bounds__(512) void masked_prefill_mfma_shared_kernel(
         *(ushort4*)(op + dt * 16) = o4;
       }
     }
-  }
-}
-
-constexpr int kDW = 4;  // waves of a decode block; each takes every fourth key tile
-
-// bytes of a decode wave's staging region: a 32-row value tile + key scales
-static inline __host__ __device__ int decode_stage_bytes(int Dv) {
-  return kKT * (Dv + kRPad) * (int)sizeof(bf16raw) + kKT * (int)sizeof(float);
-}
-
-// Single decode tokens on the matrix cores, bf16. grid (T, G, ceil(rep / 16) *
-// splits): the 16 rows of an MFMA tile are the query heads that share one
-// key/value head (all heads of a latent layer, the group of a grouped layer),
-// so a key or value row is loaded once for all of them. The visible keys are
-// numbered through (kept first tokens, then the window) and cut into 32-key
-// tiles; the four waves walk disjoint tiles. A lane loads its pieces of two
-// rows per tile straight as MFMA operands, one tile ahead; the value part
-// (kTied: the same registers) is written to a wave-private LDS tile and comes
-// back through the transposing LDS read. Statistics are fp32 in the base-2
-// domain, and the waves' partial results are joined through LDS.
-template <int kMaxDSteps, int kMaxDvTiles, bool kWide, bool kTied>
-__global__ __launch_bounds__(kDW * WAVE) void masked_decode_mfma_kernel(
-    bf16raw* __restrict__ out, int64_t out_stride, const bf16raw* __restrict__ q,
-    int64_t q_stride, const bf16raw* __restrict__ k_cache,
-    const bf16raw* __restrict__ v_cache, const int* __restrict__ block_tables,
-    int max_blocks, const int* __restrict__ token_seq,
-    const int* __restrict__ positions, int n_split, float* __restrict__ part_o,
-    float* __restrict__ part_ml, AttnArgs a) {
-  extern __shared__ __attribute__((aligned(16))) char smem[];
-  typedef QkFrag<kWide> Frag;
-  typedef typename Frag::type frag_t;
-  constexpr int kNF = kMaxDSteps * 16 / Frag::kDims;
-  constexpr int kNV = kMaxDvTiles * 16 / Frag::kDims;
-  const int H = a.H, G = a.G, D = a.D, Dv = a.Dv, bs = a.bs;
-  const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
-  const int col = lane & 15, grp = lane >> 4;
-  const int t = blockIdx.x, g = blockIdx.y, rep = H / G;
-  const int zt = blockIdx.z / n_split, sp = blockIdx.z % n_split;
-  const int h0 = g * rep + zt * 16;
-  const int nh = min(16, (g + 1) * rep - h0);
-  const int pos = positions[t];
-  const int* bt = block_tables + (size_t)token_seq[t] * max_blocks;
-  const int lo = a.lower(pos), kept = a.kept(lo), n_keys = kept + pos - lo + 1;
-  const int nf = D / Frag::kDims, nv = Dv / Frag::kDims, ndt = Dv / 16;
-  const int vrow = Dv + kRPad;
-  bf16raw* vt = (bf16raw*)(smem + (size_t)wave * decode_stage_bytes(Dv));
-  float* kc = (float*)(vt + kKT * vrow);
-  const int hq = h0 + min(col, nh - 1);
-  const float slope2 = a.slopes != nullptr ? a.slopes[hq] * kLog2e : 0.f;
-  const float cap2 = a.softcap * kLog2e;
-  frag_t qf[kNF];
-#pragma unroll
-  for (int f = 0; f < kNF; ++f)
-    if (f < nf) {
-      const bf16raw* p =
-          q + (size_t)t * q_stride + (size_t)hq * D + f * Frag::kDims + grp * Frag::kElems;
-      if constexpr (kWide) {
-        const bf16x4 x = *(const bf16x4*)p, y = *(const bf16x4*)(p + 4);
-        qf[f] = (bf16x8){x[0], x[1], x[2], x[3], y[0], y[1], y[2], y[3]};
-      } else {
-        qf[f] = *(const bf16x4*)p;
-      }
-    }
-  f32x4 oacc[kMaxDvTiles];
-#pragma unroll
-  for (int dt = 0; dt < kMaxDvTiles; ++dt) oacc[dt] = (f32x4){0.f, 0.f, 0.f, 0.f};
-  float m = -INFINITY, l = 0.f;
-  // the tiles dealt to the splits in contiguous shares
-  const int n_tiles = (n_keys + kKT - 1) / kKT;
-  const int per_split = (n_tiles + n_split - 1) / n_split;
-  const int tile_end = min(n_tiles, (sp + 1) * per_split);
-  int jn[2], bn[2];  // the lane's two keys of the tile to load, and their blocks
-  frag_t kf[2][kNF], vf[2][kTied ? 1 : kNV];
-  float ksr[2] = {0.f, 0.f};
-  auto find_rows = [&](int tile) {
-#pragma unroll
-    for (int sub = 0; sub < 2; ++sub) {
-      const int v = min(tile * kKT + sub * 16 + col, n_keys - 1);
-      jn[sub] = v < kept ? v : lo + v - kept;
-      bn[sub] = bt[jn[sub] / bs];
-    }
-  };
-  auto load_rows = [&]() {
-#pragma unroll
-    for (int sub = 0; sub < 2; ++sub) {
-      const int off = jn[sub] % bs;
-      const bf16raw* kp =
-          k_cache + (((int64_t)bn[sub] * G + g) * bs + off) * D + grp * Frag::kElems;
-#pragma unroll
-      for (int f = 0; f < kNF; ++f)
-        if (f < nf) kf[sub][f] = *(const frag_t*)(kp + f * Frag::kDims);
-      if constexpr (!kTied) {
-        const bf16raw* vp = v_cache +
-            (((int64_t)bn[sub] * (G / a.kvs) + g / a.kvs) * bs + off) * a.v_rs +
-            grp * Frag::kElems;
-#pragma unroll
-        for (int f = 0; f < kNV; ++f)
-          if (f < nv) vf[sub][f] = *(const frag_t*)(vp + f * Frag::kDims);
-      }
-      if (a.kscale != nullptr) ksr[sub] = a.kscale[(int64_t)bn[sub] * bs + off];
-    }
-  };
-  int tile = sp * per_split + wave;
-  if (tile < tile_end) {
-    find_rows(tile);
-    load_rows();
-    if (tile + kDW < tile_end) find_rows(tile + kDW);
-  }
-  for (; tile < tile_end; tile += kDW) {
-    f32x4 sacc[2];
-#pragma unroll
-    for (int sub = 0; sub < 2; ++sub) {
-      bf16raw* vw = vt + (sub * 16 + col) * vrow + grp * Frag::kElems;
-#pragma unroll
-      for (int f = 0; f < kNV; ++f)
-        if (f < nv) *(frag_t*)(vw + f * Frag::kDims) = kTied ? kf[sub][f] : vf[sub][kTied ? 0 : f];
-      if (a.kscale != nullptr && grp == 0) kc[sub * 16 + col] = ksr[sub];
-      sacc[sub] = (f32x4){0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int f = 0; f < kNF; ++f)
-        if (f < nf) sacc[sub] = mfma_qk(kf[sub][f], qf[f], sacc[sub]);
-    }
-    if (tile + kDW < tile_end) {
-      load_rows();
-      if (tile + 2 * kDW < tile_end) find_rows(tile + 2 * kDW);
-    }
-    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-    __builtin_amdgcn_wave_barrier();
-    // this lane: head `col`, keys v0 + sub * 16 + grp * 4 + i of the numbering
-    const int v0 = tile * kKT;
-    float sc[8];
-    if (v0 >= kept || v0 + kKT <= kept) {  // one stretch of positions
-      const int j0 = v0 < kept ? v0 : lo + v0 - kept;
-      base2_scores(sacc, a, slope2, cap2, (float)(j0 + grp * 4 - pos),
-                   a.kscale != nullptr ? kc + grp * 4 : nullptr, sc);
-    } else {
-      base2_scores(sacc, a, 0.f, cap2, 0.f,
-                   a.kscale != nullptr ? kc + grp * 4 : nullptr, sc);
-#pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        const int v = v0 + (e >> 2) * 16 + grp * 4 + (e & 3);
-        sc[e] += slope2 * (float)((v < kept ? v : lo + v - kept) - pos);
-      }
-    }
-    if (v0 + kKT > n_keys) {
-#pragma unroll
-      for (int e = 0; e < 8; ++e)
-        sc[e] = v0 + (e >> 2) * 16 + grp * 4 + (e & 3) < n_keys ? sc[e] : -INFINITY;
-    }
-    float mt = sc[0];
-#pragma unroll
-    for (int e = 1; e < 8; ++e) mt = fmaxf(mt, sc[e]);
-    mt = column_max(mt, lane);
-    const float m_new = fmaxf(m, mt);  // finite: the tile's first key is visible
-    const float corr = __builtin_amdgcn_exp2f(m - m_new);
-    float pv[8];
-    float ps = 0.f;
-#pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      pv[e] = __builtin_amdgcn_exp2f(sc[e] - m_new);
-      ps += pv[e];
-    }
-    union { bf16x8 v; uint32_t u[4]; } pk;
-#pragma unroll
-    for (int e = 0; e < 4; ++e) pk.u[e] = cvt_pk_bf16(pv[2 * e], pv[2 * e + 1]);
-    l = l * corr + ps;
-    m = m_new;
-    const bf16raw* vp = vt + (grp * 4 + (col >> 2)) * vrow + (col & 3) * 4;
-#pragma unroll
-    for (int dt = 0; dt < kMaxDvTiles; ++dt) {
-      if (dt < ndt) {
-        const bf16x4 v0t = lds_read_transposed(vp + dt * 16);
-        const bf16x4 v1t = lds_read_transposed(vp + dt * 16 + 16 * vrow);
-        const bf16x8 vfr = (bf16x8){v0t[0], v0t[1], v0t[2], v0t[3],
-                                    v1t[0], v1t[1], v1t[2], v1t[3]};
-        f32x4 o = oacc[dt];
-        o[0] *= corr; o[1] *= corr; o[2] *= corr; o[3] *= corr;
-        oacc[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vfr, pk.v, o, 0, 0, 0);
-      }
-    }
-    // all lanes read the tile before it is rewritten
-    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-    __builtin_amdgcn_wave_barrier();
-  }
-  l += __shfl_xor(l, 16, WAVE);
-  l += __shfl_xor(l, 32, WAVE);
-  __syncthreads();  // the staging regions are reused for the join
-  float* cm = (float*)smem;            // [waves][16] running max (base 2)
-  float* cl = cm + kDW * 16;           // [waves][16] sums
-  float* co = cl + kDW * 16;           // [waves][16][Dv] unnormalised outputs
-  if (grp == 0) {
-    cm[wave * 16 + col] = m;
-    cl[wave * 16 + col] = l;
-  }
-#pragma unroll
-  for (int dt = 0; dt < kMaxDvTiles; ++dt)
-    if (dt < ndt)
-      *(f32x4*)(co + ((size_t)wave * 16 + col) * Dv + dt * 16 + grp * 4) = oacc[dt];
-  __syncthreads();
-  for (int idx = threadIdx.x; idx < nh * Dv; idx += blockDim.x) {
-    const int hh = idx / Dv, d = idx % Dv;
-    float mx = -INFINITY;
-    for (int w = 0; w < kDW; ++w) mx = fmaxf(mx, cm[w * 16 + hh]);
-    float lsum = 0.f, x = 0.f;
-    for (int w = 0; w < kDW; ++w) {
-      const float mw = cm[w * 16 + hh];
-      const float wsc = mw == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(mw - mx);
-      lsum += cl[w * 16 + hh] * wsc;
-      x += co[((size_t)w * 16 + hh) * Dv + d] * wsc;
-    }
-    if (n_split == 1) {
-      if (a.sink != nullptr) lsum += __builtin_amdgcn_exp2f(a.sink[h0 + hh] * kLog2e - mx);
-      stf(out + (size_t)t * out_stride + (h0 + hh) * Dv + d, x * a.out_scale / lsum);
-    } else {
-      // partial result of this split: [t][head][split] -> (max, sum), values
-      const size_t row = ((size_t)t * H + h0 + hh) * n_split + sp;
-      part_o[row * Dv + d] = x;
-      if (d == 0) {
-        part_ml[row * 2] = mx;
-        part_ml[row * 2 + 1] = lsum;
-      }
-    }
-  }
-}
-
-// Join of the key splits of masked_decode_mfma_kernel: grid (T, H).
-__global__ void decode_split_join_kernel(bf16raw* __restrict__ out, int64_t out_stride,
-                                         const float* __restrict__ part_o,
-                                         const float* __restrict__ part_ml, int H,
-                                         int Dv, int n_split, float out_scale,
-                                         const float* __restrict__ sink) {
-  const int t = blockIdx.x, h = blockIdx.y;
-  const size_t row0 = ((size_t)t * H + h) * n_split;
-  float mx = -INFINITY;
-  for (int s = 0; s < n_split; ++s) mx = fmaxf(mx, part_ml[(row0 + s) * 2]);
-  for (int d = threadIdx.x; d < Dv; d += blockDim.x) {
-    float lsum = 0.f, a = 0.f;
-    for (int s = 0; s < n_split; ++s) {
-      const float ms = part_ml[(row0 + s) * 2];
-      if (ms == -INFINITY) continue;  // a split without keys wrote nothing usable
-      const float w = __builtin_amdgcn_exp2f(ms - mx);
-      lsum += part_ml[(row0 + s) * 2 + 1] * w;
-      a += part_o[(row0 + s) * Dv + d] * w;
-    }
-    if (sink != nullptr) lsum += __builtin_amdgcn_exp2f(sink[h] * kLog2e - mx);
-    stf(out + (size_t)t * out_stride + h * Dv + d, a * out_scale / lsum);
   }
 }
 
@@ -1262,6 +906,9 @@ void masked_paged_attention(torch::Tensor out, torch::Tensor q,
   args.keep = (int)keep_first;
   args.v_rs = v_rs;
   args.H = H; args.G = G; args.D = D; args.Dv = Dv; args.bs = bs; args.kvs = kvs;
+  args.bs_shift = -1;
+  for (int i = 0; i < 20; ++i)
+    if (bs == 1 << i) args.bs_shift = i;
   // one row per token and head that is key and (its leading part) value
   const bool tied = v_cache.data_ptr() == k_cache.data_ptr() && kvs == 1 && v_rs == D &&
                     Dv <= D;
@@ -1304,7 +951,7 @@ void masked_paged_attention(torch::Tensor out, torch::Tensor q,
       const int rep = H / G;
       int HW = 1;
       while (HW * 2 <= rep && HW < 8) HW *= 2;
-      const int WPB = 8;
+      constexpr int WPB = kPrefillThreads / WAVE;
       const int QW = WPB / HW;
       const int btiles = T / (QW * 16) + n_seq;
       const int zb = (rep + HW - 1) / HW;
@@ -1320,23 +967,32 @@ void masked_paged_attention(torch::Tensor out, torch::Tensor q,
                          (int)block_tables.size(1), (const int*)start_loc.data_ptr(),
                          (const int*)positions.data_ptr(), n_seq, HW, QW, args);
       };
-      // key sizes above 128 (a latent with a rotated part behind it) keep
-      // twice as many query fragments in registers
-      auto pick = [&](auto wide, auto is_tied) {
-        constexpr bool kW = decltype(wide)::value, kT = decltype(is_tied)::value;
-        if (D <= 128 && Dv <= 128)
-          launch_shared(masked_prefill_mfma_shared_kernel<8, 8, kW, kT>);
-        else if (D <= 128)
-          launch_shared(masked_prefill_mfma_shared_kernel<8, 16, kW, kT>);
-        else launch_shared(masked_prefill_mfma_shared_kernel<16, 16, kW, kT>);
+      auto sized = [&](auto is_tied) {
+        constexpr bool kT = decltype(is_tied)::value;
+        const bool shift = args.bs_shift >= 0, wide = D % 32 == 0;
+        if (shift && D == 128 && Dv == 128)
+          launch_shared(masked_prefill_mfma_shared_kernel<8, 8, true, kT, true>);
+        else if (shift && D == 64 && Dv == 64)
+          launch_shared(masked_prefill_mfma_shared_kernel<4, 4, true, kT, true>);
+        else if (shift && !kT && D == 64 && Dv == 128)
+          launch_shared(masked_prefill_mfma_shared_kernel<4, 8, true, false, true>);
+        else if (shift && kT && D == 192 && Dv == 128)
+          launch_shared(masked_prefill_mfma_shared_kernel<12, 8, true, true, true>);
+        else if (D <= 128 && Dv <= 128 && wide)
+          launch_shared(masked_prefill_mfma_shared_kernel<8, 8, true, kT, false>);
+        else if (D <= 128 && Dv <= 128)
+          launch_shared(masked_prefill_mfma_shared_kernel<8, 8, false, kT, false>);
+        // larger keys (a latent with a rotated part behind it) or values keep
+        // more fragments in registers
+        else if (D <= 128 && wide)
+          launch_shared(masked_prefill_mfma_shared_kernel<8, 16, true, kT, false>);
+        else if (wide)
+          launch_shared(masked_prefill_mfma_shared_kernel<16, 16, true, kT, false>);
+        else
+          launch_shared(masked_prefill_mfma_shared_kernel<16, 16, false, kT, false>);
       };
-      if (D % 32 == 0) {
-        if (tied) pick(std::true_type{}, std::true_type{});
-        else pick(std::true_type{}, std::false_type{});
-      } else {
-        if (tied) pick(std::false_type{}, std::true_type{});
-        else pick(std::false_type{}, std::false_type{});
-      }
+      if (tied) sized(std::true_type{});
+      else sized(std::false_type{});
     } else if (D <= 128 && Dv <= 256) {
       launch(masked_prefill_mfma_kernel<8, 16>);
     } else {
@@ -1345,70 +1001,10 @@ void masked_paged_attention(torch::Tensor out, torch::Tensor q,
     SEQ_CHECK_LAUNCH();
     return;
   }
-  // worth it when several heads share a key row (measured at 64 sequences of
-  // 1536 tokens: 16 heads on one latent 60 -> 28 us per call; groups of 4 with
-  // 128-wide keys 89 -> 65 us, with two 64-wide score maps per value head
-  // 132 -> 93 us)
-  if (q.scalar_type() == torch::kBFloat16 && max_len == 1 && H / G >= 4 && D % 16 == 0 &&
-      Dv % 16 == 0 && D <= 256 && Dv <= 128 && al8(q) && v_rs % 8 == 0 &&
-      ((size_t)k_cache.data_ptr()) % 16 == 0 && ((size_t)v_cache.data_ptr()) % 16 == 0) {
-    // decode tokens: the heads of a key/value group are the rows of a tile
-    const int rep = H / G, zb = (rep + 15) / 16;
-    const size_t stage = (size_t)kDW * decode_stage_bytes(Dv);
-    const size_t join = (size_t)kDW * (32 + 16 * Dv) * sizeof(float);
-    // split the keys over blocks so that a wave walks about two tiles at the
-    // longest context the block tables can describe; splits beyond a
-    // sequence's keys exit at once
-    int64_t cap = (int64_t)block_tables.size(1) * bs;
-    if (window > 0) cap = std::min(cap, window + keep_first);
-    if (chunk > 0) cap = std::min(cap, chunk);
-    int n_split = (int)std::min<int64_t>(16, std::max<int64_t>(1, (cap + 255) / 256));
-    // past about eight blocks a CU more splits only add joins (64 sequences of
-    // 1536 tokens on 8 key heads: 144 us with 16 splits, 91 us with 4)
-    while (n_split > 1 && (int64_t)T * G * zb * n_split > 2048) n_split /= 2;
-    TORCH_CHECK(G <= 65535 && (int64_t)zb * n_split <= 65535);
-    torch::Tensor part_o, part_ml;
-    if (n_split > 1) {
-      auto f32 = torch::TensorOptions().dtype(torch::kFloat32).device(q.device());
-      part_o = torch::empty({(int64_t)T * H * n_split, Dv}, f32);
-      part_ml = torch::empty({(int64_t)T * H * n_split, 2}, f32);
-    }
-    auto launch = [&](auto kern) {
-      hipLaunchKernelGGL(kern, dim3(T, G, zb * n_split), dim3(kDW * WAVE),
-                         stage > join ? stage : join, SEQ_STREAM(),
-                         (bf16raw*)out.data_ptr(), out.stride(0),
-                         (const bf16raw*)q.data_ptr(), q.stride(0),
-                         (const bf16raw*)k_cache.data_ptr(),
-                         (const bf16raw*)v_cache.data_ptr(),
-                         (const int*)block_tables.data_ptr(), (int)block_tables.size(1),
-                         (const int*)token_seq.data_ptr(),
-                         (const int*)positions.data_ptr(), n_split,
-                         n_split > 1 ? (float*)part_o.data_ptr() : nullptr,
-                         n_split > 1 ? (float*)part_ml.data_ptr() : nullptr, args);
-    };
-    auto pick = [&](auto wide, auto is_tied) {
-      constexpr bool kW = decltype(wide)::value, kT = decltype(is_tied)::value;
-      if (D <= 128) launch(masked_decode_mfma_kernel<8, 8, kW, kT>);
-      else launch(masked_decode_mfma_kernel<16, 8, kW, kT>);
-    };
-    if (D % 32 == 0 && Dv % 32 == 0) {
-      if (tied) pick(std::true_type{}, std::true_type{});
-      else pick(std::true_type{}, std::false_type{});
-    } else {
-      if (tied) pick(std::false_type{}, std::true_type{});
-      else pick(std::false_type{}, std::false_type{});
-    }
-    if (n_split > 1) {
-      SEQ_CHECK_LAUNCH();
-      hipLaunchKernelGGL(decode_split_join_kernel, dim3(T, H), dim3(64), 0, SEQ_STREAM(),
-                         (bf16raw*)out.data_ptr(), out.stride(0),
-                         (const float*)part_o.data_ptr(),
-                         (const float*)part_ml.data_ptr(), H, (int)Dv, n_split,
-                         (float)out_scale, args.sink);
-    }
-    SEQ_CHECK_LAUNCH();
+  if (q.scalar_type() == torch::kBFloat16 && max_len == 1 && al8(q) &&
+      masked_decode_mfma(out, q, k_cache, v_cache, block_tables, token_seq, positions, args,
+                         tied))
     return;
-  }
   SEQ_DISPATCH_ACT(q, {
     constexpr int N = Vec16<act_t>::N;
     // 16-byte row loads need whole vectors per key / value row and at most
