@@ -88,6 +88,13 @@ void latent_rope_to_cache(torch::Tensor cache, torch::Tensor x, torch::Tensor we
 void router_scores_topk(torch::Tensor logits, c10::optional<torch::Tensor> bias,
                         torch::Tensor dense, torch::Tensor weights,
                         torch::Tensor index, double scale, int64_t score);
+void route_tokens(torch::Tensor h, torch::Tensor router, c10::optional<torch::Tensor> bias,
+                  torch::Tensor dense, torch::Tensor weights, torch::Tensor index,
+                  c10::optional<torch::Tensor> extra, double scale, int64_t score);
+void expert_order(torch::Tensor index, torch::Tensor weights, torch::Tensor tok,
+                  torch::Tensor wrow, torch::Tensor place, torch::Tensor counts);
+void combine_expert_rows(torch::Tensor out, torch::Tensor y, torch::Tensor place,
+                         c10::optional<torch::Tensor> shared);
 void glu_weighted(torch::Tensor out, torch::Tensor gu, c10::optional<torch::Tensor> w,
                   int64_t group, double alpha, double limit, double up_shift,
                   bool w_sigmoid, bool w_input);
@@ -151,6 +158,11 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "latent RMS norm + rotated shared key part into a paged cache, query rotation");
   m.def("router_scores_topk", &router_scores_topk,
         "softmax scores, biased top-k choice, unnormalised score weights");
+  m.def("route_tokens", &route_tokens,
+        "router product, scores, biased top-k choice, unnormalised score weights");
+  m.def("expert_order", &expert_order, "stable sort of (token, choice) pairs by expert");
+  m.def("combine_expert_rows", &combine_expert_rows,
+        "sum of a token's expert rows and the shared expert's");
   m.def("glu_weighted", &glu_weighted,
         "clamped gate * sigmoid(alpha gate) * (up + shift) times a per-row, per-expert weight");
   m.def("embed_sinusoid", &embed_sinusoid,

@@ -594,6 +594,27 @@ class GeluMLP(nn.Module):
         return self.down(sops.gelu(self.up(h)))
 
 
+class ExpertRows:
+    """The tokens of a large step gathered by expert: rows of one buffer, so
+    that everything but the products themselves is one launch for all
+    experts. The row counts come to the host (the products need shapes)."""
+
+    def __init__(self, h, index, weights, experts: int):
+        tok, self.weight, self.place, counts = sops.expert_order(index, weights, experts)
+        self.h = h.index_select(0, tok)
+        self.counts = counts.tolist()
+
+    def products(self, x, weight_of, n_out: int):
+        """x's rows of expert e times weight_of(e) ([n_out, in]), for all e."""
+        y = torch.empty((x.shape[0], n_out), dtype=x.dtype, device=x.device)
+        s = 0
+        for e, n in enumerate(self.counts):
+            if n:
+                torch.mm(x[s : s + n], weight_of(e).t(), out=y[s : s + n])
+                s += n
+        return y
+
+
 class RoutedSquaredReluMoE(nn.Module):
     """Mixture of squared-ReLU experts (down(relu(up h)^2), no biases) with
     fp32 top-k routing, weights = softmax over the chosen logits, plus an
@@ -627,28 +648,15 @@ class RoutedSquaredReluMoE(nn.Module):
         if T <= self.DENSE_MAX_TOKENS:
             a = sops.relu_squared_weighted(self.up(h), dense, ff)
             return self.down(a)
-        out = torch.zeros((T, h.shape[1]), dtype=torch.float32, device=h.device)
-        flat = idx.flatten().long()
-        order = torch.argsort(flat, stable=True)
-        counts = torch.bincount(flat, minlength=E).tolist()
-        tok = order // self.top
-        wrow = w.flatten()[order].unsqueeze(1)
-        s = 0
-        for e in range(E):
-            n = counts[e]
-            if n == 0:
-                continue
-            rows = tok[s : s + n]
-            u = F.linear(h.index_select(0, rows), self.up.weight[e * ff : (e + 1) * ff])
-            a = sops.relu_squared_weighted(u, wrow[s : s + n], ff)
-            y = F.linear(a, self.down.weight[:, e * ff : (e + 1) * ff])
-            out.index_add_(0, rows, y.float())
-            s += n
+        rows = ExpertRows(h, idx, w, E)
+        u = rows.products(rows.h, lambda e: self.up.weight[e * ff : (e + 1) * ff], ff)
+        a = sops.relu_squared_weighted(u, rows.weight, ff)
+        y = rows.products(a, lambda e: self.down.weight[:, e * ff : (e + 1) * ff], h.shape[1])
+        shared = None
         if self.shared_ff:
             u = F.linear(h, self.up.weight[E * ff :])
-            y = F.linear(sops.relu_squared(u), self.down.weight[:, E * ff :])
-            out.add_(y)
-        return out
+            shared = F.linear(sops.relu_squared(u), self.down.weight[:, E * ff :])
+        return sops.combine_expert_rows(y, rows.place, shared)
 
 
 class RoutedGatedMoE(nn.Module):
@@ -709,11 +717,8 @@ class RoutedGatedMoE(nn.Module):
     def forward(self, h):
         T = h.shape[0]
         E, ff, sff = self.experts, self.ff, self.shared_ff
-        logits = F.linear(h.float(), self.router)
-        sg = logits[:, E:] if self.shared_gate else None
-        dense, w, idx = sops.router_scores_topk(
-            logits[:, :E] if self.shared_gate else logits, self.top, self.correction,
-            self.weight_scale, self.score)
+        dense, w, idx, sg = sops.route_tokens(h, self.router, E, self.top, self.correction,
+                                              self.weight_scale, self.score)
         at = E * 2 * ff + 2 * sff  # where the caller's extra projection starts
         if T <= self.DENSE_MAX_TOKENS:
             gu = self.gate_up(h)
@@ -725,24 +730,12 @@ class RoutedGatedMoE(nn.Module):
                                   out=a[:, E * ff :], **self.shared_act)
             y = self.down(a)
             return (y, gu[:, at:]) if self.extra_out else y
-        out = torch.zeros((T, h.shape[1]), dtype=torch.float32, device=h.device)
-        flat = idx.flatten().long()
-        order = torch.argsort(flat, stable=True)
-        counts = torch.bincount(flat, minlength=E).tolist()
-        tok = order // self.top
-        wrow = w.flatten()[order].unsqueeze(1)
-        s = 0
-        for e in range(E):
-            n = counts[e]
-            if n == 0:
-                continue
-            rows = tok[s : s + n]
-            gu = F.linear(h.index_select(0, rows),
-                          self.gate_up.weight[e * 2 * ff : (e + 1) * 2 * ff])
-            a = sops.glu_weighted(gu, wrow[s : s + n], ff, w_input=self.w_input, **self.act)
-            y = F.linear(a, self.down.weight[:, e * ff : (e + 1) * ff])
-            out.index_add_(0, rows, y.float())
-            s += n
+        rows = ExpertRows(h, idx, w, E)
+        gu = rows.products(rows.h, lambda e: self.gate_up.weight[e * 2 * ff : (e + 1) * 2 * ff],
+                           2 * ff)
+        a = sops.glu_weighted(gu, rows.weight, ff, w_input=self.w_input, **self.act)
+        y = rows.products(a, lambda e: self.down.weight[:, e * ff : (e + 1) * ff], h.shape[1])
+        shared = None
         extra = None
         if sff or self.extra_out:
             # the shared expert's rows and the caller's are one product
@@ -751,8 +744,9 @@ class RoutedGatedMoE(nn.Module):
             if sff:
                 a = sops.glu_weighted(gu[:, : 2 * sff], sg, sff, w_sigmoid=True,
                                       **self.shared_act)
-                out.add_(F.linear(a, self.down.weight[:, E * ff :]))
+                shared = F.linear(a, self.down.weight[:, E * ff :])
             extra = gu[:, 2 * sff :]
+        out = sops.combine_expert_rows(y, rows.place, shared)
         return (out, extra) if self.extra_out else out
 
 

@@ -727,6 +727,64 @@ def router_scores_topk(logits, top: int, bias=None, scale: float = 1.0,
     return dense, w, idx.to(torch.int32)
 
 
+def route_tokens(h, router, experts: int, top: int, bias=None, scale: float = 1.0,
+                 score: str = "softmax"):
+    """router_scores_topk straight from the activations: logits = h router^T
+    in fp32 (h [T, C] in the serving dtype, router fp32 [experts + n, C]), the
+    first `experts` of them routed. Returns (dense, weights, index, extra) with
+    extra fp32 [T, n] the logits of the n further rows (None for n = 0)."""
+    T, n = h.shape[0], router.shape[0] - experts
+    if h.is_cuda:
+        _require_ext()
+        f32 = dict(dtype=torch.float32, device=h.device)
+        dense, w = torch.empty((T, experts), **f32), torch.empty((T, top), **f32)
+        idx = torch.empty((T, top), dtype=torch.int32, device=h.device)
+        extra = torch.empty((T, n), **f32) if n else None
+        _C.route_tokens(h, router, bias, dense, w, idx, extra, scale,
+                        {"softmax": 0, "sigmoid": 1}[score])
+        return dense, w, idx, extra
+    logits = torch.nn.functional.linear(h.float(), router)
+    dense, w, idx = router_scores_topk(logits[:, :experts], top, bias, scale, score)
+    return dense, w, idx, logits[:, experts:] if n else None
+
+
+def expert_order(index, weights, experts: int):
+    """(token, choice) pairs sorted by expert, stably. index int32 and weights
+    fp32 [T, top] -> (token int32 [N] of every sorted row, its weight fp32
+    [N, 1], place int32 [T, top] of every pair among the sorted rows, counts
+    int32 [experts]), N = T * top."""
+    T, top = index.shape
+    N = T * top
+    if index.is_cuda:
+        _require_ext()
+        i32 = dict(dtype=torch.int32, device=index.device)
+        tok, place = torch.empty(N, **i32), torch.empty((T, top), **i32)
+        counts = torch.empty(experts, **i32)
+        wrow = torch.empty((N, 1), dtype=torch.float32, device=index.device)
+        _C.expert_order(index, weights, tok, wrow, place, counts)
+        return tok, wrow, place, counts
+    flat = index.flatten().long()
+    order = torch.argsort(flat, stable=True)
+    place = torch.empty(N, dtype=torch.int32)
+    place[order] = torch.arange(N, dtype=torch.int32)
+    return ((order // top).int(), weights.flatten()[order].unsqueeze(1), place.view(T, top),
+            torch.bincount(flat, minlength=experts).int())
+
+
+def combine_expert_rows(y, place, shared=None):
+    """out[t] = sum_k y[place[t, k]] (+ shared[t]), summed in fp32; y [N, C],
+    place int32 [T, top], shared [T, C] of y's dtype; out in y's dtype."""
+    if y.is_cuda:
+        _require_ext()
+        out = torch.empty((place.shape[0], y.shape[1]), dtype=y.dtype, device=y.device)
+        _C.combine_expert_rows(out, y, place, shared)
+        return out
+    out = y[place.long()].float().sum(1)
+    if shared is not None:
+        out += shared.float()
+    return out.to(y.dtype)
+
+
 def silu_mul_weighted(gu, w, group: int):
     """Gated expert activation with the routing weight folded in. gu
     [T, n * 2 * group] holds, per expert e, `group` gate columns followed by

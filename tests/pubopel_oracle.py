@@ -112,3 +112,62 @@ def forward(cfg, W, tokens, layers_out=None):
         if layers_out is not None:
             layers_out.append(x)
     return dyt(x, W, "final.norm") @ W["head"].T
+
+
+def random_weights(cfg, seed):
+    """{name: bfloat16 torch tensor} for a config."""
+    import torch
+
+    g = torch.Generator().manual_seed(seed)
+    W = {}
+
+    def mat(name, n_out, n_in, gain=1.0):
+        W[name] = (torch.randn(n_out, n_in, generator=g) * gain * n_in ** -0.5).bfloat16()
+
+    def vec(name, n, center, spread=0.2):
+        W[name] = (center + spread * torch.randn(n, generator=g)).bfloat16()
+
+    def norm(name, n, alpha):
+        vec(name, n, 1.0)
+        vec(name + ".b", n, 0.0)
+        W[name + ".alpha"] = torch.tensor(alpha).bfloat16()
+
+    width, vocab, taps = cfg["width"], cfg["vocab"], int(cfg["canon"]["taps"])
+    W["embed"] = torch.randn(vocab, width, generator=g).bfloat16()
+    mat("head", vocab, width, 2.0)
+    norm("final.norm", width, 0.6)
+    for i, L in enumerate(cfg["layers"]):
+        p, m, q = f"l{i}.", L["mixer"], f"l{i}.mix."
+        for n in (1, 2):
+            if n == 2 and L.get("mlp") is None:
+                continue
+            norm(f"{p}norm{n}", width, 0.4 + 0.1 * n + 0.05 * i)
+            norm(f"{p}norm{n}b", width, 0.9 - 0.1 * n)
+            W[f"{p}canon{n}"] = (0.4 * torch.randn(width, taps, generator=g)).bfloat16()
+        H, G, D = m["heads"], m["kv_heads"], m["dim"]
+        mat(q + "q", H * D, width, 2.0)
+        mat(q + "k", G * D, width, 2.0)
+        vec(q + "q.norm", H * D, 1.2, 0.4)
+        vec(q + "k.norm", G * D, 1.2, 0.4)
+        vec(q + "temp", H, 1.1, 0.5)
+        vec(q + "sink", H, 0.5, 1.0)
+        mat(q + "o", width, H * D)
+        mlp = L.get("mlp")
+        if mlp is None:
+            continue
+        q = p + "mlp."
+        names = [f"{q}e{e}." for e in range(mlp["router"]["experts"])]
+        sizes = [mlp["expert"]["ff"]] * len(names)
+        if mlp.get("shared"):
+            names.append(q + "shared.")
+            sizes.append(mlp["shared"]["ff"])
+        for n, ff in zip(names, sizes):
+            mat(n + "gate", ff, width, 3.0)
+            mat(n + "up", ff, width, 3.0)
+            mat(n + "down", width, ff)
+        mat(q + "router", mlp["router"]["experts"], width, 3.0)
+    return W
+
+
+def as_float64(W):
+    return {k: v.double().numpy() for k, v in W.items()}
