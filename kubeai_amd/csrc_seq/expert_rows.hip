@@ -12,7 +12,9 @@ constexpr int kEB = 8;   // experts accumulated at a time
 // N channels a lane and step), scores = softmax or sigmoid of the first E, the
 // `top` largest s + bias in the order (value descending, index ascending),
 // weights s * wscale. LDS holds the wave's logits, then scores [TPW][R].
-template <typename T, int TPW, bool kVec>
+// kJoint (few tokens): the block's waves share one token's channels, and the
+// first wave routes it.
+template <typename T, int TPW, bool kVec, bool kJoint>
 __global__ __launch_bounds__(kRW * WAVE) void route_tokens_kernel(
     const T* __restrict__ h, int64_t h_stride, const float* __restrict__ router,
     const float* __restrict__ bias, float* __restrict__ dense,
@@ -21,9 +23,11 @@ __global__ __launch_bounds__(kRW * WAVE) void route_tokens_kernel(
   constexpr int N = kVec ? Vec16<T>::N : 1;
   extern __shared__ float lds[];
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
-  const int t0 = (blockIdx.x * kRW + wave) * TPW;
-  if (t0 >= n_tok) return;  // a whole wave; no block barrier follows
+  const int t0 = kJoint ? blockIdx.x : (blockIdx.x * kRW + wave) * TPW;
+  if (t0 >= n_tok) return;  // a whole wave (kJoint: never)
   float* z = lds + (size_t)wave * TPW * R;
+  const int c_first = (kJoint ? wave * WAVE + lane : lane) * N;
+  const int c_step = (kJoint ? kRW : 1) * WAVE * N;
   const int nt = min(TPW, n_tok - t0);
   for (int e0 = 0; e0 < R; e0 += kEB) {
     float acc[TPW][kEB];
@@ -31,7 +35,7 @@ __global__ __launch_bounds__(kRW * WAVE) void route_tokens_kernel(
     for (int i = 0; i < TPW; ++i)
 #pragma unroll
       for (int e = 0; e < kEB; ++e) acc[i][e] = 0.f;
-    for (int c = lane * N; c < C; c += WAVE * N) {
+    for (int c = c_first; c < C; c += c_step) {
       float x[TPW][N];
 #pragma unroll
       for (int i = 0; i < TPW; ++i) {
@@ -65,6 +69,15 @@ __global__ __launch_bounds__(kRW * WAVE) void route_tokens_kernel(
         const float s = wave_sum(acc[i][e]);
         if (lane == 0 && e0 + e < R) z[i * R + e0 + e] = s;
       }
+  }
+  if constexpr (kJoint) {
+    __syncthreads();
+    if (wave > 0) return;
+    for (int e = lane; e < R; e += WAVE) {
+      float s = z[e];
+      for (int w = 1; w < kRW; ++w) s += lds[(size_t)w * R + e];
+      z[e] = s;
+    }
   }
   __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
   __builtin_amdgcn_wave_barrier();
@@ -229,11 +242,12 @@ void route_tokens(torch::Tensor h, torch::Tensor router, c10::optional<torch::Te
     TORCH_CHECK(bias->numel() == E);
   }
   if (T == 0) return;
-  // several tokens a wave share the router's rows; few tokens take a wave each
-  const int tpw = T > 1024 ? 4 : 1;
+  // several tokens a wave share the router's rows; few tokens take a block each
+  const bool joint = T <= 1024;
+  const int tpw = joint ? 1 : 4;
   const size_t lds = (size_t)kRW * tpw * R * 4;
   TORCH_CHECK(lds <= 64 * 1024, "too many experts");
-  const int per = kRW * tpw;
+  const int per = joint ? 1 : kRW * tpw;
   SEQ_DISPATCH_ACT(h, {
     constexpr int n = Vec16<act_t>::N;
     const bool vec = C % n == 0 && h.stride(0) % n == 0 && ((size_t)h.data_ptr()) % 16 == 0 &&
@@ -248,10 +262,10 @@ void route_tokens(torch::Tensor h, torch::Tensor router, c10::optional<torch::Te
                          extra.has_value() ? (float*)extra->data_ptr() : nullptr, T, C, E, R,
                          top, (float)scale, (int)score);
     };
-    if (vec && tpw == 4) launch(route_tokens_kernel<act_t, 4, true>);
-    else if (vec) launch(route_tokens_kernel<act_t, 1, true>);
-    else if (tpw == 4) launch(route_tokens_kernel<act_t, 4, false>);
-    else launch(route_tokens_kernel<act_t, 1, false>);
+    if (vec && joint) launch(route_tokens_kernel<act_t, 1, true, true>);
+    else if (vec) launch(route_tokens_kernel<act_t, 4, true, false>);
+    else if (joint) launch(route_tokens_kernel<act_t, 1, false, true>);
+    else launch(route_tokens_kernel<act_t, 4, false, false>);
   });
   SEQ_CHECK_LAUNCH();
 }

@@ -348,7 +348,8 @@ def test_attention_mask_bias_cap_sink(device, name, H, G, D):
 @pytest.mark.parametrize("device", GPU)
 @pytest.mark.parametrize("name", sorted(FEATURES))
 @pytest.mark.parametrize("H,G,D", [(8, 2, 128), (8, 2, 64), (4, 2, 64), (4, 1, 48), (16, 1, 96),
-                                   (20, 1, 32), (4, 4, 16), (5, 1, 144), (8, 1, 256)])
+                                   (20, 1, 32), (4, 4, 16), (5, 1, 144), (8, 1, 256),
+                                   (2, 1, 320)])
 def test_attention_matrix_core_kernels(device, name, H, G, D):
     g = torch.Generator().manual_seed(H + D)
     T = 150
