@@ -3,7 +3,8 @@
 // packed token over its own sequence's cached keys under a chunk / window
 // mask, with separate key and value sizes. Options: first tokens that stay
 // visible behind a window, a tanh cap, a bias per position, a scale per cached
-// key, and a sink (a score without a value: one more term in the denominator).
+// key, a sink (a score without a value: one more term in the denominator), and
+// a sigmoid gate per token and head on the output.
 #include "attn_masked.h"
 
 #include <type_traits>
@@ -197,6 +198,74 @@ __global__ __launch_bounds__(256) void qnorm_rows_cache_kernel(
   }
 }
 
+// grid (T), 256 threads. RMS norm of every q and k head by itself, without a
+// weight (q in place, k into the key cache), v copied to the value cache. kVec:
+// `lpr` neighbouring lanes (a power of two) own a head's row, a 16-byte piece
+// each; otherwise a wave owns it. fp32 inside.
+template <typename T, bool kVec>
+__global__ __launch_bounds__(256) void headnorm_qk_cache_kernel(
+    T* __restrict__ q, int64_t q_stride, const T* __restrict__ k, int64_t k_stride,
+    const T* __restrict__ v, int64_t v_stride, float eps, T* __restrict__ k_cache,
+    T* __restrict__ v_cache, const int64_t* __restrict__ slot_mapping, int H, int G,
+    int D, int Dv, int bs, int lpr) {
+  constexpr int N = kVec ? Vec16<T>::N : 1;
+  const int t = blockIdx.x;
+  const int64_t slot = slot_mapping[t];
+  const int64_t blk = slot >= 0 ? slot / bs : 0;
+  const int off = slot >= 0 ? (int)(slot % bs) : 0;
+  const int per = kVec ? lpr : WAVE;  // lanes of a row
+  const int lane = threadIdx.x % per, step = blockDim.x / per;
+  const int n_rows = slot >= 0 ? H + G : H;
+  // every lane of a wave walks the same number of rows: the shuffles need all
+  for (int r0 = 0; r0 < n_rows; r0 += step) {
+    const int row = r0 + threadIdx.x / per;
+    const bool on = row < n_rows, is_q = row < H;
+    const T* src = q;
+    T* dst = q;
+    if (on) {
+      const int g = row - H;
+      src = is_q ? q + (size_t)t * q_stride + row * D : k + (size_t)t * k_stride + g * D;
+      dst = is_q ? q + (size_t)t * q_stride + row * D
+                 : k_cache + (((size_t)blk * G + g) * bs + off) * D;
+    }
+    if constexpr (kVec) {
+      float x[N];
+      float ss = 0.f;
+      const bool mine = on && lane * N < D;
+      if (mine) {
+        Vec16<T>::load(src + lane * N, x);
+#pragma unroll
+        for (int e = 0; e < N; ++e) ss += x[e] * x[e];
+      }
+      for (int o = lpr >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, WAVE);
+      const float r = 1.0f / sqrtf(ss / (float)D + eps);
+      if (mine) {
+#pragma unroll
+        for (int e = 0; e < N; ++e) x[e] *= r;
+        Vec16<T>::store(dst + lane * N, x);
+      }
+    } else {
+      float ss = 0.f;
+      if (on)
+        for (int d = lane; d < D; d += WAVE) {
+          const float x = ldf(src + d);
+          ss += x * x;
+        }
+      const float r = 1.0f / sqrtf(wave_sum(ss) / (float)D + eps);
+      if (on)
+        for (int d = lane; d < D; d += WAVE) stf(dst + d, ldf(src + d) * r);
+    }
+  }
+  if (slot < 0) return;
+  const T* vr = v + (size_t)t * v_stride;
+  for (int i = threadIdx.x * N; i < G * Dv; i += blockDim.x * N) {
+    const int g = i / Dv, d = i % Dv;
+    T* dst = v_cache + (((size_t)blk * G + g) * bs + off) * Dv + d;
+    if constexpr (kVec) *(uint4*)dst = *(const uint4*)(vr + i);
+    else *dst = vr[i];
+  }
+}
+
 constexpr int kMaxDvPerLane = 16;  // value size <= 1024
 constexpr int kDecWaves = 4;
 
@@ -337,7 +406,7 @@ __global__ __launch_bounds__(kDecWaves * WAVE) void masked_paged_attention_kerne
     lsum += stat[2 * w + 1] * wsc[w];
   }
   if (a.sink != nullptr) lsum += expf(a.sink[h] - mx);
-  const float inv = a.out_scale / lsum;
+  const float inv = a.out_factor<T>(t, h) / lsum;
   for (int d = threadIdx.x; d < Dv; d += blockDim.x) {
     float x = 0.f;
     for (int w = 0; w < kDecWaves; ++w) {
@@ -458,7 +527,7 @@ __global__ __launch_bounds__(WAVE) void masked_prefill_mfma_kernel(
   l += __shfl_xor(l, 32, WAVE);
   if (a.sink != nullptr) l += expf(a.sink[h] - m);
   if (q_ok) {
-    const float inv = a.out_scale / l;
+    const float inv = a.out_factor<bf16raw>(tq, h) / l;
     bf16raw* op = out + (size_t)tq * out_stride + h * Dv + grp * 4;
 #pragma unroll
     for (int dt = 0; dt < kMaxDvTiles; ++dt) {
@@ -707,7 +776,7 @@ __global__ __launch_bounds__(kPrefillThreads) void masked_prefill_mfma_shared_ke
   l += __shfl_xor(l, 32, WAVE);
   if (a.sink != nullptr) l += __builtin_amdgcn_exp2f(a.sink[h] * kLog2e - m);
   if (q_ok) {
-    const float inv = a.out_scale / l;
+    const float inv = a.out_factor<bf16raw>(tq, h) / l;
     bf16raw* op = out + (size_t)tq * out_stride + h * Dv + grp * 4;
 #pragma unroll
     for (int dt = 0; dt < kMaxDvTiles; ++dt) {
@@ -815,6 +884,49 @@ void qknorm_rope_half_and_cache(torch::Tensor q, torch::Tensor k, torch::Tensor 
   SEQ_CHECK_LAUNCH();
 }
 
+void headnorm_qk_to_cache(torch::Tensor q, torch::Tensor k, torch::Tensor v, double eps,
+                          torch::Tensor k_cache, torch::Tensor v_cache,
+                          torch::Tensor slot_mapping) {
+  TORCH_CHECK(q.is_cuda() && k.is_cuda() && v.is_cuda() && dense_heads3(q) &&
+              dense_heads3(k) && dense_heads3(v));
+  TORCH_CHECK(slot_mapping.scalar_type() == torch::kInt64 &&
+              slot_mapping.is_contiguous() && slot_mapping.is_cuda());
+  const int T = q.size(0), H = q.size(1), D = q.size(2), G = k.size(1), Dv = v.size(2);
+  TORCH_CHECK(k.size(0) == T && v.size(0) == T && k.size(2) == D && v.size(1) == G &&
+              slot_mapping.numel() == T);
+  TORCH_CHECK(k_cache.is_cuda() && v_cache.is_cuda() && k_cache.is_contiguous() &&
+              v_cache.is_contiguous() && k_cache.dim() == 4 && v_cache.dim() == 4);
+  TORCH_CHECK(k_cache.size(1) == G && k_cache.size(3) == D && v_cache.size(1) == G &&
+              v_cache.size(3) == Dv && v_cache.size(2) == k_cache.size(2) &&
+              v_cache.size(0) == k_cache.size(0));
+  TORCH_CHECK(k.scalar_type() == q.scalar_type() && v.scalar_type() == q.scalar_type() &&
+              k_cache.scalar_type() == q.scalar_type() &&
+              v_cache.scalar_type() == q.scalar_type());
+  if (T == 0) return;
+  const int n = 16 / q.element_size();
+  auto al = [&](const torch::Tensor& x) {
+    return ((size_t)x.data_ptr()) % 16 == 0 && x.stride(0) % n == 0;
+  };
+  int lpr = 1;
+  while (lpr * n < D) lpr *= 2;
+  const bool vec = D % n == 0 && Dv % n == 0 && lpr <= WAVE && al(q) && al(k) && al(v) &&
+                   ((size_t)k_cache.data_ptr()) % 16 == 0 &&
+                   ((size_t)v_cache.data_ptr()) % 16 == 0;
+  SEQ_DISPATCH_ACT(q, {
+    auto launch = [&](auto kern) {
+      hipLaunchKernelGGL(kern, dim3(T), dim3(256), 0, SEQ_STREAM(), (act_t*)q.data_ptr(),
+                         q.stride(0), (const act_t*)k.data_ptr(), k.stride(0),
+                         (const act_t*)v.data_ptr(), v.stride(0), (float)eps,
+                         (act_t*)k_cache.data_ptr(), (act_t*)v_cache.data_ptr(),
+                         (const int64_t*)slot_mapping.data_ptr(), H, G, D, Dv,
+                         (int)k_cache.size(2), lpr);
+    };
+    if (vec) launch(headnorm_qk_cache_kernel<act_t, true>);
+    else launch(headnorm_qk_cache_kernel<act_t, false>);
+  });
+  SEQ_CHECK_LAUNCH();
+}
+
 void qnorm_rows_to_cache(torch::Tensor q, torch::Tensor k, torch::Tensor q_weight,
                          double eps, torch::Tensor cache, torch::Tensor key_scale,
                          torch::Tensor slot_mapping) {
@@ -859,7 +971,8 @@ void masked_paged_attention(torch::Tensor out, torch::Tensor q,
                             int64_t chunk, int64_t window, double out_scale,
                             c10::optional<torch::Tensor> sink_scores,
                             int64_t keep_first, c10::optional<torch::Tensor> slopes,
-                            c10::optional<torch::Tensor> key_scale) {
+                            c10::optional<torch::Tensor> key_scale,
+                            c10::optional<torch::Tensor> head_gate) {
   check_i32(start_loc, "start_loc");
   check_i32(block_tables, "block_tables");
   check_i32(token_seq, "token_seq");
@@ -895,6 +1008,14 @@ void masked_paged_attention(torch::Tensor out, torch::Tensor q,
     check_f32(*key_scale, "key_scale");
     TORCH_CHECK(key_scale->numel() == k_cache.size(0) * bs, "one scale per cached key");
     args.kscale = (const float*)key_scale->data_ptr();
+  }
+  if (head_gate.has_value()) {
+    check_rows(*head_gate, "head_gate");
+    TORCH_CHECK(head_gate->size(0) == T && head_gate->size(1) == H &&
+                head_gate->scalar_type() == q.scalar_type(),
+                "one gate per token and head, of q's dtype");
+    args.gate = head_gate->data_ptr();
+    args.gate_rs = head_gate->stride(0);
   }
   TORCH_CHECK(keep_first >= 0 && (keep_first == 0 || (chunk == 0 && window > 0)),
               "kept first tokens belong to a window");

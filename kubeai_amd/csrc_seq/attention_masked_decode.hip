@@ -241,7 +241,8 @@ void masked_decode_mfma_kernel(
     }
     if (n_split == 1) {
       if (a.sink != nullptr) lsum += __builtin_amdgcn_exp2f(a.sink[h0 + hh] * kLog2e - mx);
-      stf(out + (size_t)t * out_stride + (h0 + hh) * Dv + d, x * a.out_scale / lsum);
+      stf(out + (size_t)t * out_stride + (h0 + hh) * Dv + d,
+          x * a.out_factor<bf16raw>(t, h0 + hh) / lsum);
     } else {
       // partial result of this split: [t][head][split] -> (max, sum), values
       const size_t row = ((size_t)t * H + h0 + hh) * n_split + sp;
@@ -258,8 +259,8 @@ void masked_decode_mfma_kernel(
 // n_split <= 32. A lane holds one split's weight; splits without keys weigh 0.
 __global__ __launch_bounds__(WAVE) void decode_split_join_kernel(
     bf16raw* __restrict__ out, int64_t out_stride, const float* __restrict__ part_o,
-    const float* __restrict__ part_ml, int H, int Dv, int n_split, float out_scale,
-    const float* __restrict__ sink) {
+    const float* __restrict__ part_ml, int n_split, AttnArgs a) {
+  const int H = a.H, Dv = a.Dv;
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const size_t row0 = ((size_t)t * H + h) * n_split;
   float2 ml = make_float2(-INFINITY, 0.f);
@@ -267,8 +268,8 @@ __global__ __launch_bounds__(WAVE) void decode_split_join_kernel(
   const float mx = wave_max(ml.x);
   const float w = __builtin_amdgcn_exp2f(ml.x - mx);
   float lsum = wave_sum(ml.y * w);
-  if (sink != nullptr) lsum += __builtin_amdgcn_exp2f(sink[h] * kLog2e - mx);
-  const float inv = out_scale / lsum;
+  if (a.sink != nullptr) lsum += __builtin_amdgcn_exp2f(a.sink[h] * kLog2e - mx);
+  const float inv = a.out_factor<bf16raw>(t, h) / lsum;
   for (int d = lane; d < Dv; d += WAVE) {
     float x = 0.f;
 #pragma unroll 4
@@ -343,8 +344,8 @@ bool masked_decode_mfma(const torch::Tensor& out, const torch::Tensor& q,
   if (n_split > 1) {
     hipLaunchKernelGGL(decode_split_join_kernel, dim3(T, H), dim3(WAVE), 0, SEQ_STREAM(),
                        (bf16raw*)out.data_ptr(), out.stride(0),
-                       (const float*)part_o.data_ptr(), (const float*)part_ml.data_ptr(), H,
-                       Dv, n_split, args.out_scale, args.sink);
+                       (const float*)part_o.data_ptr(), (const float*)part_ml.data_ptr(),
+                       n_split, args);
     SEQ_CHECK_LAUNCH();
   }
   return true;

@@ -14,6 +14,8 @@ struct AttnArgs {
   const float* sink;    // [H] or null: score of a key without a value
   const float* slopes;  // [H] or null: slopes[h] * (i - j) comes off a score
   const float* kscale;  // [blocks, bs] or null: factor of a cached key's scores
+  const void* gate;     // [T, H] or null: head h's output times sigmoid(gate[t, h])
+  int64_t gate_rs;      // elements between gate rows
   int64_t v_rs;         // elements between value rows
   int H, G, D, Dv, bs, kvs;
   int bs_shift;         // log2 of bs, or -1
@@ -25,6 +27,12 @@ struct AttnArgs {
     return lo;
   }
   DEV_INLINE int kept(int lo) const { return min(keep, lo); }
+  // factor of head h's output at token t; gate holds elements of type T
+  template <typename T>
+  DEV_INLINE float out_factor(int t, int h) const {
+    if (gate == nullptr) return out_scale;
+    return out_scale * sigmoid_f(ldf((const T*)gate + (size_t)t * gate_rs + h));
+  }
 };
 
 // Query tiles of a packed step: with `size` queries a tile, run s owns tile

@@ -37,7 +37,11 @@ void masked_paged_attention(torch::Tensor out, torch::Tensor q,
                             int64_t chunk, int64_t window, double out_scale,
                             c10::optional<torch::Tensor> sink_scores,
                             int64_t keep_first, c10::optional<torch::Tensor> slopes,
-                            c10::optional<torch::Tensor> key_scale);
+                            c10::optional<torch::Tensor> key_scale,
+                            c10::optional<torch::Tensor> head_gate);
+void headnorm_qk_to_cache(torch::Tensor q, torch::Tensor k, torch::Tensor v, double eps,
+                          torch::Tensor k_cache, torch::Tensor v_cache,
+                          torch::Tensor slot_mapping);
 void qnorm_rows_to_cache(torch::Tensor q, torch::Tensor k, torch::Tensor q_weight,
                          double eps, torch::Tensor cache, torch::Tensor key_scale,
                          torch::Tensor slot_mapping);
@@ -80,11 +84,13 @@ void scaled_add_rmsnorm(torch::Tensor out, torch::Tensor residual,
 void rmsnorm_rows(torch::Tensor out, torch::Tensor x, torch::Tensor weight, double eps);
 void gelu(torch::Tensor out, torch::Tensor x);
 void tanh_cap(torch::Tensor x, double cap);
-void latent_rope_to_cache(torch::Tensor cache, torch::Tensor x, torch::Tensor weight,
-                          double eps, c10::optional<torch::Tensor> q_rot,
+void latent_rope_to_cache(c10::optional<torch::Tensor> cache,
+                          c10::optional<torch::Tensor> x,
+                          c10::optional<torch::Tensor> weight, double eps,
+                          c10::optional<torch::Tensor> q_rot,
                           c10::optional<torch::Tensor> q_out, torch::Tensor positions,
                           torch::Tensor inv_freq, double rot_mult,
-                          torch::Tensor slot_mapping);
+                          torch::Tensor slot_mapping, bool halves);
 void router_scores_topk(torch::Tensor logits, c10::optional<torch::Tensor> bias,
                         torch::Tensor dense, torch::Tensor weights,
                         torch::Tensor index, double scale, int64_t score);
@@ -99,7 +105,8 @@ void glu_weighted(torch::Tensor out, torch::Tensor gu, c10::optional<torch::Tens
                   int64_t group, double alpha, double limit, double up_shift,
                   bool w_sigmoid, bool w_input);
 void embed_sinusoid(torch::Tensor out, torch::Tensor ids, torch::Tensor table,
-                    double scale, torch::Tensor positions, torch::Tensor freqs);
+                    double scale, c10::optional<torch::Tensor> positions,
+                    c10::optional<torch::Tensor> freqs);
 void hyper_mix_rmsnorm(torch::Tensor out, torch::Tensor streams,
                        c10::optional<torch::Tensor> y, c10::optional<torch::Tensor> gate,
                        c10::optional<torch::Tensor> mix,
@@ -133,7 +140,9 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("rope_pairs_and_cache", &rope_pairs_and_cache,
         "interleaved-pair rotary + paged cache write");
   m.def("masked_paged_attention", &masked_paged_attention,
-        "chunk/window-masked paged softmax attention, optional sink");
+        "chunk/window-masked paged softmax attention, optional sink and head gates");
+  m.def("headnorm_qk_to_cache", &headnorm_qk_to_cache,
+        "per-head q/k RMS norm + paged cache write");
   m.def("qknorm_rope_half_and_cache", &qknorm_rope_half_and_cache,
         "whole-row q/k RMS norm + split-half rotary + paged cache write");
   m.def("qnorm_rows_to_cache", &qnorm_rows_to_cache,
@@ -166,7 +175,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("glu_weighted", &glu_weighted,
         "clamped gate * sigmoid(alpha gate) * (up + shift) times a per-row, per-expert weight");
   m.def("embed_sinusoid", &embed_sinusoid,
-        "embedding lookup + sinusoidal position vector into every residual stream");
+        "embedding lookup (+ sinusoidal position vector) into every residual stream");
   m.def("hyper_mix_rmsnorm", &hyper_mix_rmsnorm,
         "residual streams: gated write, stream mix, read, RMS norm");
   m.def("scale_q_and_cache", &scale_q_and_cache,

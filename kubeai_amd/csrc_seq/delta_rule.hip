@@ -4,13 +4,15 @@
 //   S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
 //
 // with q, k unit vectors per head (q times D^-1/2), beta = sigmoid(b),
-// g = exp(-exp(a_log) softplus(a + dt_bias)). Everything but the loads of
-// q, k, v, a, b (serving dtype) is fp32. The value columns of a head are
-// independent of each other, so a head is split over waves by column.
+// g = exp(-exp(a_log) softplus(a + dt_bias)): one number per head, or one per
+// head and key channel, which then scales that channel's row of S (kChannel).
+// Everything but the loads of q, k, v, a, b (serving dtype) is fp32. The value
+// columns of a head are independent of each other, so a head is split over
+// waves by column.
 //
 // Long runs are cut into segments that run in parallel. Over a segment the
 // state goes S -> P S + B with P [D, D] the product of the tokens'
-// g (I - beta k k^T) and B [D, Dv] what the segment writes from zero. Both
+// (I - beta k k^T) diag(g) and B [D, Dv] what the segment writes from zero. Both
 // come out of the same recurrence: B by walking from zero, P by walking the
 // identity with zero values. Pass 1 (compose) walks every segment but the
 // last for P and B, pass 2 (fold) chains S_(i+1) = P_i S_i + B_i per column
@@ -28,7 +30,7 @@ DEV_INLINE float softplus_f(float x) { return x > 20.f ? x : log1pf(expf(x)); }
 // Any size: grid (n_seq * H, column blocks), block = the block's columns
 // rounded up to a wave, that part of the head's state in LDS, thread j owns
 // value column c0 + j.
-template <typename T>
+template <typename T, bool kChannel>
 __global__ void gated_delta_scan_kernel(
     float* __restrict__ o, const T* __restrict__ q, int64_t q_stride,
     const T* __restrict__ k, int64_t k_stride, const T* __restrict__ v,
@@ -49,6 +51,7 @@ __global__ void gated_delta_scan_kernel(
   float* ks = qs + kTile * D;         // [tile][D]
   float* vs = ks + kTile * D;         // [tile][CB]
   float* gb = vs + kTile * CB;        // [tile][2]: decay, beta
+  float* gs = gb + 2 * kTile;         // [tile][D]: decay per channel (kChannel)
   const int tid = threadIdx.x, nthr = blockDim.x;
   const bool carry = slot >= 0 && positions[s0] > 0;
   float* sp = state + ((size_t)(slot < 0 ? 0 : slot) * H + h) * D * Dv;
@@ -56,7 +59,7 @@ __global__ void gated_delta_scan_kernel(
     const int r = i / CB, c = i % CB;
     S[i] = (carry && c < nc) ? sp[(size_t)r * Dv + c0 + c] : 0.f;
   }
-  const float rate = -expf(a_log[h]), bias = dt_bias[h];
+  const float rate = -expf(a_log[h]), bias = kChannel ? 0.f : dt_bias[h];
   const float qscale = 1.0f / sqrtf((float)D);
   for (int t0 = s0; t0 < s1; t0 += kTile) {
     const int nt = min(kTile, s1 - t0);
@@ -65,6 +68,9 @@ __global__ void gated_delta_scan_kernel(
       const int tt = i / D, d = i % D;
       qs[i] = ldf(q + (size_t)(t0 + tt) * q_stride + hk * D + d);
       ks[i] = ldf(k + (size_t)(t0 + tt) * k_stride + hk * D + d);
+      if constexpr (kChannel)
+        gs[i] = expf(rate * softplus_f(ldf(decay_pre + (size_t)(t0 + tt) * a_stride + h * D + d) +
+                                       dt_bias[h * D + d]));
     }
     for (int i = tid; i < nt * CB; i += nthr) {
       const int tt = i / CB, d = i % CB;
@@ -82,8 +88,10 @@ __global__ void gated_delta_scan_kernel(
         qs[tid * D + d] *= rq;
         ks[tid * D + d] *= rk;
       }
-      const float a = ldf(decay_pre + (size_t)(t0 + tid) * a_stride + h);
-      gb[2 * tid] = expf(rate * softplus_f(a + bias));
+      if constexpr (!kChannel) {
+        const float a = ldf(decay_pre + (size_t)(t0 + tid) * a_stride + h);
+        gb[2 * tid] = expf(rate * softplus_f(a + bias));
+      }
       gb[2 * tid + 1] = sigmoid_f(ldf(beta_pre + (size_t)(t0 + tid) * b_stride + h));
     }
     __syncthreads();
@@ -91,10 +99,11 @@ __global__ void gated_delta_scan_kernel(
       for (int tt = 0; tt < nt; ++tt) {
         const float* qt = qs + tt * D;
         const float* kt = ks + tt * D;
-        const float g = gb[2 * tt], beta = gb[2 * tt + 1];
+        const float* gt = gs + tt * D;
+        const float g = kChannel ? 1.f : gb[2 * tt], beta = gb[2 * tt + 1];
         float dot = 0.f;
         for (int i = 0; i < D; ++i) {
-          const float st = g * S[i * CB + tid];
+          const float st = (kChannel ? gt[i] : g) * S[i * CB + tid];
           S[i * CB + tid] = st;
           dot += st * kt[i];
         }
@@ -122,8 +131,9 @@ __global__ void gated_delta_scan_kernel(
 // (r, c) keeps rows [r D/4, (r+1) D/4) of column c in registers, so a token
 // costs two passes over D/4 registers and two pairs of shuffles (the dot
 // with k before the write, the dot with q after it). q, k of kTile tokens
-// are staged through LDS, normalised once per token; the next tile is
-// fetched into registers while the current one is walked.
+// are staged through LDS, normalised once per token (and per-channel decays,
+// activated once per token); the next tile is fetched into registers while the
+// current one is walked.
 //
 // mode 0 (walk): columns are value columns; the segment starts from the
 //   slot's state (first segment), or from seg_state[seg] (later ones);
@@ -131,7 +141,7 @@ __global__ void gated_delta_scan_kernel(
 // mode 1 (compose): column blocks [0, D/16) are columns of the identity
 //   walked with zero values (-> seg_p, stored transposed), the rest value
 //   columns walked from zero (-> seg_b); the run's last segment is skipped.
-template <typename T, int kQ>
+template <typename T, int kQ, bool kChannel>
 __global__ __launch_bounds__(WAVE) void gated_delta_scan_reg_kernel(
     float* __restrict__ o, const T* __restrict__ q, int64_t q_stride,
     const T* __restrict__ k, int64_t k_stride, const T* __restrict__ v,
@@ -157,6 +167,7 @@ __global__ __launch_bounds__(WAVE) void gated_delta_scan_reg_kernel(
   if (compose && s1 == s1_run) return;
   __shared__ __attribute__((aligned(16))) float qs[kTile * D];
   __shared__ __attribute__((aligned(16))) float ks[kTile * D];
+  __shared__ __attribute__((aligned(16))) float gs[kChannel ? kTile * D : 4];
   __shared__ float vs[kTile * 16];
   __shared__ float gb[kTile * 2];
   const int lane = threadIdx.x, r = lane >> 4, c = lane & 15;
@@ -180,13 +191,14 @@ __global__ __launch_bounds__(WAVE) void gated_delta_scan_reg_kernel(
     for (int i = 0; i < R; ++i)
       S[i] = (carry && valid) ? sp[(size_t)(r * R + i) * Dv + j] : 0.f;
   }
-  const float rate = -expf(a_log[h]), bias = dt_bias[h];
+  const float rate = -expf(a_log[h]), bias = kChannel ? 0.f : dt_bias[h];
   const float qscale = 1.0f / sqrtf((float)D);
   // staging: lane (st_tt, st_part) owns a quarter row of one token of the tile
   typedef typename Raw4<T>::type raw4;
   const int st_tt = lane >> 2, st_part = lane & 3;
-  raw4 pq[kQ], pk[kQ];
+  raw4 pq[kQ], pk[kQ], pg[kChannel ? kQ : 1];
   T pv[4], pa, pb;
+  const float* db = dt_bias + (size_t)h * D + st_part * R;  // kChannel; stays in cache
   auto prefetch = [&](int tile0) {
     const int t = tile0 + st_tt;
     if (t < s1) {
@@ -197,13 +209,18 @@ __global__ __launch_bounds__(WAVE) void gated_delta_scan_reg_kernel(
         pq[b] = *(const raw4*)(qp + 4 * b);
         pk[b] = *(const raw4*)(kp + 4 * b);
       }
+      if constexpr (kChannel) {
+        const T* gp = decay_pre + (size_t)t * a_stride + h * D + st_part * R;
+#pragma unroll
+        for (int b = 0; b < kQ; ++b) pg[b] = *(const raw4*)(gp + 4 * b);
+      }
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const int col = (cb - pcb) * 16 + st_part * 4 + e;
         pv[e] = (!ident && col < Dv) ? v[(size_t)t * v_stride + h * Dv + col] : (T)0;
       }
       if (st_part == 0) {
-        pa = decay_pre[(size_t)t * a_stride + h];
+        if constexpr (!kChannel) pa = decay_pre[(size_t)t * a_stride + h];
         pb = beta_pre[(size_t)t * b_stride + h];
       }
     }
@@ -244,8 +261,20 @@ __global__ __launch_bounds__(WAVE) void gated_delta_scan_reg_kernel(
         }
 #pragma unroll
         for (int e = 0; e < 4; ++e) vs[st_tt * 16 + st_part * 4 + e] = ldf(&pv[e]);
+        if constexpr (kChannel) {
+          float ga[R];
+#pragma unroll
+          for (int b = 0; b < kQ; ++b) cvt4(pg[b], ga + 4 * b);
+#pragma unroll
+          for (int i = 0; i < R; ++i) ga[i] = expf(rate * softplus_f(ga[i] + db[i]));
+#pragma unroll
+          for (int b = 0; b < kQ; ++b)
+            *(float4*)(gs + at + 4 * b) =
+                make_float4(ga[4 * b], ga[4 * b + 1], ga[4 * b + 2], ga[4 * b + 3]);
+        }
         if (st_part == 0) {
-          gb[2 * st_tt] = expf(rate * softplus_f(ldf(&pa) + bias));
+          if constexpr (!kChannel)
+            gb[2 * st_tt] = expf(rate * softplus_f(ldf(&pa) + bias));
           gb[2 * st_tt + 1] = sigmoid_f(ldf(&pb));
         }
       }
@@ -254,7 +283,7 @@ __global__ __launch_bounds__(WAVE) void gated_delta_scan_reg_kernel(
     if (t0 + kTile < s1) prefetch(t0 + kTile);
     for (int tt = 0; tt < nt; ++tt) {
       const float vj = vs[tt * 16 + c];
-      const float g = gb[2 * tt], beta = gb[2 * tt + 1];
+      const float g = kChannel ? 1.f : gb[2 * tt], beta = gb[2 * tt + 1];
       const float4* q4 = (const float4*)(qs + tt * D + r * R);
       const float4* k4 = (const float4*)(ks + tt * D + r * R);
       float ka[R];
@@ -264,10 +293,21 @@ __global__ __launch_bounds__(WAVE) void gated_delta_scan_reg_kernel(
         const float4 kk = k4[b];
         ka[4 * b] = kk.x; ka[4 * b + 1] = kk.y; ka[4 * b + 2] = kk.z; ka[4 * b + 3] = kk.w;
       }
+      if constexpr (kChannel) {
+        const float4* g4 = (const float4*)(gs + tt * D + r * R);
 #pragma unroll
-      for (int i = 0; i < R; ++i) {
-        S[i] *= g;
-        dot += S[i] * ka[i];
+        for (int b = 0; b < kQ; ++b) {
+          const float4 gg = g4[b];
+          S[4 * b] *= gg.x; S[4 * b + 1] *= gg.y; S[4 * b + 2] *= gg.z; S[4 * b + 3] *= gg.w;
+        }
+#pragma unroll
+        for (int i = 0; i < R; ++i) dot += S[i] * ka[i];
+      } else {
+#pragma unroll
+        for (int i = 0; i < R; ++i) {
+          S[i] *= g;
+          dot += S[i] * ka[i];
+        }
       }
       dot += __shfl_xor(dot, 16, WAVE);
       dot += __shfl_xor(dot, 32, WAVE);
@@ -313,7 +353,8 @@ __global__ __launch_bounds__(WAVE) void gated_delta_scan_reg_kernel(
 
 #define DELTA_CASE(KQ)                                              \
   case KQ:                                                          \
-    launch(gated_delta_scan_reg_kernel<act_t, KQ>);                 \
+    if (channel) launch(gated_delta_scan_reg_kernel<act_t, KQ, true>);  \
+    else launch(gated_delta_scan_reg_kernel<act_t, KQ, false>);     \
     break;
 
 void gated_delta_scan(torch::Tensor o, torch::Tensor q, torch::Tensor k,
@@ -329,7 +370,9 @@ void gated_delta_scan(torch::Tensor o, torch::Tensor q, torch::Tensor k,
   check_i32(slots, "slots");
   check_i32(positions, "positions");
   check_rows(beta_pre, "beta_pre");
-  check_rows(decay_pre, "decay_pre");
+  // decay per head [T, H], or per head and key channel [T, H, D]
+  const bool channel = decay_pre.dim() == 3;
+  if (!channel) check_rows(decay_pre, "decay_pre");
   TORCH_CHECK(q.dim() == 3 && k.dim() == 3 && v.dim() == 3 && q.is_cuda());
   const int T = q.size(0), G = q.size(1), D = q.size(2), H = v.size(1), Dv = v.size(2);
   auto dense_heads = [](const torch::Tensor& t) {
@@ -343,7 +386,10 @@ void gated_delta_scan(torch::Tensor o, torch::Tensor q, torch::Tensor k,
               beta_pre.scalar_type() == q.scalar_type() &&
               decay_pre.scalar_type() == q.scalar_type());
   TORCH_CHECK(beta_pre.size(0) == T && beta_pre.size(1) == H && decay_pre.size(0) == T &&
-              decay_pre.size(1) == H && a_log.numel() == H && dt_bias.numel() == H);
+              decay_pre.size(1) == H && a_log.numel() == H && decay_pre.is_cuda());
+  TORCH_CHECK(dt_bias.numel() == (channel ? (int64_t)H * D : H));
+  TORCH_CHECK(!channel || (decay_pre.size(2) == D && dense_heads(decay_pre)),
+              "decays per channel must be laid out heads x key size");
   TORCH_CHECK(o.size(0) == T && o.size(1) == H && o.size(2) == Dv);
   TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == D &&
               state.size(3) == Dv);
@@ -354,7 +400,7 @@ void gated_delta_scan(torch::Tensor o, torch::Tensor q, torch::Tensor k,
     const size_t bytes = 4 * t.element_size();
     return ((size_t)t.data_ptr()) % bytes == 0 && t.stride(0) % 4 == 0;
   };
-  if (D % 16 == 0 && D <= 128 && vec_ok(q) && vec_ok(k)) {
+  if (D % 16 == 0 && D <= 128 && vec_ok(q) && vec_ok(k) && (!channel || vec_ok(decay_pre))) {
     const int ncb = (Dv + 15) / 16;
     int seg_len, nseg;
     delta_segments(max_len, n_seq, H, D, Dv, &seg_len, &nseg);
@@ -403,7 +449,8 @@ void gated_delta_scan(torch::Tensor o, torch::Tensor q, torch::Tensor k,
   // value columns per block: all of them if the state fits LDS, else fewer
   // (columns are independent), in whole waves
   auto lds_for = [&](int cb) {
-    return ((size_t)D * cb + 2 * kTile * D + (size_t)kTile * cb + 2 * kTile) * sizeof(float);
+    return ((size_t)D * cb + (channel ? 3 : 2) * kTile * D + (size_t)kTile * cb + 2 * kTile) *
+           sizeof(float);
   };
   int CB = std::min(((Dv + WAVE - 1) / WAVE) * WAVE, 1024);
   while (CB > WAVE && lds_for(CB) > 144 * 1024) CB -= WAVE;
@@ -412,9 +459,10 @@ void gated_delta_scan(torch::Tensor o, torch::Tensor q, torch::Tensor k,
   const int threads = CB, ncb_gen = (Dv + CB - 1) / CB;
   TORCH_CHECK(ncb_gen <= 65535);
   SEQ_DISPATCH_ACT(q, {
-    auto kern = gated_delta_scan_kernel<act_t>;
+    auto kern = channel ? gated_delta_scan_kernel<act_t, true>
+                        : gated_delta_scan_kernel<act_t, false>;
     // raise the dynamic-LDS cap once per kernel, outside any capture
-    static thread_local const void* raised[2] = {nullptr, nullptr};
+    static thread_local const void* raised[4] = {nullptr, nullptr, nullptr, nullptr};
     if (lds > 48 * 1024) {
       bool seen = false;
       for (auto p : raised) seen |= p == (const void*)kern;

@@ -65,33 +65,42 @@ __global__ __launch_bounds__(kBlock) void rmsnorm_to_cache_kernel(
 }
 
 // grid (T). Cache row of a latent with a rotated key part behind it:
-// row[:R] = x[:R] / rms(x[:R]) * w, row[R + 2i], row[R + 2i + 1] = the pair
-// (x[R + 2i], x[R + 2i + 1]) rotated by a = position * inv_freq[i] and scaled
-// by mult. The same rotation is applied to the H query slices q_rot[t, h, :]
-// (heads q_hs apart) into q_out[t, h, :] (heads o_hs apart). Angles, sin and
-// cos are fp32. Rows with slot < 0 rotate their queries and write no cache.
+// row[:R] = x[:R] / rms(x[:R]) * w, behind it the pairs of x[R:] rotated by a =
+// position * inv_freq[i] and scaled by mult: dimensions (2i, 2i + 1), or with
+// halves (i, i + half). The same rotation is applied to the H query slices
+// q_rot[t, h, :] (heads q_hs apart) into q_out[t, h, :] (heads o_hs apart).
+// Angles, sin and cos are fp32, taken once per token and kept in LDS. Rows with
+// slot < 0, or all rows when x is null (the layer reads another's cache), rotate
+// their queries and write no cache.
 template <typename T>
 __global__ __launch_bounds__(kBlock) void latent_rope_to_cache_kernel(
     T* __restrict__ cache, const T* __restrict__ x, int64_t x_stride,
     const float* __restrict__ w, float eps, const T* __restrict__ q_rot,
     int64_t q_ts, int64_t q_hs, T* __restrict__ q_out, int64_t o_ts, int64_t o_hs,
     int H, const int* __restrict__ positions, const float* __restrict__ inv_freq,
-    float mult, const int64_t* __restrict__ slot_mapping, int R, int half) {
+    float mult, const int64_t* __restrict__ slot_mapping, int R, int half, int halves) {
+  extern __shared__ float turn[];  // [half] cos, [half] sin
   __shared__ float red[16];
   const int t = blockIdx.x;
-  const int64_t slot = slot_mapping[t];
+  const int64_t slot = x != nullptr ? slot_mapping[t] : -1;
   const float pos = (float)positions[t];
-  for (int idx = threadIdx.x; idx < H * half; idx += kBlock) {
-    const int h = idx / half, i = idx % half;
+  // a pair's first element and the distance to its second
+  const int step = halves ? 1 : 2, mate = halves ? half : 1;
+  for (int i = threadIdx.x; i < half; i += kBlock) {
     float sn, cs;
     sincosf(pos * inv_freq[i], &sn, &cs);
-    sn *= mult;
-    cs *= mult;
-    const T* qp = q_rot + (size_t)t * q_ts + (size_t)h * q_hs + 2 * i;
-    const float u = ldf(qp), v = ldf(qp + 1);
-    T* op = q_out + (size_t)t * o_ts + (size_t)h * o_hs + 2 * i;
+    turn[i] = cs * mult;
+    turn[half + i] = sn * mult;
+  }
+  __syncthreads();
+  for (int idx = threadIdx.x; idx < H * half; idx += kBlock) {
+    const int h = idx / half, i = idx % half;
+    const float cs = turn[i], sn = turn[half + i];
+    const T* qp = q_rot + (size_t)t * q_ts + (size_t)h * q_hs + step * i;
+    const float u = ldf(qp), v = ldf(qp + mate);
+    T* op = q_out + (size_t)t * o_ts + (size_t)h * o_hs + step * i;
     stf(op, u * cs - v * sn);
-    stf(op + 1, v * cs + u * sn);
+    stf(op + mate, v * cs + u * sn);
   }
   if (slot < 0) return;  // uniform over the block
   const T* xr = x + (size_t)t * x_stride;
@@ -104,13 +113,11 @@ __global__ __launch_bounds__(kBlock) void latent_rope_to_cache_kernel(
   T* row = cache + (size_t)slot * (R + 2 * half);
   for (int c = threadIdx.x; c < R; c += kBlock) stf(row + c, ldf(xr + c) * r * w[c]);
   for (int i = threadIdx.x; i < half; i += kBlock) {
-    float sn, cs;
-    sincosf(pos * inv_freq[i], &sn, &cs);
-    sn *= mult;
-    cs *= mult;
-    const float u = ldf(xr + R + 2 * i), v = ldf(xr + R + 2 * i + 1);
-    stf(row + R + 2 * i, u * cs - v * sn);
-    stf(row + R + 2 * i + 1, v * cs + u * sn);
+    const float cs = turn[i], sn = turn[half + i];
+    const int at = R + step * i;
+    const float u = ldf(xr + at), v = ldf(xr + at + mate);
+    stf(row + at, u * cs - v * sn);
+    stf(row + at + mate, v * cs + u * sn);
   }
 }
 
@@ -193,26 +200,38 @@ void rmsnorm_to_cache(torch::Tensor cache, torch::Tensor x, torch::Tensor weight
   SEQ_CHECK_LAUNCH();
 }
 
-void latent_rope_to_cache(torch::Tensor cache, torch::Tensor x, torch::Tensor weight,
-                          double eps, c10::optional<torch::Tensor> q_rot,
+void latent_rope_to_cache(c10::optional<torch::Tensor> cache,
+                          c10::optional<torch::Tensor> x,
+                          c10::optional<torch::Tensor> weight, double eps,
+                          c10::optional<torch::Tensor> q_rot,
                           c10::optional<torch::Tensor> q_out, torch::Tensor positions,
                           torch::Tensor inv_freq, double rot_mult,
-                          torch::Tensor slot_mapping) {
-  check_rows(x, "x");
-  check_f32(weight, "weight");
+                          torch::Tensor slot_mapping, bool halves) {
   check_f32(inv_freq, "inv_freq");
   check_i32(positions, "positions");
   TORCH_CHECK(slot_mapping.scalar_type() == torch::kInt64 &&
               slot_mapping.is_contiguous() && slot_mapping.is_cuda());
-  const int T = x.size(0), R = weight.numel(), half = inv_freq.numel();
-  const int C = R + 2 * half;
-  TORCH_CHECK(x.size(1) == C, "x must hold the latent and the rotated key part");
-  TORCH_CHECK(cache.is_contiguous() && cache.is_cuda() && cache.dim() == 4 &&
-              cache.size(1) == 1 && cache.size(3) == C &&
-              cache.scalar_type() == x.scalar_type(),
-              "cache must be [blocks, 1, block, latent + rotated] of the activations' dtype");
-  TORCH_CHECK(slot_mapping.numel() == T && positions.numel() == T);
+  const int T = positions.numel(), half = inv_freq.numel();
+  TORCH_CHECK(slot_mapping.numel() == T);
   TORCH_CHECK(q_rot.has_value() == q_out.has_value());
+  TORCH_CHECK((size_t)half * 8 <= 32 * 1024, "too many rotated pairs");
+  int R = 0;
+  if (x.has_value()) {
+    TORCH_CHECK(weight.has_value() && cache.has_value());
+    check_rows(*x, "x");
+    check_f32(*weight, "weight");
+    R = weight->numel();
+    const int C = R + 2 * half;
+    TORCH_CHECK(x->size(0) == T && x->size(1) == C,
+                "x must hold the latent and the rotated key part");
+    TORCH_CHECK(cache->is_contiguous() && cache->is_cuda() && cache->dim() == 4 &&
+                cache->size(1) == 1 && cache->size(3) == C &&
+                cache->scalar_type() == x->scalar_type(),
+                "cache must be [blocks, 1, block, latent + rotated] of the activations' dtype");
+  } else {
+    TORCH_CHECK(q_rot.has_value(), "neither a latent nor queries");
+  }
+  const torch::Tensor& act = x.has_value() ? *x : *q_rot;
   int H = 0;
   const void* qp = nullptr;
   void* op = nullptr;
@@ -223,7 +242,7 @@ void latent_rope_to_cache(torch::Tensor cache, torch::Tensor x, torch::Tensor we
                 q.size(0) == T && o.size(0) == T && q.size(1) == o.size(1) &&
                 q.size(2) == 2 * half && o.size(2) == 2 * half &&
                 q.stride(2) == 1 && o.stride(2) == 1 &&
-                q.scalar_type() == x.scalar_type() && o.scalar_type() == x.scalar_type());
+                q.scalar_type() == act.scalar_type() && o.scalar_type() == act.scalar_type());
     H = q.size(1);
     qp = q.data_ptr();
     op = o.data_ptr();
@@ -231,15 +250,17 @@ void latent_rope_to_cache(torch::Tensor cache, torch::Tensor x, torch::Tensor we
     o_ts = o.stride(0); o_hs = o.stride(1);
   }
   if (T == 0) return;
-  SEQ_DISPATCH_ACT(x, {
-    hipLaunchKernelGGL((latent_rope_to_cache_kernel<act_t>), dim3(T), dim3(kBlock), 0,
-                       SEQ_STREAM(), (act_t*)cache.data_ptr(),
-                       (const act_t*)x.data_ptr(), x.stride(0),
-                       (const float*)weight.data_ptr(), (float)eps, (const act_t*)qp,
-                       q_ts, q_hs, (act_t*)op, o_ts, o_hs, H,
+  SEQ_DISPATCH_ACT(act, {
+    hipLaunchKernelGGL((latent_rope_to_cache_kernel<act_t>), dim3(T), dim3(kBlock),
+                       (size_t)half * 8, SEQ_STREAM(),
+                       x.has_value() ? (act_t*)cache->data_ptr() : nullptr,
+                       x.has_value() ? (const act_t*)x->data_ptr() : nullptr,
+                       x.has_value() ? x->stride(0) : 0,
+                       x.has_value() ? (const float*)weight->data_ptr() : nullptr,
+                       (float)eps, (const act_t*)qp, q_ts, q_hs, (act_t*)op, o_ts, o_hs, H,
                        (const int*)positions.data_ptr(),
                        (const float*)inv_freq.data_ptr(), (float)rot_mult,
-                       (const int64_t*)slot_mapping.data_ptr(), R, half);
+                       (const int64_t*)slot_mapping.data_ptr(), R, half, halves ? 1 : 0);
   });
   SEQ_CHECK_LAUNCH();
 }

@@ -1,5 +1,5 @@
 // Kernels around several residual streams and differential attention:
-// embedding lookup + sinusoidal position vector into every stream, the fused
+// embedding lookup (+ sinusoidal position vector) into every stream, the fused
 // stream update / read / RMS norm between sublayers, the query temperature +
 // paged cache write for caches whose value heads are fewer than their key
 // heads, and the join of two attention maps (difference, per-head RMS norm).
@@ -11,7 +11,7 @@ constexpr int kBlock = 256;
 constexpr int kMaxStreams = 8;
 
 // grid (T). out[t, s, c] = table[id, c] * scale + (c odd ? cos : sin)(pos * freqs[c / 2])
-// for every stream s. The angle is formed and reduced to [0, 2 pi) in double
+// for every stream s (freqs null: no position vector). The angle is formed and reduced to [0, 2 pi) in double
 // (an fp32 product loses the phase at positions in the thousands); sinf /
 // cosf are the precise library functions.
 template <typename T>
@@ -21,13 +21,16 @@ __global__ __launch_bounds__(kBlock) void embed_sinusoid_kernel(
     int S, int C) {
   const int t = blockIdx.x;
   const T* row = table + (size_t)ids[t] * C;
-  const double p = (double)positions[t];
+  const double p = freqs != nullptr ? (double)positions[t] : 0.0;
   constexpr double kTwoPi = 6.283185307179586476925;
   for (int c = threadIdx.x; c < C; c += kBlock) {
-    double a = p * freqs[c >> 1];
-    a -= kTwoPi * floor(a / kTwoPi);
-    const float ang = (float)a;
-    const float x = ldf(row + c) * scale + ((c & 1) ? cosf(ang) : sinf(ang));
+    float x = ldf(row + c) * scale;
+    if (freqs != nullptr) {
+      double a = p * freqs[c >> 1];
+      a -= kTwoPi * floor(a / kTwoPi);
+      const float ang = (float)a;
+      x += (c & 1) ? cosf(ang) : sinf(ang);
+    }
     for (int s = 0; s < S; ++s) out[((size_t)t * S + s) * C + c] = x;
   }
 }
@@ -148,23 +151,28 @@ __global__ __launch_bounds__(kBlock) void diff_combine_kernel(
 }  // namespace
 
 void embed_sinusoid(torch::Tensor out, torch::Tensor ids, torch::Tensor table,
-                    double scale, torch::Tensor positions, torch::Tensor freqs) {
+                    double scale, c10::optional<torch::Tensor> positions,
+                    c10::optional<torch::Tensor> freqs) {
   check_f32(out, "out");
   check_i32(ids, "ids");
-  check_i32(positions, "positions");
-  TORCH_CHECK(freqs.scalar_type() == torch::kFloat64 && freqs.is_contiguous() &&
-              freqs.is_cuda(), "freqs must be a contiguous float64 GPU tensor");
   TORCH_CHECK(table.is_cuda() && table.is_contiguous() && table.dim() == 2 &&
               out.dim() == 3);
   const int T = out.size(0), S = out.size(1), C = out.size(2);
-  TORCH_CHECK(table.size(1) == C && ids.numel() == T && positions.numel() == T &&
-              freqs.numel() >= (C + 1) / 2);
+  TORCH_CHECK(table.size(1) == C && ids.numel() == T);
+  if (freqs.has_value()) {
+    TORCH_CHECK(freqs->scalar_type() == torch::kFloat64 && freqs->is_contiguous() &&
+                freqs->is_cuda(), "freqs must be a contiguous float64 GPU tensor");
+    TORCH_CHECK(positions.has_value() && freqs->numel() >= (C + 1) / 2);
+    check_i32(*positions, "positions");
+    TORCH_CHECK(positions->numel() == T);
+  }
   if (T == 0) return;
   SEQ_DISPATCH_ACT(table, {
     hipLaunchKernelGGL((embed_sinusoid_kernel<act_t>), dim3(T), dim3(kBlock), 0,
                        SEQ_STREAM(), (float*)out.data_ptr(), (const int*)ids.data_ptr(),
                        (const act_t*)table.data_ptr(), (float)scale,
-                       (const int*)positions.data_ptr(), (const double*)freqs.data_ptr(),
+                       freqs.has_value() ? (const int*)positions->data_ptr() : nullptr,
+                       freqs.has_value() ? (const double*)freqs->data_ptr() : nullptr,
                        S, C);
   });
   SEQ_CHECK_LAUNCH();

@@ -87,6 +87,8 @@ class ModelArchConfig:
             return vigonex_arch_config(cfg)
         if cfg.get("architecture") == "Pubopel":
             return pubopel_arch_config(cfg)
+        if cfg.get("architecture") == "Lipulorn":
+            return lipulorn_arch_config(cfg)
         hidden = cfg["hidden_size"]
         n_heads = cfg["num_attention_heads"]
         arch = (cfg.get("architectures") or ["LlamaForCausalLM"])[0]
@@ -381,6 +383,39 @@ def pubopel_arch_config(cfg: dict) -> ModelArchConfig:
             norm_eps=float(cfg["norm"]["eps"]),
             embedding_scale=1.0,
             canon_taps=taps,
+        ),
+    )
+
+
+def lipulorn_arch_config(cfg: dict) -> ModelArchConfig:
+    """Lipulorn config.json -> arch config: the list of layers (mixer type, the
+    mixer's sizes and constants, the feed-forward), the number of residual
+    streams and the norm epsilon, all as the file gives them."""
+    layers = [
+        HybridLayerSpec(type=L["type"], mixer=L["mixer"], mlp=L.get("mlp"), weights_of=i)
+        for i, L in enumerate(cfg["layers"])
+    ]
+    streams = int(cfg["streams"])
+    if streams < 1:
+        raise ValueError("streams must be at least 1")
+    return ModelArchConfig(
+        architecture="lipulorn",
+        vocab_size=int(cfg["vocab"]),
+        hidden_size=int(cfg["width"]),
+        num_hidden_layers=len(layers),
+        intermediate_size=0,
+        num_attention_heads=0,
+        num_key_value_heads=0,
+        head_dim=0,
+        max_position_embeddings=1 << 30,  # positions are computed, not tabulated
+        bos_token_id=-1,
+        eos_token_id=-1,  # the design defines no end token
+        hybrid=HybridSpec(
+            layers=layers,
+            norm_eps=float(cfg["norm"]["eps"]),
+            embedding_scale=1.0,
+            canon_taps=0,
+            streams=streams,
         ),
     )
 
@@ -961,6 +996,38 @@ def pubopel_preset(width: int, layers: int, vocab: int = 32000, head_dim: int = 
     })
 
 
+def lipulorn_preset(width: int, layers: int, vocab: int = 32000, head_dim: int = 128,
+                    window: int = 1024, kv_rank: int = 128, rot_dim: int = 64,
+                    streams: int = 4, ff_scale: float = 1.0) -> ModelArchConfig:
+    """A Lipulorn stack of the given size with random-init weights: the layer
+    pattern (chunked attention, channel-decay delta rule, latent attention
+    with its own latent, latent attention reading that latent) repeats to the
+    requested depth. width/head_dim heads, a quarter as many key/value heads in
+    chunked attention, half as many query/key heads in the delta rule; the
+    feed-forward is a dense 3.5 x width gated layer (times ff_scale, for
+    matching another model's size)."""
+    heads = max(1, width // head_dim)
+    mlp = {"kind": "dense", "ff": max(16, int(3.5 * ff_scale * width) // 16 * 16)}
+    att = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": head_dim,
+           "vdim": head_dim, "scale": head_dim ** -0.5, "mask": {"size": window}}
+    delta = {"heads": heads, "kv_heads": max(1, heads // 2), "dim": head_dim,
+             "vdim": head_dim, "conv": 4}
+    lat = {"heads": heads, "dim": head_dim, "rot_dim": rot_dim, "vdim": head_dim,
+           "kv_rank": kv_rank, "q_rank": max(64, width // 2),
+           "scale": (head_dim + rot_dim) ** -0.5, "mask": {"size": window},
+           "rot": {"base": 10000.0, "dims": rot_dim}}
+    out = []
+    for i in range(layers):
+        kind, mixer = [("attention", att), ("channel_delta", delta),
+                       ("latent_attention", lat),
+                       ("latent_attention", dict(lat, kv_from=i - 1))][i % 4]
+        out.append({"type": kind, "mixer": dict(mixer), "mlp": mlp})
+    return lipulorn_arch_config({
+        "architecture": "Lipulorn", "vocab": vocab, "width": width, "streams": streams,
+        "norm": {"eps": 1e-5}, "layers": out,
+    })
+
+
 def dulotar_preset(width: int, layers: int, vocab: int = 32000, head_dim: int = 128,
                    chunk: int = 1024, ff_mult: int = 4) -> ModelArchConfig:
     """A Dulotar stack of the given size with random-init weights: the
@@ -1012,6 +1079,11 @@ PRESETS.update({
     "pubopel-1k": pubopel_preset(1024, 12),
     "pubopel-2k": pubopel_preset(2048, 12),
     "pubopel-4k": pubopel_preset(4096, 6),
+    "lipulorn-tiny": lipulorn_preset(128, 4, vocab=512, head_dim=32, window=40,
+                                     kv_rank=48, rot_dim=16),
+    "lipulorn-1k": lipulorn_preset(1024, 12),
+    "lipulorn-2k": lipulorn_preset(2048, 12),
+    "lipulorn-4k": lipulorn_preset(4096, 6),
     "dulotar-tiny": dulotar_preset(128, 3, vocab=512, head_dim=32, chunk=64),
     "dulotar-1k": dulotar_preset(1024, 12),
     "dulotar-2k": dulotar_preset(2048, 12),

@@ -379,7 +379,11 @@ class LatentAttention(nn.Module):
                 down-projection followed by an up-projection (0 = one matrix)
       rot_dim   every query head has rot_dim more dimensions that are rotated
                 by position, against one rotated key part shared by all heads
-                and cached behind the latent (0 = no positions enter)
+                and cached behind the latent (0 = no positions enter);
+                rot_halves pairs dimension i with i + rot_dim / 2 instead of
+                2i with 2i + 1
+      window    a position sees itself and the window - 1 tokens before it
+                (0 = everything before it)
       sink      a learned score per head that joins the softmax denominator
                 without a value
       gate      "channel": every output channel times sigmoid of a projection
@@ -390,11 +394,12 @@ class LatentAttention(nn.Module):
     run against the cached rows (the rotated parts just extend the dot
     product), and the value up-projection is applied to the attended latent.
     With own_latent=False the layer has no down-projection and reads the
-    cache of another layer (bound by the model)."""
+    cache of another layer (bound by the model), rotated key part included;
+    only its queries are rotated here."""
 
     def __init__(self, width, heads, dim, vdim, kv_rank, scale, own_latent=True,
                  eps=1e-5, q_rank=0, rot_dim=0, rot_base=10000.0, rot_scaling=None,
-                 sink=False, gate="channel"):
+                 sink=False, gate="channel", rot_halves=False, window=0):
         super().__init__()
         self.heads, self.dim, self.vdim, self.rank = heads, dim, vdim, kv_rank
         self.scale, self.own_latent, self.eps = float(scale), bool(own_latent), eps
@@ -403,8 +408,7 @@ class LatentAttention(nn.Module):
             raise ValueError(f"unknown gate {gate!r}")
         if self.rot_dim % 2:
             raise ValueError("rot_dim must be even")
-        if self.rot_dim and not own_latent:
-            raise ValueError("a borrowed latent carries no rotated key part")
+        self.rot_halves, self.window = bool(rot_halves), int(window or 0)
         qd = dim + self.rot_dim
         n_q = self.q_rank if self.q_rank else heads * qd
         n_g = {"channel": heads * vdim, "head": heads, None: 0}[gate]
@@ -452,18 +456,22 @@ class LatentAttention(nn.Module):
             q = proj[:, :nq]
         q = q.unflatten(-1, (H, D + r))
         ql = torch.empty((T, H, R + r), dtype=h.dtype, device=h.device)
-        if self.own_latent and r:
-            sops.latent_rope_to_cache(proj[:, nq + ng :], self.latent_norm, self.eps,
+        if r:
+            own = self.own_latent
+            sops.latent_rope_to_cache(proj[:, nq + ng :] if own else None,
+                                      self.latent_norm, self.eps,
                                       q[..., D:], ql[..., R:], fb.positions,
-                                      self.inv_freq, self.rot_mult, c_cache,
-                                      fb.slot_mapping)
+                                      self.inv_freq, self.rot_mult,
+                                      c_cache if own else None, fb.slot_mapping,
+                                      self.rot_halves)
         elif self.own_latent:
             sops.rmsnorm_to_cache(proj[:, nq + ng :], self.latent_norm, self.eps,
                                   c_cache, fb.slot_mapping)
         sops.head_linear(q[..., :D], self.uk_r, out=ql[..., :R])  # [T, H, R]
         lat = torch.empty((T, H, R), dtype=h.dtype, device=h.device)
         sops.masked_paged_attention(ql, c_cache, c_cache[..., :R] if r else c_cache,
-                                    fb.seq, self.scale, lat, sink=self.sink_scores)
+                                    fb.seq, self.scale, lat, window=self.window,
+                                    sink=self.sink_scores)
         o = sops.head_linear(lat, self.uv,
                              gate=proj[:, nq : nq + ng] if ng else None)  # [T, H, Dv]
         return self.o_proj(o.view(T, H * Dv))
@@ -540,22 +548,67 @@ class GatedDeltaMixer(nn.Module):
     q and k have kv_heads heads shared by groups of value heads; q, k and v
     pass a short causal convolution with silu; q and k are unit vectors per
     head (q times dim^-1/2). The read-out is RMS-normed per head (one weight
-    vector shared by the heads) and gated by silu of a projection."""
+    vector shared by the heads) and gated by gate_act of a projection.
 
-    def __init__(self, width, heads, kv_heads, dim, vdim, conv_taps, eps):
+    channel_decay: one decay per head and key channel instead of one per head.
+    decay_rank, gate_rank > 0: the decay's / the gate's projection goes through
+    a bottleneck of that size, W2 (W1 h). The W1 matrices are rows of the input
+    product and the W2 matrices one product over both bottlenecks (block
+    diagonal), so either costs no launch of its own."""
+
+    def __init__(self, width, heads, kv_heads, dim, vdim, conv_taps, eps,
+                 channel_decay=False, decay_rank=0, gate_rank=0, gate_act="silu"):
         super().__init__()
         if heads % kv_heads:
             raise ValueError("heads must be a multiple of kv_heads")
+        self.width = width
         self.heads, self.kv_heads, self.dim, self.vdim, self.eps = heads, kv_heads, dim, vdim, eps
+        self.channel_decay, self.gate_act = bool(channel_decay), gate_act
         nqk, nv = kv_heads * dim, heads * vdim
-        self.sizes = (nqk, nqk, nv, nv, heads, heads)  # q | k | v | gate | beta | decay
-        self.in_proj = Proj(width, sum(self.sizes))
+        self.n_decay = heads * dim if channel_decay else heads
+        self.set_ranks(decay_rank, gate_rank)
         self.conv = CausalConvTails(2 * nqk + nv, conv_taps, residual=False, act="silu")
         self.a_log = _f32(heads)
-        self.dt_bias = _f32(heads)
+        self.dt_bias = _f32(self.n_decay)
         self.norm = _f32(nv)  # the per-head weight, repeated for every head
         nn.init.ones_(self.norm)
         self.o_proj = Proj(nv, width)
+
+    def set_ranks(self, decay_rank, gate_rank):
+        """(Re)build the projections for these bottleneck sizes (a checkpoint
+        gives them by the shapes of its tensors). `at` holds every section's
+        columns of the input product, the bottlenecks side by side; sections
+        start at multiples of eight columns, so that products and kernels
+        read aligned rows (the columns between are zero rows of the weight)."""
+        self.decay_rank, self.gate_rank = int(decay_rank or 0), int(gate_rank or 0)
+        nqk, nv = self.kv_heads * self.dim, self.heads * self.vdim
+        low = self.decay_rank + self.gate_rank
+        self.at, end = {}, 0
+        for name, n in (("qkv", 2 * nqk + nv), ("low", low),
+                        ("gate", 0 if self.gate_rank else nv), ("beta", self.heads),
+                        ("decay", 0 if self.decay_rank else self.n_decay)):
+            if n:
+                self.at[name] = slice(end, end + n)
+                end = (end + n + 7) // 8 * 8
+        # columns of the second product: decay, then gate
+        self.up_decay = slice(0, self.n_decay if self.decay_rank else 0)
+        end_up = (self.up_decay.stop + 7) // 8 * 8
+        self.up_gate = slice(end_up, end_up + (nv if self.gate_rank else 0))
+        old = getattr(self, "in_proj", None)
+        like = dict(device=old.weight.device, dtype=old.weight.dtype) if old is not None else {}
+        self.in_proj = Proj(self.width, end).to(**like)
+        self.low_proj = Proj(low, (self.up_gate.stop + 7) // 8 * 8).to(**like) if low else None
+        # nothing may leak between the sections: zero what no matrix fills
+        keep = torch.zeros(end, dtype=torch.bool)
+        for part in self.at.values():
+            keep[part] = True
+        if self.in_proj.weight.device.type != "meta":
+            self.in_proj.weight.data[~keep.to(self.in_proj.weight.device)] = 0
+            if low:
+                w = self.low_proj.weight.data
+                w[:, : self.decay_rank][self.up_decay.stop :] = 0
+                w[:, self.decay_rank :][: self.up_gate.start] = 0
+                w[self.up_gate.stop :] = 0
 
     def state_spec(self):
         return {"conv": self.conv.state_shape(),
@@ -569,16 +622,18 @@ class GatedDeltaMixer(nn.Module):
         H, G, D, Dv = self.heads, self.kv_heads, self.dim, self.vdim
         nqk, nv = G * D, H * Dv
         proj = self.in_proj(h)
-        qkv = self.conv(proj[:, : 2 * nqk + nv], fb, state["conv"])
-        at = 2 * nqk + 2 * nv
+        qkv = self.conv(proj[:, self.at["qkv"]], fb, state["conv"])
+        up = self.low_proj(proj[:, self.at["low"]]) if self.low_proj is not None else None
+        decay = up[:, self.up_decay] if self.decay_rank else proj[:, self.at["decay"]]
+        gate = up[:, self.up_gate] if self.gate_rank else proj[:, self.at["gate"]]
+        if self.channel_decay:
+            decay = decay.unflatten(-1, (H, D))
         o = sops.gated_delta_scan(
             qkv[:, :nqk].unflatten(-1, (G, D)), qkv[:, nqk : 2 * nqk].unflatten(-1, (G, D)),
-            qkv[:, 2 * nqk :].unflatten(-1, (H, Dv)), proj[:, at : at + H],
-            proj[:, at + H : at + 2 * H], self.a_log, self.dt_bias,
-            state["s"], fb.seq)
+            qkv[:, 2 * nqk :].unflatten(-1, (H, Dv)), proj[:, self.at["beta"]], decay,
+            self.a_log, self.dt_bias, state["s"], fb.seq)
         y = torch.empty((T, nv), dtype=h.dtype, device=h.device)
-        sops.gated_rmsnorm(o.view(T, nv), self.norm, proj[:, 2 * nqk + nv : at], H,
-                           "silu", self.eps, y)
+        sops.gated_rmsnorm(o.view(T, nv), self.norm, gate, H, self.gate_act, self.eps, y)
         return self.o_proj(y)
 
 
@@ -752,16 +807,17 @@ class RoutedGatedMoE(nn.Module):
 
 class SiluGatedMLP(nn.Module):
     """Dense gated feed-forward: down(silu(gate h) * (up h)); the gate and up
-    matrices are one stacked [2 ff, width] product. extra_out > 0 appends
-    that many rows (with a bias) for a projection of the same input that the
-    caller owns; forward then returns (output, that projection)."""
+    matrices are one stacked [2 ff, width] product. bias: all three have one.
+    extra_out > 0 appends that many rows (with a bias) for a projection of the
+    same input that the caller owns; forward then returns (output, that
+    projection)."""
 
-    def __init__(self, width: int, ff: int, extra_out: int = 0):
+    def __init__(self, width: int, ff: int, extra_out: int = 0, bias: bool = False):
         super().__init__()
         self.ff, self.extra_out = ff, int(extra_out or 0)
         n_in = 2 * ff + self.extra_out
-        self.gate_up = BiasProj(width, n_in) if self.extra_out else Proj(width, n_in)
-        self.down = Proj(ff, width)
+        self.gate_up = (BiasProj if bias or self.extra_out else Proj)(width, n_in)
+        self.down = (BiasProj if bias else Proj)(ff, width)
 
     def forward(self, h):
         gu = self.gate_up(h)
@@ -781,6 +837,31 @@ class BiasProj(nn.Module):
 
     def forward(self, x):
         return F.linear(x, self.weight, self.bias)
+
+
+class HyperConnection(nn.Module):
+    """Read weights, write weights and the stream-to-stream matrix of one
+    sublayer, with its input norm and residual gate (own_gate=False: the
+    sublayer computes the gate's projection inside its own input product)."""
+
+    def __init__(self, width: int, streams: int, own_gate: bool = True):
+        super().__init__()
+        self.norm = _f32(width)
+        nn.init.ones_(self.norm)
+        self.read = _f32(streams)
+        self.write = _f32(streams)
+        self.mix = _f32(streams, streams)
+        nn.init.constant_(self.read, 1.0 / streams)
+        nn.init.ones_(self.write)
+        self.mix.data.copy_(torch.eye(streams))
+        self.gate = BiasProj(width, width) if own_gate else None
+
+    def written(self, X, y, gate=None):
+        """The streams [T, S, C] after this sublayer's output y (times sigmoid
+        of its gate's pre-activation) is written, X left as it is."""
+        z = y.float() if gate is None else y.float() * torch.sigmoid(gate.float())
+        return (torch.einsum("st,nsc->ntc", self.mix, X)
+                + self.write.view(1, -1, 1) * z.unsqueeze(1))
 
 
 class DifferentialAttention(nn.Module):
@@ -855,6 +936,49 @@ class DifferentialAttention(nn.Module):
         sops.diff_combine(att.view(T, G, 2, H // G, Dv), self.lam, self.gain, self.eps,
                           out)
         return self.o_proj(out.view(T, H * Dv))
+
+
+class HeadGatedAttention(nn.Module):
+    """Softmax attention with grouped key/value heads and separate key and
+    value sizes, whose queries and keys are divided by their root mean square
+    per head (no weight) and whose heads' outputs are multiplied by one sigmoid
+    gate each, read from the layer's input. No positions enter. Options, each
+    a constructor argument: position-aligned chunks, a sliding window, biases on
+    q, k and v. q | k | v | gate are one product."""
+
+    def __init__(self, width, heads, kv_heads, dim, vdim, scale, chunk=0, window=0,
+                 bias=True, eps=1e-5):
+        super().__init__()
+        if heads % kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        self.heads, self.kv_heads, self.dim, self.vdim, self.eps = heads, kv_heads, dim, vdim, eps
+        self.scale, self.chunk, self.window = float(scale), int(chunk or 0), int(window or 0)
+        self.sizes = (heads * dim, kv_heads * dim, kv_heads * vdim, heads)
+        # q | k | v | gate, and zero rows up to a whole number of 16-byte pieces
+        self.n_in = (sum(self.sizes) + 7) // 8 * 8
+        self.in_proj = (BiasProj if bias else Proj)(width, self.n_in)
+        self.o_proj = Proj(heads * vdim, width)
+
+    def state_spec(self):
+        return {}
+
+    def kv_spec(self):
+        return (self.kv_heads, self.dim, self.vdim)
+
+    def forward(self, h, fb, state, kv_cache):
+        T = h.shape[0]
+        nq, nk, nv, _ = self.sizes
+        proj = self.in_proj(h)
+        q = proj[:, :nq].unflatten(-1, (self.heads, self.dim))
+        k = proj[:, nq : nq + nk].unflatten(-1, (self.kv_heads, self.dim))
+        v = proj[:, nq + nk : nq + nk + nv].unflatten(-1, (self.kv_heads, self.vdim))
+        k_cache, v_cache = kv_cache
+        sops.headnorm_qk_to_cache(q, k, v, self.eps, k_cache, v_cache, fb.slot_mapping)
+        out = torch.empty((T, self.heads, self.vdim), dtype=h.dtype, device=h.device)
+        sops.masked_paged_attention(q, k_cache, v_cache, fb.seq, self.scale, out,
+                                    chunk=self.chunk, window=self.window,
+                                    head_gate=proj[:, nq + nk + nv :][:, : self.heads])
+        return self.o_proj(out.view(T, self.heads * self.vdim))
 
 
 class GeneralDeltaMixer(nn.Module):

@@ -39,6 +39,12 @@ def _pubopel():
     return PubopelForCausalLM
 
 
+def _lipulorn():
+    from .lipulorn import LipulornForCausalLM
+
+    return LipulornForCausalLM
+
+
 MODEL_REGISTRY = {
     "llama": _llama,
     "mixtral": _llama,
@@ -47,6 +53,7 @@ MODEL_REGISTRY = {
     "vekusun": _vekusun,
     "vigonex": _vigonex,
     "pubopel": _pubopel,
+    "lipulorn": _lipulorn,
 }
 
 
@@ -69,6 +76,7 @@ MODEL_EXTENSIONS = {
     "vekusun": ("_C_seq",),
     "vigonex": ("_C_seq",),
     "pubopel": ("_C_seq",),
+    "lipulorn": ("_C_seq",),
 }
 
 

@@ -226,8 +226,10 @@ class VekusunForCausalLM(nn.Module):
                     put(m.sink_scores, get(q + "sink"))
                 put(m.o_proj.weight, get(q + "o"))
             else:
-                put(m.in_proj.weight,
-                    torch.cat([get(q + n) for n in ("q", "k", "v", "g", "b", "a")]))
+                rows = torch.zeros_like(m.in_proj.weight, device="cpu")
+                for name, part in (("qkv", "qkv"), ("gate", "g"), ("beta", "b"), ("decay", "a")):
+                    rows[m.at[name]] = torch.cat([get(q + n) for n in part])
+                put(m.in_proj.weight, rows)
                 put(m.conv.weight,
                     torch.cat([get(q + n + ".conv") for n in ("q", "k", "v")]))
                 put(m.a_log, get(q + "A_log"))

@@ -32,9 +32,9 @@ from kubeai_amd.engine.batch import ForwardBatch
 from kubeai_amd.ops import seq as sops
 from .config import HybridLayerSpec, ModelArchConfig
 from .mixers import (
-    BiasProj,
     DifferentialAttention,
     GeneralDeltaMixer,
+    HyperConnection,
     RoutedGatedMoE,
     SiluGatedMLP,
     _f32,
@@ -78,24 +78,6 @@ def build_mlp(mlp: dict | None, width: int):
             extra_out=width,
         )
     raise ValueError(f"unknown feed-forward kind {kind!r}")
-
-
-class HyperConnection(nn.Module):
-    """Read weights, write weights and the stream-to-stream matrix of one
-    sublayer, with its input norm and residual gate (own_gate=False: the
-    sublayer computes the gate's projection inside its own input product)."""
-
-    def __init__(self, width: int, streams: int, own_gate: bool = True):
-        super().__init__()
-        self.norm = _f32(width)
-        nn.init.ones_(self.norm)
-        self.read = _f32(streams)
-        self.write = _f32(streams)
-        self.mix = _f32(streams, streams)
-        nn.init.constant_(self.read, 1.0 / streams)
-        nn.init.ones_(self.write)
-        self.mix.data.copy_(torch.eye(streams))
-        self.gate = BiasProj(width, width) if own_gate else None
 
 
 class VigonexLayer(nn.Module):
@@ -171,11 +153,6 @@ class VigonexForCausalLM(nn.Module):
         self.states = states
 
     # --------------------------------------------------------------------
-    def _streams_after(self, X, y, gate, hc):
-        z = y.float() * torch.sigmoid(gate.float())
-        return (torch.einsum("st,nsc->ntc", hc.mix, X)
-                + hc.write.view(1, -1, 1) * z.unsqueeze(1)).sum(1)
-
     @torch.inference_mode()
     def forward(self, fb: ForwardBatch) -> torch.Tensor:
         hs = self.cfg.hybrid
@@ -201,7 +178,7 @@ class VigonexForCausalLM(nn.Module):
                 hc = layer.hc2
                 y, gate = layer.mlp(h)
             if self.capture_layers is not None:
-                self.capture_layers.append(self._streams_after(X, y, gate, hc))
+                self.capture_layers.append(hc.written(X, y, gate).sum(1))
         return sops.hyper_mix_rmsnorm(
             X, y, gate, hc.mix if hc is not None else None,
             hc.write if hc is not None else None, self.final_read, self.final_norm,

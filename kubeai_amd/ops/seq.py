@@ -402,9 +402,11 @@ def gated_delta_scan(q, k, v, beta_pre, decay_pre, a_log, dt_bias, state,
 
     so a token's read-out sees its own write. q, k [T, G, D] with H a
     multiple of G (head h uses q/k head h // (H/G)), v [T, H, Dv], beta_pre
-    and decay_pre [T, H] (strided column views allowed), a_log and dt_bias
-    fp32 [H], state fp32 [slots, H, D, Dv]. Everything but the loads is fp32.
-    Returns o fp32 [T, H, Dv]."""
+    [T, H], state fp32 [slots, H, D, Dv], a_log fp32 [H]. The decay is one
+    number per head (decay_pre [T, H], dt_bias fp32 [H]), or one per head and
+    key channel (decay_pre [T, H, D], dt_bias fp32 [H * D]), which then
+    multiplies that channel's row of S. Strided column views are fine;
+    everything but the loads is fp32. Returns o fp32 [T, H, Dv]."""
     T, G, D = q.shape
     H, Dv = v.shape[1], v.shape[2]
     if q.is_cuda:
@@ -423,12 +425,13 @@ def gated_delta_scan(q, k, v, beta_pre, decay_pre, a_log, dt_bias, state,
         qs = qs.repeat_interleave(rep, dim=1)
         ks = ks.repeat_interleave(rep, dim=1)
         beta = torch.sigmoid(beta_pre[s0 : s0 + n].float())
-        g = torch.exp(-torch.exp(a_log) * torch.nn.functional.softplus(
-            decay_pre[s0 : s0 + n].float() + dt_bias))
+        pre = decay_pre[s0 : s0 + n].float()
+        rate = torch.nn.functional.softplus(pre + dt_bias.view(pre.shape[1:]))
+        g = torch.exp(-torch.exp(a_log).view((H,) + (1,) * (pre.dim() - 2)) * rate)
         S = (state[slot].clone() if (slot >= 0 and p0 > 0)
              else torch.zeros(H, D, Dv))
         for t in range(n):
-            S = S * g[t].view(H, 1, 1)
+            S = S * g[t].view(H, -1, 1)
             u = beta[t].view(H, 1) * (vs[t] - torch.einsum("hkv,hk->hv", S, ks[t]))
             S = S + ks[t].unsqueeze(-1) * u.unsqueeze(-2)
             o[s0 + t] = torch.einsum("hkv,hk->hv", S, qs[t])
@@ -559,41 +562,51 @@ def rmsnorm_to_cache(x, weight, eps: float, cache, slot_mapping):
 
 
 def latent_rope_to_cache(x, weight, eps: float, q_rot, q_out, positions,
-                         inv_freq, rot_mult: float, cache, slot_mapping):
+                         inv_freq, rot_mult: float, cache, slot_mapping,
+                         halves: bool = False):
     """Cache row of a latent-attention layer with a shared rotated key part.
 
     x [T, R + r] (strided rows fine): the first R = len(weight) columns are
     RMS-normed (times weight) into the cache row's first R columns; the last
     r = 2 len(inv_freq) columns are rotated and written behind them. The
-    rotation pairs dimension 2i with 2i+1: (u, w) -> (u cos a - w sin a,
-    w cos a + u sin a) * rot_mult, a = position * inv_freq[i], fp32. The same
+    rotation pairs dimension 2i with 2i+1, or with halves dimension i with
+    i + r / 2: (u, w) -> (u cos a - w sin a, w cos a + u sin a) * rot_mult,
+    a = position * inv_freq[i], fp32. The same
     rotation is applied to q_rot [T, H, r] (a strided slice of the query
     heads), written to q_out [T, H, r] (a strided slice of the folded query).
     r may be 0 (q_rot/q_out None): only the norm runs. cache
-    [blocks, 1, block, R + r]; rows with slot < 0 are not written."""
-    R = weight.numel()
+    [blocks, 1, block, R + r]; rows with slot < 0 are not written. x, weight
+    and cache None: only the queries rotate (a layer that reads another
+    layer's cache)."""
     half = inv_freq.numel()
-    if x.is_cuda:
+    if positions.is_cuda:
         _require_ext()
         _C.latent_rope_to_cache(cache, x, weight, eps, q_rot, q_out, positions,
-                                inv_freq, rot_mult, slot_mapping)
+                                inv_freq, rot_mult, slot_mapping, halves)
         return
+    if half:
+        a = positions.float().unsqueeze(-1) * inv_freq
+        cs, sn = torch.cos(a) * rot_mult, torch.sin(a) * rot_mult
+        first = slice(0, half) if halves else slice(0, None, 2)
+        second = slice(half, None) if halves else slice(1, None, 2)
+
+        def rot(t, cs, sn):
+            u, w = t[..., first], t[..., second]
+            o = torch.empty_like(t)
+            o[..., first] = u * cs - w * sn
+            o[..., second] = w * cs + u * sn
+            return o
+
+        if q_rot is not None:
+            q_out.copy_(rot(q_rot.float(), cs.unsqueeze(1), sn.unsqueeze(1)).to(q_out.dtype))
+    if x is None:
+        return
+    R = weight.numel()
     xf = x.float()
     c = xf[:, :R]
     row = [c * torch.rsqrt((c * c).mean(-1, keepdim=True) + eps) * weight]
     if half:
-        a = positions.float().unsqueeze(-1) * inv_freq
-        cs, sn = torch.cos(a) * rot_mult, torch.sin(a) * rot_mult
-
-        def rot(t, cs, sn):
-            u, w = t[..., 0::2], t[..., 1::2]
-            o = torch.empty_like(t)
-            o[..., 0::2] = u * cs - w * sn
-            o[..., 1::2] = w * cs + u * sn
-            return o
-
         row.append(rot(xf[:, R:], cs, sn))
-        q_out.copy_(rot(q_rot.float(), cs.unsqueeze(1), sn.unsqueeze(1)).to(q_out.dtype))
     y = torch.cat(row, dim=-1)
     ok = slot_mapping >= 0
     flat = cache.view(-1, cache.shape[-1])
@@ -623,6 +636,31 @@ def qnorm_rows_to_cache(q, k, q_weight, eps: float, cache, key_scale, slot_mappi
     off = (slot_mapping[ok] % bs).long()
     cache[blk, :, off] = k[ok].to(cache.dtype)
     key_scale[blk, off, 0] = torch.rsqrt((kf * kf).mean(-1) + eps)[ok]
+    return q
+
+
+def headnorm_qk_to_cache(q, k, v, eps: float, k_cache, v_cache, slot_mapping):
+    """Every q and k head divided by its own root mean square (no weight),
+    x / sqrt(mean(x^2) + eps) in fp32: q in place, k into the key cache at
+    slot_mapping, v copied to the value cache (slot < 0: no write). q [T, H, D],
+    k [T, G, D], v [T, G, Dv] may be strided views; caches
+    [blocks, G, block, D | Dv]."""
+    if q.is_cuda:
+        _require_ext()
+        _C.headnorm_qk_to_cache(q, k, v, eps, k_cache, v_cache, slot_mapping)
+        return q
+
+    def norm(x):
+        xf = x.float()
+        return (xf * torch.rsqrt((xf * xf).mean(-1, keepdim=True) + eps)).to(x.dtype)
+
+    q.copy_(norm(q))
+    bs = k_cache.shape[2]
+    ok = slot_mapping >= 0
+    blk = (slot_mapping[ok] // bs).long()
+    off = (slot_mapping[ok] % bs).long()
+    k_cache[blk, :, off] = norm(k)[ok].to(k_cache.dtype)
+    v_cache[blk, :, off] = v[ok].to(v_cache.dtype)
     return q
 
 
@@ -842,7 +880,8 @@ def masked_paged_attention(q, k_cache, v_cache, meta: SeqMeta, scale: float,
                            sink: Optional[torch.Tensor] = None,
                            keep_first: int = 0,
                            slopes: Optional[torch.Tensor] = None,
-                           key_scale: Optional[torch.Tensor] = None):
+                           key_scale: Optional[torch.Tensor] = None,
+                           head_gate: Optional[torch.Tensor] = None):
     """Softmax attention of every packed token over its own sequence's cached
     keys. The token at position i sees j <= i with, when chunk > 0,
     floor(j / chunk) == floor(i / chunk) (position-aligned chunks) and, when
@@ -859,7 +898,9 @@ def masked_paged_attention(q, k_cache, v_cache, meta: SeqMeta, scale: float,
     fewer heads than k_cache (Gv dividing G: query head h reads key head
     h // (H / G) and value head h // (H / Gv), so several score maps share
     one value head);
-    out [T, H, Dv] may be a strided view; out = attention * out_scale.
+    out [T, H, Dv] may be a strided view; out = attention * out_scale, times
+    sigmoid(head_gate[t, h]) if a gate is given (q's dtype, [T, H], rows may be
+    strided).
     sink=True stands for a score of 0 on every head."""
     if keep_first and chunk:
         raise ValueError("kept first tokens and chunks do not combine")
@@ -874,7 +915,8 @@ def masked_paged_attention(q, k_cache, v_cache, meta: SeqMeta, scale: float,
         _C.masked_paged_attention(out, q, k_cache, v_cache, meta.block_tables,
                                   meta.start_loc, meta.token_seq, meta.positions,
                                   meta.max_len, scale, softcap, chunk, window,
-                                  out_scale, sink, keep_first, slopes, key_scale)
+                                  out_scale, sink, keep_first, slopes, key_scale,
+                                  head_gate)
         return out
     T, H, D = q.shape
     G, bs = k_cache.shape[1], k_cache.shape[2]
@@ -918,6 +960,8 @@ def masked_paged_attention(q, k_cache, v_cache, meta: SeqMeta, scale: float,
         if sink is not None:
             p = p[..., :-1]
         o = torch.einsum("htl,lhd->thd", p, vs) * out_scale
+        if head_gate is not None:
+            o = o * torch.sigmoid(head_gate[s0 : s0 + n].float()).unsqueeze(-1)
         out[s0 : s0 + n] = o.to(out.dtype)
     return out
 
@@ -943,6 +987,18 @@ def embed_sinusoid(ids, table, scale: float, positions, freqs, copies: int = 1):
     pe = torch.stack([torch.sin(ang), torch.cos(ang)], dim=-1).reshape(T, -1)[:, :C]
     x = table[ids.long()].float() * scale + pe
     return x.unsqueeze(1).repeat(1, copies, 1)
+
+
+def embed_streams(ids, table, copies: int):
+    """fp32 [T, copies, C], every copy table[ids] (table [V, C] in the serving
+    dtype)."""
+    if table.is_cuda:
+        _require_ext()
+        out = torch.empty((ids.shape[0], copies, table.shape[1]), dtype=torch.float32,
+                          device=table.device)
+        _C.embed_sinusoid(out, ids, table, 1.0, None, None)
+        return out
+    return table[ids.long()].float().unsqueeze(1).repeat(1, copies, 1)
 
 
 def hyper_mix_rmsnorm(streams, y, gate, mix, out_w, in_w, weight, eps: float,
