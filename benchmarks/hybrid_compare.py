@@ -1,15 +1,17 @@
 """Prefill and decode throughput of a layer-list design (Dulotar, Nugopel,
-Vekusun, Vigonex, Pubopel) beside the closest existing stack of equal width, depth and
-(about) parameter count, random weights, one GPU: a dense Llama for Dulotar,
+Vekusun, Vigonex, Pubopel, Lipulorn) beside the closest existing stack of equal width,
+depth and (about) parameter count, random weights, one GPU: a dense Llama for Dulotar,
 a Mixtral-style routed Llama (same number of experts and choices) for
 Nugopel, Nugopel itself (latent attention, routed experts) for Vekusun,
 Vekusun (full causal attention, a delta rule, dense and routed gated
-feed-forwards, sequence state) for Vigonex, and Nugopel (window attention with
+feed-forwards, sequence state) for Vigonex, Nugopel (window attention with
 a sink and whole-projection norms, norms on both sides of a sublayer, routed
-experts with a shared one) for Pubopel; the feed-forward sizes of the last
-three are scaled so that the parameter counts agree.
+experts with a shared one) for Pubopel, and Vekusun again (latent attention
+with a query latent and a rotated key part, a gated delta rule, sequence
+state) for Lipulorn; the feed-forward sizes of the last four are scaled so
+that the parameter counts agree.
 
-    python bench.py --compare-hybrid [--compare-design dulotar|nugopel|vekusun|vigonex|pubopel]
+    python bench.py --compare-hybrid [--compare-design dulotar|nugopel|vekusun|vigonex|pubopel|lipulorn]
                     [--compare-sizes 1k,2k,4k]
 
 Prefill: one sequence's whole prompt as a single fixed step (both families
@@ -30,7 +32,8 @@ from kubeai_amd.models import config as configs
 from kubeai_amd.models.config import PRESETS, ModelArchConfig
 
 # design -> the layer-list design it is compared with at equal parameter count
-SIZED_LIKE = {"vekusun": "nugopel", "vigonex": "vekusun", "pubopel": "nugopel"}
+SIZED_LIKE = {"vekusun": "nugopel", "vigonex": "vekusun", "pubopel": "nugopel",
+              "lipulorn": "vekusun"}
 SIZES = {"1k": (1024, 12), "2k": (2048, 12), "4k": (4096, 6)}
 
 
@@ -145,7 +148,7 @@ def main(args) -> None:
     prefill_lens = [2048, 8192] if device == "cuda" else [64]
     batches = [(64, 1536), (8, 3584)] if device == "cuda" else [(2, 32)]
     design = getattr(args, "compare_design", None) or "dulotar"
-    if design not in ("dulotar", "nugopel", "vekusun", "vigonex", "pubopel"):
+    if design not in ("dulotar", "nugopel", "vekusun", "vigonex", "pubopel", "lipulorn"):
         raise SystemExit(f"unknown design {design!r}")
     for key in sizes:
         width, layers = SIZES[key]

@@ -35,21 +35,6 @@ struct AttnArgs {
   }
 };
 
-// Query tiles of a packed step: with `size` queries a tile, run s owns tile
-// numbers start_loc[s] / size + s and on (never fewer than it needs), so T /
-// size + n_seq blocks cover every batch, whatever its mix of lengths. Returns
-// the run of tile number b and b's place in the run.
-DEV_INLINE int find_tile(const int* start_loc, int n_seq, int size, int b, int* tile) {
-  int lo = 0, hi = n_seq - 1;  // the last run whose first number is <= b
-  while (lo < hi) {
-    const int mid = (lo + hi + 1) >> 1;
-    if (start_loc[mid] / size + mid <= b) lo = mid;
-    else hi = mid - 1;
-  }
-  *tile = b - (start_loc[lo] / size + lo);
-  return lo;
-}
-
 // softcap * tanh(x / softcap) times log2 e as cap2 - 2 cap2 / (e^(2x/cap) + 1):
 // absolute error below 1e-6 of the cap. x comes multiplied by 2 log2(e) / cap.
 DEV_INLINE float cap_base2(float x, float cap2) {

@@ -11,7 +11,7 @@ void relu_squared(torch::Tensor out, torch::Tensor x);
 void causal_conv(torch::Tensor y, torch::Tensor x, torch::Tensor w,
                  torch::Tensor tails, torch::Tensor start_loc,
                  torch::Tensor slots, torch::Tensor token_seq,
-                 torch::Tensor positions, bool residual, int64_t act);
+                 torch::Tensor positions, bool residual, int64_t act, int64_t max_len);
 void token_shift_mix(torch::Tensor out, torch::Tensor h, torch::Tensor mu,
                      torch::Tensor prev, torch::Tensor start_loc,
                      torch::Tensor slots, torch::Tensor token_seq,

@@ -42,18 +42,88 @@ __global__ void causal_conv_kernel(
   stf(y + (size_t)t * C + c, acc);
 }
 
+constexpr int kSpan = 16;  // tokens a thread of the vector kernel walks
+
+DEV_INLINE float conv_act(float x, int act, bool exact) {
+  if (act != 1) return x;
+  return exact ? silu_f(x)
+               : x * __builtin_amdgcn_rcpf(
+                         1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * x));
+}
+
+// The same for kTaps taps and whole, aligned 16-byte pieces of channels: grid
+// (T / kSpan + n_seq, pieces), a thread walks up to kSpan tokens of one run
+// with the last taps - 1 inputs of its channels in registers. A run that fits
+// one span advances its tail here (nobody else reads it); longer runs leave it
+// to tail_update_kernel.
+template <typename T, int kTaps>
+__global__ __launch_bounds__(128) void causal_conv_vec_kernel(
+    T* __restrict__ y, const T* __restrict__ x, int64_t x_stride,
+    const float* __restrict__ w, float* __restrict__ tails,
+    const int* __restrict__ start_loc, const int* __restrict__ slots,
+    const int* __restrict__ positions, int n_seq, int C, int residual, int act) {
+  constexpr int N = Vec16<T>::N, K1 = kTaps - 1;
+  int tile;
+  const int s = find_tile(start_loc, n_seq, kSpan, blockIdx.x, &tile);
+  const int c = (blockIdx.y * blockDim.x + threadIdx.x) * N;
+  const int s0 = start_loc[s], s1 = start_loc[s + 1], slot = slots[s];
+  const int t0 = s0 + tile * kSpan, t1 = min(t0 + kSpan, s1);
+  if (c >= C || t0 >= s1) return;
+  float wt[kTaps][N];
+#pragma unroll
+  for (int e = 0; e < N; ++e)
+#pragma unroll
+    for (int j = 0; j < kTaps; ++j) wt[j][e] = w[(size_t)(c + e) * kTaps + j];
+  float win[kTaps][N];  // inputs t - K1 .. t
+  const int p0 = positions[s0];
+#pragma unroll
+  for (int i = 0; i < K1; ++i) {
+    const int src = t0 - K1 + i, sp = p0 + src - s0;
+    if (src >= s0) {
+      Vec16<T>::load(x + (size_t)src * x_stride + c, win[i]);
+    } else {
+#pragma unroll
+      for (int e = 0; e < N; ++e)
+        win[i][e] = sp >= 0 && slot >= 0
+                        ? tails[((size_t)slot * K1 + (sp - (p0 - K1))) * C + c + e] : 0.f;
+    }
+  }
+  for (int t = t0; t < t1; ++t) {
+    Vec16<T>::load(x + (size_t)t * x_stride + c, win[K1]);
+    float o[N];
+#pragma unroll
+    for (int e = 0; e < N; ++e) {
+      float acc = residual ? win[K1][e] : 0.f;
+#pragma unroll
+      for (int j = 0; j < kTaps; ++j) acc += wt[j][e] * win[j][e];
+      o[e] = conv_act(acc, act, sizeof(T) == 4);
+#pragma unroll
+      for (int j = 0; j < K1; ++j) win[j][e] = win[j + 1][e];
+    }
+    Vec16<T>::store(y + (size_t)t * C + c, o);
+  }
+  if (slot >= 0 && s1 - s0 <= kSpan) {
+#pragma unroll
+    for (int i = 0; i < K1; ++i)
+#pragma unroll
+      for (int e = 0; e < N; e += 4)
+        st4(tails + ((size_t)slot * K1 + i) * C + c + e, win[i] + e);
+  }
+}
+
 // grid (n_seq, ceil(C / 256)): advance a run's tail past its tokens. One
 // thread owns a channel's whole tail, so old rows are read before any write.
+// Runs of up to `done` tokens are left alone.
 template <typename T>
 __global__ void tail_update_kernel(
     float* __restrict__ tails, const T* __restrict__ x, int64_t x_stride,
     const int* __restrict__ start_loc, const int* __restrict__ slots,
-    const int* __restrict__ positions, int C, int K1) {
+    const int* __restrict__ positions, int C, int K1, int done) {
   const int s = blockIdx.x;
   const int c = blockIdx.y * blockDim.x + threadIdx.x;
   if (c >= C) return;
   const int slot = slots[s], s0 = start_loc[s], n = start_loc[s + 1] - s0;
-  if (slot < 0 || n <= 0) return;
+  if (slot < 0 || n <= done) return;
   const int p0 = positions[s0];
   float buf[kMaxTail];
   for (int i = 0; i < K1; ++i) {
@@ -90,7 +160,7 @@ __global__ void token_shift_mix_kernel(
 
 static void launch_tail_update(torch::Tensor tails, torch::Tensor x,
                                torch::Tensor start_loc, torch::Tensor slots,
-                               torch::Tensor positions, int C, int K1) {
+                               torch::Tensor positions, int C, int K1, int done = 0) {
   const int n_seq = slots.numel();
   if (n_seq == 0 || K1 == 0) return;
   SEQ_DISPATCH_ACT(x, {
@@ -98,7 +168,7 @@ static void launch_tail_update(torch::Tensor tails, torch::Tensor x,
                        dim3(256), 0, SEQ_STREAM(), (float*)tails.data_ptr(),
                        (const act_t*)x.data_ptr(), x.stride(0),
                        (const int*)start_loc.data_ptr(), (const int*)slots.data_ptr(),
-                       (const int*)positions.data_ptr(), C, K1);
+                       (const int*)positions.data_ptr(), C, K1, done);
   });
   SEQ_CHECK_LAUNCH();
 }
@@ -106,7 +176,7 @@ static void launch_tail_update(torch::Tensor tails, torch::Tensor x,
 void causal_conv(torch::Tensor y, torch::Tensor x, torch::Tensor w,
                  torch::Tensor tails, torch::Tensor start_loc,
                  torch::Tensor slots, torch::Tensor token_seq,
-                 torch::Tensor positions, bool residual, int64_t act) {
+                 torch::Tensor positions, bool residual, int64_t act, int64_t max_len) {
   check_rows(x, "x");
   TORCH_CHECK(act == 0 || act == 1, "act: 0 none, 1 silu");
   check_f32(w, "w");
@@ -124,6 +194,28 @@ void causal_conv(torch::Tensor y, torch::Tensor x, torch::Tensor w,
               start_loc.numel() == slots.numel() + 1);
   TORCH_CHECK((C + 255) / 256 <= 65535);
   if (T == 0) return;
+  const int n = 16 / x.element_size(), n_seq = slots.numel();
+  if (taps >= 2 && taps <= 4 && C % n == 0 && x.stride(0) % n == 0 &&
+      ((size_t)x.data_ptr()) % 16 == 0 && n_seq > 0) {
+    const int pieces = (C / n + 127) / 128;
+    SEQ_DISPATCH_ACT(x, {
+      auto launch = [&](auto kern) {
+        hipLaunchKernelGGL(kern, dim3(T / kSpan + n_seq, pieces), dim3(128), 0,
+                           SEQ_STREAM(), (act_t*)y.data_ptr(), (const act_t*)x.data_ptr(),
+                           x.stride(0), (const float*)w.data_ptr(), (float*)tails.data_ptr(),
+                           (const int*)start_loc.data_ptr(), (const int*)slots.data_ptr(),
+                           (const int*)positions.data_ptr(), n_seq, C, residual ? 1 : 0,
+                           (int)act);
+      };
+      if (taps == 2) launch(causal_conv_vec_kernel<act_t, 2>);
+      else if (taps == 3) launch(causal_conv_vec_kernel<act_t, 3>);
+      else launch(causal_conv_vec_kernel<act_t, 4>);
+    });
+    SEQ_CHECK_LAUNCH();
+    if (max_len > kSpan)
+      launch_tail_update(tails, x, start_loc, slots, positions, C, taps - 1, kSpan);
+    return;
+  }
   SEQ_DISPATCH_ACT(x, {
     hipLaunchKernelGGL((causal_conv_kernel<act_t>), dim3(T, (C + 255) / 256),
                        dim3(256), 0, SEQ_STREAM(), (act_t*)y.data_ptr(),

@@ -126,23 +126,51 @@ __global__ void gated_delta_scan_kernel(
     }
 }
 
+// exp(rate * softplus(x)) for rate <= 0, on the hardware's base-2 exponential
+// and logarithm. ln(1 + e) = ln(u) * e / (u - 1) with u the rounded 1 + e keeps
+// the relative accuracy of a softplus near zero, which is what a decay near one
+// is made of.
+DEV_INLINE float decay_f(float rate, float x) {
+  constexpr float kL2e = 1.4426950408889634f, kLn2 = 0.6931471805599453f;
+  const float e = __builtin_amdgcn_exp2f(x * kL2e);
+  const float u = 1.f + e, d = u - 1.f;
+  float sp = __builtin_amdgcn_logf(u) * kLn2 * (e * __builtin_amdgcn_rcpf(d));
+  sp = d == 0.f ? e : sp;
+  sp = x > 20.f ? x : sp;
+  return __builtin_amdgcn_exp2f(rate * kL2e * sp);
+}
+
+// sum over the four lanes 16 apart, in every one of them
+DEV_INLINE float quad_sum(float x) {
+  const unsigned a = __builtin_bit_cast(unsigned, x);
+  const auto p = __builtin_amdgcn_permlane16_swap(a, a, false, false);
+  x = __builtin_bit_cast(float, (unsigned)p[0]) + __builtin_bit_cast(float, (unsigned)p[1]);
+  const unsigned b = __builtin_bit_cast(unsigned, x);
+  const auto q = __builtin_amdgcn_permlane32_swap(b, b, false, false);
+  return __builtin_bit_cast(float, (unsigned)q[0]) + __builtin_bit_cast(float, (unsigned)q[1]);
+}
+
+constexpr int kCols = 2;  // value columns of a lane (register-state kernel)
+
 // Register-state form for key sizes D = 16 * kQ (<= 128). One wave per block
-// owns 16 columns of one head's state over one segment of one run: lane
-// (r, c) keeps rows [r D/4, (r+1) D/4) of column c in registers, so a token
-// costs two passes over D/4 registers and two pairs of shuffles (the dot
-// with k before the write, the dot with q after it). q, k of kTile tokens
-// are staged through LDS, normalised once per token (and per-channel decays,
-// activated once per token); the next tile is fetched into registers while the
-// current one is walked.
+// owns 16 kCols columns of one head's state over one segment of one run: lane
+// (r, c) keeps rows [r D/4, (r+1) D/4) of columns kCols c .. in registers, so
+// what a token brings (k, q, decays) is read from LDS once for all of them, a
+// token costs two passes over the registers, and the sums over the four lanes
+// of a column (the dot with k before the write, the one with q after it) are
+// lane swaps. q, k of kTile tokens are staged through LDS, normalised once per
+// token (and per-channel decays, activated once per token); the next tile is
+// fetched into registers while the current one is walked.
 //
 // mode 0 (walk): columns are value columns; the segment starts from the
 //   slot's state (first segment), or from seg_state[seg] (later ones);
 //   writes o, and the slot's state after the run's last segment.
-// mode 1 (compose): column blocks [0, D/16) are columns of the identity
-//   walked with zero values (-> seg_p, stored transposed), the rest value
-//   columns walked from zero (-> seg_b); the run's last segment is skipped.
+// mode 1 (compose): the first ceil(D / 16 kCols) column blocks are columns of
+//   the identity walked with zero values (-> seg_p, stored transposed), the
+//   rest value columns walked from zero (-> seg_b); the run's last segment is
+//   skipped.
 template <typename T, int kQ, bool kChannel>
-__global__ __launch_bounds__(WAVE) void gated_delta_scan_reg_kernel(
+__global__ __launch_bounds__(WAVE, 2) void gated_delta_scan_reg_kernel(
     float* __restrict__ o, const T* __restrict__ q, int64_t q_stride,
     const T* __restrict__ k, int64_t k_stride, const T* __restrict__ v,
     int64_t v_stride, const T* __restrict__ beta_pre, int64_t b_stride,
@@ -153,7 +181,7 @@ __global__ __launch_bounds__(WAVE) void gated_delta_scan_reg_kernel(
     int Dv, int ncb, float norm_eps, int nseg, int seg_len, int mode,
     float* __restrict__ seg_p, float* __restrict__ seg_b,
     const float* __restrict__ seg_state) {
-  constexpr int R = 4 * kQ, D = 4 * R;
+  constexpr int R = 4 * kQ, D = 4 * R, W = 16 * kCols;
   const int cb = blockIdx.x % ncb;
   const int h = (blockIdx.x / ncb) % H;
   const int seg = (blockIdx.x / (ncb * H)) % nseg;
@@ -168,28 +196,60 @@ __global__ __launch_bounds__(WAVE) void gated_delta_scan_reg_kernel(
   __shared__ __attribute__((aligned(16))) float qs[kTile * D];
   __shared__ __attribute__((aligned(16))) float ks[kTile * D];
   __shared__ __attribute__((aligned(16))) float gs[kChannel ? kTile * D : 4];
-  __shared__ float vs[kTile * 16];
+  __shared__ __attribute__((aligned(16))) float vs[kTile * W];
   __shared__ float gb[kTile * 2];
   const int lane = threadIdx.x, r = lane >> 4, c = lane & 15;
-  // compose: the first D/16 column blocks walk the identity
-  const int pcb = compose ? D / 16 : 0;
+  // compose: the first column blocks walk the identity
+  const int pcb = compose ? (D + W - 1) / W : 0;
   const bool ident = cb < pcb;
-  const int j = (cb - pcb) * 16 + c;  // value column (when not ident)
-  const bool valid = ident || j < Dv;
-  float S[R];
-  if (compose) {
+  const int vc0 = (cb - pcb) * W;       // the block's first value column (when not ident)
+  const int j0 = vc0 + kCols * c;       // the lane's
+  const bool even = Dv % kCols == 0;    // whole pairs: aligned, all or none valid
+  float S[kCols][R];
+  auto load_cols = [&](const float* base) {
+    const float* p = base + (size_t)r * R * Dv + min(j0, Dv - 1);
+    if (even && j0 < Dv) {
 #pragma unroll
-    for (int i = 0; i < R; ++i) S[i] = (ident && r * R + i == cb * 16 + c) ? 1.f : 0.f;
-  } else if (seg > 0) {
-    const float* ss = seg_state + (((size_t)s * nseg + seg) * H + h) * D * Dv;
+      for (int i = 0; i < R; ++i) {
+        const float2 x = *(const float2*)(p + (size_t)i * Dv);
+        S[0][i] = x.x;
+        S[1][i] = x.y;
+      }
+    } else {
+      const int step = j0 + 1 < Dv ? 1 : 0;  // columns past the end are never stored
 #pragma unroll
-    for (int i = 0; i < R; ++i) S[i] = valid ? ss[(size_t)(r * R + i) * Dv + j] : 0.f;
+      for (int i = 0; i < R; ++i) {
+        S[0][i] = p[(size_t)i * Dv];
+        S[1][i] = p[(size_t)i * Dv + step];
+      }
+    }
+  };
+  auto store_cols = [&](float* base) {
+    float* p = base + (size_t)r * R * Dv + j0;
+    if (j0 >= Dv) return;
+    if (even) {
+#pragma unroll
+      for (int i = 0; i < R; ++i) *(float2*)(p + (size_t)i * Dv) = make_float2(S[0][i], S[1][i]);
+    } else {
+#pragma unroll
+      for (int i = 0; i < R; ++i) p[(size_t)i * Dv] = S[0][i];
+      if (j0 + 1 < Dv) {
+#pragma unroll
+        for (int i = 0; i < R; ++i) p[(size_t)i * Dv + 1] = S[1][i];
+      }
+    }
+  };
+  const size_t head_at = ((size_t)(slot < 0 ? 0 : slot) * H + h) * D * Dv;
+  if (!compose && seg > 0) {
+    load_cols(seg_state + (((size_t)s * nseg + seg) * H + h) * D * Dv);
+  } else if (!compose && slot >= 0 && positions[r0] > 0) {
+    load_cols(state + head_at);
   } else {
-    const bool carry = slot >= 0 && positions[r0] > 0;
-    const float* sp = state + ((size_t)(slot < 0 ? 0 : slot) * H + h) * D * Dv;
 #pragma unroll
-    for (int i = 0; i < R; ++i)
-      S[i] = (carry && valid) ? sp[(size_t)(r * R + i) * Dv + j] : 0.f;
+    for (int e = 0; e < kCols; ++e)
+#pragma unroll
+      for (int i = 0; i < R; ++i)
+        S[e][i] = (ident && r * R + i == cb * W + kCols * c + e) ? 1.f : 0.f;
   }
   const float rate = -expf(a_log[h]), bias = kChannel ? 0.f : dt_bias[h];
   const float qscale = 1.0f / sqrtf((float)D);
@@ -197,31 +257,33 @@ __global__ __launch_bounds__(WAVE) void gated_delta_scan_reg_kernel(
   typedef typename Raw4<T>::type raw4;
   const int st_tt = lane >> 2, st_part = lane & 3;
   raw4 pq[kQ], pk[kQ], pg[kChannel ? kQ : 1];
-  T pv[4], pa, pb;
-  const float* db = dt_bias + (size_t)h * D + st_part * R;  // kChannel; stays in cache
+  T pv[W / 4], pa, pb;
+  // (tokens past the end repeat the last one, columns past the end too: what
+  // they stage is never used)
   auto prefetch = [&](int tile0) {
-    const int t = tile0 + st_tt;
-    if (t < s1) {
-      const T* qp = q + (size_t)t * q_stride + hk * D + st_part * R;
-      const T* kp = k + (size_t)t * k_stride + hk * D + st_part * R;
+    const int t = min(tile0 + st_tt, s1 - 1);
+    const T* qp = q + (size_t)t * q_stride + hk * D + st_part * R;
+    const T* kp = k + (size_t)t * k_stride + hk * D + st_part * R;
+#pragma unroll
+    for (int b = 0; b < kQ; ++b) {
+      pq[b] = *(const raw4*)(qp + 4 * b);
+      pk[b] = *(const raw4*)(kp + 4 * b);
+    }
+    const T* vp = v + (size_t)t * v_stride + h * Dv;
+#pragma unroll
+    for (int e = 0; e < W / 4; ++e)
+      pv[e] = vp[max(0, min(vc0 + st_part * (W / 4) + e, Dv - 1))];
+    if constexpr (!kChannel) pa = decay_pre[(size_t)t * a_stride + h];
+    pb = beta_pre[(size_t)t * b_stride + h];
+    if constexpr (kChannel) {
+      // decays: four channels a lane, dealt over the wave, so that a single
+      // decode token is activated by many lanes
 #pragma unroll
       for (int b = 0; b < kQ; ++b) {
-        pq[b] = *(const raw4*)(qp + 4 * b);
-        pk[b] = *(const raw4*)(kp + 4 * b);
-      }
-      if constexpr (kChannel) {
-        const T* gp = decay_pre + (size_t)t * a_stride + h * D + st_part * R;
-#pragma unroll
-        for (int b = 0; b < kQ; ++b) pg[b] = *(const raw4*)(gp + 4 * b);
-      }
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int col = (cb - pcb) * 16 + st_part * 4 + e;
-        pv[e] = (!ident && col < Dv) ? v[(size_t)t * v_stride + h * Dv + col] : (T)0;
-      }
-      if (st_part == 0) {
-        if constexpr (!kChannel) pa = decay_pre[(size_t)t * a_stride + h];
-        pb = beta_pre[(size_t)t * b_stride + h];
+        const int w = b * WAVE + lane, d = w % R * 4;
+        if (tile0 + b * WAVE / R < s1)  // wave-uniform
+          pg[b] = *(const raw4*)(decay_pre + (size_t)min(tile0 + w / R, s1 - 1) * a_stride +
+                                 h * D + d);
       }
     }
   };
@@ -232,120 +294,142 @@ __global__ __launch_bounds__(WAVE) void gated_delta_scan_reg_kernel(
     {
       float qa[R], ka[R];
       float sq = 0.f, sk = 0.f;
-      if (st_tt < nt) {
 #pragma unroll
-        for (int b = 0; b < kQ; ++b) {
-          cvt4(pq[b], qa + 4 * b);
-          cvt4(pk[b], ka + 4 * b);
-        }
+      for (int b = 0; b < kQ; ++b) {
+        cvt4(pq[b], qa + 4 * b);
+        cvt4(pk[b], ka + 4 * b);
+      }
 #pragma unroll
-        for (int i = 0; i < R; ++i) {
-          sq += qa[i] * qa[i];
-          sk += ka[i] * ka[i];
-        }
+      for (int i = 0; i < R; ++i) {
+        sq += qa[i] * qa[i];
+        sk += ka[i] * ka[i];
       }
       // the four lanes of a token are neighbours
       sq += __shfl_xor(sq, 1, WAVE);
       sq += __shfl_xor(sq, 2, WAVE);
       sk += __shfl_xor(sk, 1, WAVE);
       sk += __shfl_xor(sk, 2, WAVE);
-      if (st_tt < nt) {
-        const float rq = qscale / sqrtf(sq + norm_eps), rk = 1.0f / sqrtf(sk + norm_eps);
-        const int at = st_tt * D + st_part * R;
+      const float rq = qscale / sqrtf(sq + norm_eps), rk = 1.0f / sqrtf(sk + norm_eps);
+      const int at = st_tt * D + st_part * R;
+#pragma unroll
+      for (int b = 0; b < kQ; ++b) {
+        *(float4*)(qs + at + 4 * b) = make_float4(qa[4 * b] * rq, qa[4 * b + 1] * rq,
+                                                  qa[4 * b + 2] * rq, qa[4 * b + 3] * rq);
+        *(float4*)(ks + at + 4 * b) = make_float4(ka[4 * b] * rk, ka[4 * b + 1] * rk,
+                                                  ka[4 * b + 2] * rk, ka[4 * b + 3] * rk);
+      }
+#pragma unroll
+      for (int e = 0; e < W / 4; ++e)
+        vs[st_tt * W + st_part * (W / 4) + e] = ident ? 0.f : ldf(&pv[e]);
+      if (st_part == 0) {
+        if constexpr (!kChannel) gb[2 * st_tt] = expf(rate * softplus_f(ldf(&pa) + bias));
+        gb[2 * st_tt + 1] = sigmoid_f(ldf(&pb));
+      }
+      if constexpr (kChannel) {
 #pragma unroll
         for (int b = 0; b < kQ; ++b) {
-          *(float4*)(qs + at + 4 * b) = make_float4(qa[4 * b] * rq, qa[4 * b + 1] * rq,
-                                                    qa[4 * b + 2] * rq, qa[4 * b + 3] * rq);
-          *(float4*)(ks + at + 4 * b) = make_float4(ka[4 * b] * rk, ka[4 * b + 1] * rk,
-                                                    ka[4 * b + 2] * rk, ka[4 * b + 3] * rk);
-        }
-#pragma unroll
-        for (int e = 0; e < 4; ++e) vs[st_tt * 16 + st_part * 4 + e] = ldf(&pv[e]);
-        if constexpr (kChannel) {
-          float ga[R];
-#pragma unroll
-          for (int b = 0; b < kQ; ++b) cvt4(pg[b], ga + 4 * b);
-#pragma unroll
-          for (int i = 0; i < R; ++i) ga[i] = expf(rate * softplus_f(ga[i] + db[i]));
-#pragma unroll
-          for (int b = 0; b < kQ; ++b)
-            *(float4*)(gs + at + 4 * b) =
-                make_float4(ga[4 * b], ga[4 * b + 1], ga[4 * b + 2], ga[4 * b + 3]);
-        }
-        if (st_part == 0) {
-          if constexpr (!kChannel)
-            gb[2 * st_tt] = expf(rate * softplus_f(ldf(&pa) + bias));
-          gb[2 * st_tt + 1] = sigmoid_f(ldf(&pb));
+          const int w = b * WAVE + lane, d = w % R * 4;
+          if (b * WAVE / R < nt) {  // wave-uniform
+            float x[4];
+            cvt4(pg[b], x);
+            const float4 db = *(const float4*)(dt_bias + (size_t)h * D + d);
+            *(float4*)(gs + 4 * w) =
+                make_float4(decay_f(rate, x[0] + db.x), decay_f(rate, x[1] + db.y),
+                            decay_f(rate, x[2] + db.z), decay_f(rate, x[3] + db.w));
+          }
         }
       }
     }
     __syncthreads();
     if (t0 + kTile < s1) prefetch(t0 + kTile);
     for (int tt = 0; tt < nt; ++tt) {
-      const float vj = vs[tt * 16 + c];
-      const float g = kChannel ? 1.f : gb[2 * tt], beta = gb[2 * tt + 1];
+      const float2 vj = *(const float2*)(vs + tt * W + kCols * c);
+      const float beta = gb[2 * tt + 1];
       const float4* q4 = (const float4*)(qs + tt * D + r * R);
       const float4* k4 = (const float4*)(ks + tt * D + r * R);
       float ka[R];
-      float dot = 0.f;
 #pragma unroll
       for (int b = 0; b < kQ; ++b) {
         const float4 kk = k4[b];
         ka[4 * b] = kk.x; ka[4 * b + 1] = kk.y; ka[4 * b + 2] = kk.z; ka[4 * b + 3] = kk.w;
       }
+      // two partial sums per column: shorter dependence chains
+      float dot[kCols][2] = {};
       if constexpr (kChannel) {
         const float4* g4 = (const float4*)(gs + tt * D + r * R);
 #pragma unroll
         for (int b = 0; b < kQ; ++b) {
           const float4 gg = g4[b];
-          S[4 * b] *= gg.x; S[4 * b + 1] *= gg.y; S[4 * b + 2] *= gg.z; S[4 * b + 3] *= gg.w;
-        }
+          const float ga[4] = {gg.x, gg.y, gg.z, gg.w};
 #pragma unroll
-        for (int i = 0; i < R; ++i) dot += S[i] * ka[i];
+          for (int x = 0; x < 4; ++x)
+#pragma unroll
+            for (int e = 0; e < kCols; ++e) {
+              S[e][4 * b + x] *= ga[x];
+              dot[e][x & 1] += S[e][4 * b + x] * ka[4 * b + x];
+            }
+        }
       } else {
+        const float g = gb[2 * tt];
 #pragma unroll
-        for (int i = 0; i < R; ++i) {
-          S[i] *= g;
-          dot += S[i] * ka[i];
-        }
+        for (int i = 0; i < R; ++i)
+#pragma unroll
+          for (int e = 0; e < kCols; ++e) {
+            S[e][i] *= g;
+            dot[e][i & 1] += S[e][i] * ka[i];
+          }
       }
-      dot += __shfl_xor(dot, 16, WAVE);
-      dot += __shfl_xor(dot, 32, WAVE);
-      const float u = beta * (vj - dot);
-      float acc = 0.f;
+      const float u[kCols] = {beta * (vj.x - quad_sum(dot[0][0] + dot[0][1])),
+                              beta * (vj.y - quad_sum(dot[1][0] + dot[1][1]))};
+      float acc[kCols][2] = {};
 #pragma unroll
       for (int b = 0; b < kQ; ++b) {
         const float4 qq = q4[b];
         const float qa[4] = {qq.x, qq.y, qq.z, qq.w};
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          const int i = 4 * b + e;
-          S[i] += ka[i] * u;
-          acc += qa[e] * S[i];
+        for (int x = 0; x < 4; ++x) {
+          const int i = 4 * b + x;
+#pragma unroll
+          for (int e = 0; e < kCols; ++e) {
+            S[e][i] += ka[i] * u[e];
+            acc[e][x & 1] += qa[x] * S[e][i];
+          }
         }
       }
       if (!compose) {
-        acc += __shfl_xor(acc, 16, WAVE);
-        acc += __shfl_xor(acc, 32, WAVE);
-        if (r == 0 && valid) o[((size_t)(t0 + tt) * H + h) * Dv + j] = acc;
+        const float a0 = quad_sum(acc[0][0] + acc[0][1]);
+        const float a1 = quad_sum(acc[1][0] + acc[1][1]);
+        if (r == 0) {
+          float* op = o + ((size_t)(t0 + tt) * H + h) * Dv + j0;
+          if (even) {
+            if (j0 < Dv) *(float2*)op = make_float2(a0, a1);
+          } else {
+            if (j0 < Dv) op[0] = a0;
+            if (j0 + 1 < Dv) op[1] = a1;
+          }
+        }
       }
     }
   }
   if (compose) {
     const size_t sh = ((size_t)s * nseg + seg) * H + h;
     if (ident) {
-      float* pp = seg_p + sh * D * D;
 #pragma unroll
-      for (int i = 0; i < R; ++i) pp[(size_t)(cb * 16 + c) * D + r * R + i] = S[i];  // P^T
-    } else if (valid) {
-      float* bp = seg_b + sh * D * Dv;
+      for (int e = 0; e < kCols; ++e) {
+        const int col = cb * W + kCols * c + e;
+        float* pp = seg_p + sh * D * D + (size_t)col * D + r * R;  // P^T
+        if (col < D) {
 #pragma unroll
-      for (int i = 0; i < R; ++i) bp[(size_t)(r * R + i) * Dv + j] = S[i];
+          for (int b = 0; b < kQ; ++b)
+            *(float4*)(pp + 4 * b) = make_float4(S[e][4 * b], S[e][4 * b + 1], S[e][4 * b + 2],
+                                                 S[e][4 * b + 3]);
+        }
+      }
+    } else {
+      store_cols(seg_b + sh * D * Dv);
     }
-  } else if (slot >= 0 && valid && s1 == s1_run) {
-    float* sp = state + ((size_t)slot * H + h) * D * Dv;
-#pragma unroll
-    for (int i = 0; i < R; ++i) sp[(size_t)(r * R + i) * Dv + j] = S[i];
+  } else if (slot >= 0 && s1 == s1_run) {
+    store_cols(state + head_at);
   }
 }
 
@@ -401,7 +485,8 @@ void gated_delta_scan(torch::Tensor o, torch::Tensor q, torch::Tensor k,
     return ((size_t)t.data_ptr()) % bytes == 0 && t.stride(0) % 4 == 0;
   };
   if (D % 16 == 0 && D <= 128 && vec_ok(q) && vec_ok(k) && (!channel || vec_ok(decay_pre))) {
-    const int ncb = (Dv + 15) / 16;
+    constexpr int W = 16 * kCols;
+    const int ncb = (Dv + W - 1) / W;
     int seg_len, nseg;
     delta_segments(max_len, n_seq, H, D, Dv, &seg_len, &nseg);
     torch::Tensor ws_p, ws_b, ws_s;
@@ -412,7 +497,7 @@ void gated_delta_scan(torch::Tensor o, torch::Tensor q, torch::Tensor k,
     }
     SEQ_DISPATCH_ACT(q, {
       auto launch1 = [&](auto kern, int mode) {
-        const int blocks_cb = mode == 1 ? ncb + D / 16 : ncb;
+        const int blocks_cb = mode == 1 ? ncb + (D + W - 1) / W : ncb;
         hipLaunchKernelGGL(kern, dim3(n_seq * nseg * H * blocks_cb), dim3(WAVE), 0,
                            SEQ_STREAM(), (float*)o.data_ptr(),
                            (const act_t*)q.data_ptr(), q.stride(0),

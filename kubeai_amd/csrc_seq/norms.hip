@@ -60,6 +60,39 @@ __global__ __launch_bounds__(128) void gated_rmsnorm_kernel(
   }
 }
 
+// The same with `lpg` neighbouring lanes (a power of two, at most a wave) on a
+// group, four elements each: gs a multiple of four, at most 256; rows aligned.
+template <typename T>
+__global__ __launch_bounds__(256) void gated_rmsnorm_vec_kernel(
+    T* __restrict__ out, int64_t out_stride, const float* __restrict__ o,
+    const float* __restrict__ w, const T* __restrict__ gate,
+    int64_t gate_stride, int64_t n_groups, int C, int gs, int lpg, int act, float eps,
+    float out_scale) {
+  const int64_t g = (int64_t)blockIdx.x * (blockDim.x / lpg) + threadIdx.x / lpg;
+  const int i = (threadIdx.x % lpg) * 4;
+  const int groups = C / gs;
+  const bool on = g < n_groups && i < gs;
+  const int64_t t = on ? g / groups : 0;
+  const int c = on ? (int)(g % groups) * gs + i : 0;
+  float x[4] = {0.f, 0.f, 0.f, 0.f}, y[4];
+  if (on) {
+    cvt4(*(const float4*)(o + t * C + c), x);
+    cvt4(*(const typename Raw4<T>::type*)(gate + t * gate_stride + c), y);
+  }
+  float ss = x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3];
+  for (int off = lpg >> 1; off > 0; off >>= 1) ss += __shfl_xor(ss, off, WAVE);
+  if (!on) return;
+  const float r = out_scale / sqrtf(ss / (float)gs + eps);
+  float wv[4];
+  cvt4(*(const float4*)(w + c), wv);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    const float g_ = act == 1 ? sigmoid_f(y[e]) : act == 2 ? silu_f(y[e]) : y[e];
+    x[e] *= r * wv[e] * g_;
+  }
+  st4(out + t * out_stride + c, x);
+}
+
 template <typename T>
 __global__ void relu_squared_kernel(T* __restrict__ out,
                                     const T* __restrict__ x, int64_t n) {
@@ -128,6 +161,24 @@ void gated_rmsnorm(torch::Tensor out, torch::Tensor o, torch::Tensor weight,
               gate.size(1) == C && gate.scalar_type() == out.scalar_type());
   TORCH_CHECK(groups <= 65535);
   if (T == 0) return;
+  const int gs = C / groups;
+  auto al4 = [](const torch::Tensor& x) {
+    return ((size_t)x.data_ptr()) % (4 * x.element_size()) == 0 && x.stride(0) % 4 == 0;
+  };
+  if (gs % 4 == 0 && gs <= 4 * WAVE && al4(out) && al4(gate)) {
+    int lpg = 1;
+    while (lpg * 4 < gs) lpg *= 2;
+    const int64_t n = (int64_t)T * groups, per = 256 / lpg;
+    SEQ_DISPATCH_ACT(out, {
+      hipLaunchKernelGGL((gated_rmsnorm_vec_kernel<act_t>), dim3((n + per - 1) / per),
+                         dim3(256), 0, SEQ_STREAM(), (act_t*)out.data_ptr(), out.stride(0),
+                         (const float*)o.data_ptr(), (const float*)weight.data_ptr(),
+                         (const act_t*)gate.data_ptr(), gate.stride(0), n, C, gs, lpg,
+                         (int)act, (float)eps, (float)out_scale);
+    });
+    SEQ_CHECK_LAUNCH();
+    return;
+  }
   SEQ_DISPATCH_ACT(out, {
     hipLaunchKernelGGL((gated_rmsnorm_kernel<act_t>), dim3(T, groups), dim3(128),
                        0, SEQ_STREAM(), (act_t*)out.data_ptr(), out.stride(0),

@@ -43,6 +43,12 @@ DEV_INLINE void cvt4(const ushort4& v, float* o) {
   o[2] = bf16_to_f32(v.z); o[3] = bf16_to_f32(v.w);
 }
 
+DEV_INLINE void st4(float* p, const float* o) { *(float4*)p = make_float4(o[0], o[1], o[2], o[3]); }
+DEV_INLINE void st4(bf16raw* p, const float* o) {
+  *(ushort4*)p = make_ushort4(f32_to_bf16(o[0]), f32_to_bf16(o[1]), f32_to_bf16(o[2]),
+                              f32_to_bf16(o[3]));
+}
+
 // one 16-byte load: 8 bf16 or 4 fp32 activations (pointer 16-byte aligned)
 template <typename T> struct Vec16;
 template <> struct Vec16<float> {
@@ -114,6 +120,21 @@ DEV_INLINE float block_sum(float v, float* smem) {
   float total = 0.f;
   for (int w = 0; w < n_waves; ++w) total += smem[w];
   return total;
+}
+
+// Tiles of a packed step: with `size` tokens a tile, run s owns tile
+// numbers start_loc[s] / size + s and on (never fewer than it needs), so T /
+// size + n_seq blocks cover every batch, whatever its mix of lengths. Returns
+// the run of tile number b and b's place in the run.
+DEV_INLINE int find_tile(const int* start_loc, int n_seq, int size, int b, int* tile) {
+  int lo = 0, hi = n_seq - 1;  // the last run whose first number is <= b
+  while (lo < hi) {
+    const int mid = (lo + hi + 1) >> 1;
+    if (start_loc[mid] / size + mid <= b) lo = mid;
+    else hi = mid - 1;
+  }
+  *tile = b - (start_loc[lo] / size + lo);
+  return lo;
 }
 
 #define SEQ_CHECK_LAUNCH()                                                   \

@@ -5,6 +5,8 @@
 // heads, and the join of two attention maps (difference, per-head RMS norm).
 #include "seq_common.h"
 
+#include <algorithm>
+
 namespace {
 
 constexpr int kBlock = 256;
@@ -92,6 +94,75 @@ __global__ __launch_bounds__(kBlock) void hyper_mix_rmsnorm_kernel(
   const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)C + eps);
   for (int c = threadIdx.x; c < C; c += kBlock)
     stf(out + (size_t)t * C + c, row[c] * r * w[c]);
+}
+
+// The same for a fixed number of streams and C a multiple of four: 16-byte
+// accesses, blockDim (up to 1024) chosen so that a thread has one piece of most
+// rows, whose loads are all in flight at once.
+template <typename T, typename A, int S>
+__global__ __launch_bounds__(1024) void hyper_mix_rmsnorm_vec_kernel(
+    T* __restrict__ out, float* __restrict__ streams, const A* __restrict__ y,
+    const T* __restrict__ gate, int64_t gate_stride, const float* __restrict__ mix,
+    const float* __restrict__ wr, const float* __restrict__ rd,
+    const float* __restrict__ w, int C, float eps) {
+  extern __shared__ __attribute__((aligned(16))) float vrow_u[];
+  __shared__ float red[16];
+  const int t = blockIdx.x;
+  float* xs = streams + (size_t)t * S * C;
+  float cm[S][S], cw[S], cr[S];  // uniform: scalar registers
+#pragma unroll
+  for (int s = 0; s < S; ++s) {
+    cr[s] = rd[s];
+    cw[s] = y != nullptr ? wr[s] : 0.f;
+#pragma unroll
+    for (int d = 0; d < S; ++d) cm[s][d] = y != nullptr ? mix[s * S + d] : 0.f;
+  }
+  float ss = 0.f;
+  for (int c = threadIdx.x * 4; c < C; c += blockDim.x * 4) {
+    float x[S][4], u[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int s = 0; s < S; ++s) cvt4(*(const float4*)(xs + (size_t)s * C + c), x[s]);
+    if (y != nullptr) {
+      float z[4];
+      cvt4(*(const typename Raw4<A>::type*)(y + (size_t)t * C + c), z);
+      if (gate != nullptr) {
+        float g[4];
+        cvt4(*(const typename Raw4<T>::type*)(gate + (size_t)t * gate_stride + c), g);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) z[e] *= sigmoid_f(g[e]);
+      }
+#pragma unroll
+      for (int d = 0; d < S; ++d) {
+        float acc[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          acc[e] = cw[d] * z[e];
+#pragma unroll
+          for (int s = 0; s < S; ++s) acc[e] += cm[s][d] * x[s][e];
+          u[e] += cr[d] * acc[e];
+        }
+        st4(xs + (size_t)d * C + c, acc);
+      }
+    } else {
+#pragma unroll
+      for (int s = 0; s < S; ++s)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) u[e] += cr[s] * x[s][e];
+    }
+    st4(vrow_u + c, u);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss += u[e] * u[e];
+  }
+  // every thread re-reads only the entries it wrote
+  const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)C + eps);
+  for (int c = threadIdx.x * 4; c < C; c += blockDim.x * 4) {
+    float u[4], g[4];
+    cvt4(*(const float4*)(vrow_u + c), u);
+    cvt4(*(const float4*)(w + c), g);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) u[e] *= r * g[e];
+    st4(out + (size_t)t * C + c, u);
+  }
 }
 
 // grid (T). q rows are scaled in place by the temperature of their position,
@@ -229,8 +300,28 @@ void hyper_mix_rmsnorm(torch::Tensor out, torch::Tensor streams,
     };
     const float* f = nullptr;
     const act_t* n = nullptr;
-    if (wide) launch(hyper_mix_rmsnorm_kernel<act_t, float>, f);
-    else launch(hyper_mix_rmsnorm_kernel<act_t, act_t>, n);
+    const bool vec = C % 4 == 0 && gs % 4 == 0 && ((size_t)gp) % 8 == 0 &&
+                     (S == 1 || S == 2 || S == 4);
+    if (vec) {
+      const int block = std::min(1024, (C / 4 + WAVE - 1) / WAVE * WAVE);
+      auto launch_vec = [&](auto kern, auto* yt) {
+        hipLaunchKernelGGL(kern, dim3(T), dim3(block), (size_t)C * 4, SEQ_STREAM(),
+                           (act_t*)out.data_ptr(), (float*)streams.data_ptr(),
+                           (decltype(yt))yp, (const act_t*)gp, gs, mp, wp,
+                           (const float*)read_w.data_ptr(), (const float*)weight.data_ptr(),
+                           C, (float)eps);
+      };
+      if (S == 1 && wide) launch_vec(hyper_mix_rmsnorm_vec_kernel<act_t, float, 1>, f);
+      else if (S == 1) launch_vec(hyper_mix_rmsnorm_vec_kernel<act_t, act_t, 1>, n);
+      else if (S == 2 && wide) launch_vec(hyper_mix_rmsnorm_vec_kernel<act_t, float, 2>, f);
+      else if (S == 2) launch_vec(hyper_mix_rmsnorm_vec_kernel<act_t, act_t, 2>, n);
+      else if (wide) launch_vec(hyper_mix_rmsnorm_vec_kernel<act_t, float, 4>, f);
+      else launch_vec(hyper_mix_rmsnorm_vec_kernel<act_t, act_t, 4>, n);
+    } else if (wide) {
+      launch(hyper_mix_rmsnorm_kernel<act_t, float>, f);
+    } else {
+      launch(hyper_mix_rmsnorm_kernel<act_t, act_t>, n);
+    }
   });
   SEQ_CHECK_LAUNCH();
 }

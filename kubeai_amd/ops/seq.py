@@ -265,7 +265,7 @@ def causal_conv(x, w, tails, meta: SeqMeta, residual: bool, act: str = "none"):
         y = torch.empty(x.shape, dtype=x.dtype, device=x.device)
         _C.causal_conv(y, x, w, tails, meta.start_loc, meta.slots,
                        meta.token_seq, meta.positions, residual,
-                       {"none": 0, "silu": 1}[act])
+                       {"none": 0, "silu": 1}[act], meta.max_len)
         return y
     y = torch.empty(x.shape, dtype=x.dtype)
     C = x.shape[1]
