@@ -12,13 +12,14 @@
 namespace {
 
 // Fold: grid (n_seq * H * column blocks), 256 threads. A block chains
-// seg_state[i + 1] = P_i seg_state[i] + B_i for CB = 4 * (256 / (D / 4))
+// seg_state[i + 1] = P_i seg_state[i] + B_i for CB = 2 * (256 / (D / 4))
 // value columns of one head (seg_state[0] is not written: the first segment
-// starts from the slot). Every thread owns a 4 x 4 tile of the column block.
+// starts from the slot). Every thread owns a 4 x 2 tile of the column block.
 // P_i arrives transposed (seg_pt[k][i] = P_i[i][k]) and is staged in LDS as a
 // whole, fetched into registers while the previous step is computed; the
 // column block passes through LDS between the steps. Per contraction index a
-// thread reads one float4 of P^T and one of S for 16 products.
+// thread reads four numbers of P^T and two of S for 8 products. B_i is fetched
+// with P_i.
 template <int kD>
 __global__ __launch_bounds__(256) void gated_delta_fold_kernel(
     float* __restrict__ seg_state, const float* __restrict__ seg_pt,
@@ -28,7 +29,7 @@ __global__ __launch_bounds__(256) void gated_delta_fold_kernel(
     int seg_len) {
   constexpr int RT = kD / 4;                       // row tiles
   constexpr int CT = 256 / RT;                     // column tiles of a block
-  constexpr int CB = 4 * CT;                       // columns of a block
+  constexpr int CB = 2 * CT;                       // columns of a block
   constexpr int PV = (kD * kD / 4 + 255) / 256;    // float4 of P per thread
   extern __shared__ __attribute__((aligned(16))) float fold_sm[];
   float* pt = fold_sm;            // [kD][kD]
@@ -42,24 +43,31 @@ __global__ __launch_bounds__(256) void gated_delta_fold_kernel(
   const int tid = threadIdx.x;
   const int rt = tid % RT, ct = tid / RT;
   const bool active = ct < CT;
-  const int i0 = rt * 4, c0 = ct * 4, j0 = cb * CB + c0;
+  const int i0 = rt * 4, c0 = ct * 2, j0 = cb * CB + c0;
   const bool carry = slot >= 0 && positions[r0] > 0;
   const float* sp = state + ((size_t)(slot < 0 ? 0 : slot) * H + h) * kD * Dv;
-  float S[4][4];
+  float S[4][2], nb[4][2];
 #pragma unroll
   for (int a = 0; a < 4; ++a)
 #pragma unroll
-    for (int b = 0; b < 4; ++b)
+    for (int b = 0; b < 2; ++b)
       S[a][b] = (carry && active && j0 + b < Dv) ? sp[(size_t)(i0 + a) * Dv + j0 + b] : 0.f;
-  float4 pre[PV];
+  typedef __attribute__((ext_vector_type(4))) float f4;  // stays in registers
+  f4 pre[PV];
   auto fetch = [&](int seg) {
-    const float4* src =
-        (const float4*)(seg_pt + (((size_t)s * nseg + seg) * H + h) * kD * kD);
+    const f4* src =
+        (const f4*)(seg_pt + (((size_t)s * nseg + seg) * H + h) * kD * kD);
 #pragma unroll
     for (int v = 0; v < PV; ++v) {
       const int idx = v * 256 + tid;
       if (idx < kD * kD / 4) pre[v] = src[idx];
     }
+    const float* bp = seg_b + (((size_t)s * nseg + seg) * H + h) * kD * Dv;
+#pragma unroll
+    for (int a = 0; a < 4; ++a)
+#pragma unroll
+      for (int b = 0; b < 2; ++b)
+        nb[a][b] = (active && j0 + b < Dv) ? bp[(size_t)(i0 + a) * Dv + j0 + b] : 0.f;
   };
   fetch(0);
   for (int seg = 0; seg + 1 < used; ++seg) {
@@ -68,38 +76,36 @@ __global__ __launch_bounds__(256) void gated_delta_fold_kernel(
 #pragma unroll
     for (int v = 0; v < PV; ++v) {
       const int idx = v * 256 + tid;
-      if (idx < kD * kD / 4) ((float4*)pt)[idx] = pre[v];
+      if (idx < kD * kD / 4) ((f4*)pt)[idx] = pre[v];
     }
     if (active) {
 #pragma unroll
       for (int a = 0; a < 4; ++a)
-        *(float4*)(sc + (i0 + a) * CB + c0) = make_float4(S[a][0], S[a][1], S[a][2], S[a][3]);
+        *(float2*)(sc + (i0 + a) * CB + c0) = make_float2(S[a][0], S[a][1]);
     }
     __syncthreads();
+#pragma unroll
+    for (int a = 0; a < 4; ++a)
+#pragma unroll
+      for (int b = 0; b < 2; ++b) S[a][b] = nb[a][b];
     if (seg + 2 < used) fetch(seg + 1);
     if (active) {
-      const float* bp = seg_b + sh * kD * Dv;
-#pragma unroll
-      for (int a = 0; a < 4; ++a)
-#pragma unroll
-        for (int b = 0; b < 4; ++b)
-          S[a][b] = j0 + b < Dv ? bp[(size_t)(i0 + a) * Dv + j0 + b] : 0.f;
 #pragma unroll 4
       for (int k = 0; k < kD; ++k) {
         const float4 p = *(const float4*)(pt + k * kD + i0);
-        const float4 x = *(const float4*)(sc + k * CB + c0);
+        const float2 x = *(const float2*)(sc + k * CB + c0);
         const float pa[4] = {p.x, p.y, p.z, p.w};
-        const float xa[4] = {x.x, x.y, x.z, x.w};
+        const float xa[2] = {x.x, x.y};
 #pragma unroll
         for (int a = 0; a < 4; ++a)
 #pragma unroll
-          for (int b = 0; b < 4; ++b) S[a][b] += pa[a] * xa[b];
+          for (int b = 0; b < 2; ++b) S[a][b] += pa[a] * xa[b];
       }
       float* out = seg_state + (sh + H) * kD * Dv;  // segment seg + 1
 #pragma unroll
       for (int a = 0; a < 4; ++a)
 #pragma unroll
-        for (int b = 0; b < 4; ++b)
+        for (int b = 0; b < 2; ++b)
           if (j0 + b < Dv) out[(size_t)(i0 + a) * Dv + j0 + b] = S[a][b];
     }
   }
@@ -133,7 +139,7 @@ static inline void delta_fold_launch_one(K kern, int D, int n_seq, int H, int Dv
                                          torch::Tensor& ws_p, torch::Tensor& ws_b,
                                          torch::Tensor& state, torch::Tensor& start_loc,
                                          torch::Tensor& slots, torch::Tensor& positions) {
-  const int cbk = 4 * (256 / (D / 4));  // value columns of a fold block
+  const int cbk = 2 * (256 / (D / 4));  // value columns of a fold block
   const int ncbk = (Dv + cbk - 1) / cbk;
   const size_t fold_lds = ((size_t)D * D + (size_t)D * cbk) * sizeof(float);
   // raise the dynamic-LDS cap once per kernel, outside any capture

@@ -140,32 +140,67 @@ DEV_INLINE float decay_f(float rate, float x) {
   return __builtin_amdgcn_exp2f(rate * kL2e * sp);
 }
 
-// sum over the four lanes 16 apart, in every one of them
-DEV_INLINE float quad_sum(float x) {
-  const unsigned a = __builtin_bit_cast(unsigned, x);
-  const auto p = __builtin_amdgcn_permlane16_swap(a, a, false, false);
-  x = __builtin_bit_cast(float, (unsigned)p[0]) + __builtin_bit_cast(float, (unsigned)p[1]);
-  const unsigned b = __builtin_bit_cast(unsigned, x);
-  const auto q = __builtin_amdgcn_permlane32_swap(b, b, false, false);
-  return __builtin_bit_cast(float, (unsigned)q[0]) + __builtin_bit_cast(float, (unsigned)q[1]);
+// A wave is eight lane groups r = lane / 8 of eight lanes c; every lane brings
+// partial sums x[0..3] of its group. Returns, in the 16-lane row e of the wave,
+// the total of x[e] over the eight groups that share c.
+DEV_INLINE float sum_to_rows(const float* x) {
+  auto bits = [](float f) { return __builtin_bit_cast(unsigned, f); };
+  auto flt = [](unsigned u) { return __builtin_bit_cast(float, u); };
+  const auto a = __builtin_amdgcn_permlane32_swap(bits(x[0]), bits(x[2]), false, false);
+  const auto b = __builtin_amdgcn_permlane32_swap(bits(x[1]), bits(x[3]), false, false);
+  const float y0 = flt(a[0]) + flt(a[1]);  // halves of the wave: columns 0, 2
+  const float y1 = flt(b[0]) + flt(b[1]);  // 1, 3
+  const auto z = __builtin_amdgcn_permlane16_swap(bits(y0), bits(y1), false, false);
+  const float t = flt(z[0]) + flt(z[1]);
+  const int other = __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, t), 0x128, 0xf, 0xf,
+                                                false);  // eight lanes on in the row
+  return t + __builtin_bit_cast(float, other);
 }
 
-constexpr int kCols = 2;  // value columns of a lane (register-state kernel)
+// the inverse way: row e's value in u[e] of every lane with the same c
+DEV_INLINE void rows_to_all(float x, float* u) {
+  const unsigned v = __builtin_bit_cast(unsigned, x);
+  const auto a = __builtin_amdgcn_permlane16_swap(v, v, false, false);
+  const auto even = __builtin_amdgcn_permlane32_swap(a[0], a[0], false, false);
+  const auto odd = __builtin_amdgcn_permlane32_swap(a[1], a[1], false, false);
+  u[0] = __builtin_bit_cast(float, (unsigned)even[0]);
+  u[1] = __builtin_bit_cast(float, (unsigned)odd[0]);
+  u[2] = __builtin_bit_cast(float, (unsigned)even[1]);
+  u[3] = __builtin_bit_cast(float, (unsigned)odd[1]);
+}
+
+// kN floats from LDS in the widest pieces that kN allows
+template <int kN>
+DEV_INLINE void lds_read_n(const float* p, float* x) {
+  if constexpr (kN % 4 == 0) {
+#pragma unroll
+    for (int b = 0; b < kN; b += 4) cvt4(*(const float4*)(p + b), x + b);
+  } else {
+#pragma unroll
+    for (int b = 0; b < kN; b += 2) {
+      const float2 v = *(const float2*)(p + b);
+      x[b] = v.x;
+      x[b + 1] = v.y;
+    }
+  }
+}
+
+constexpr int kCols = 4;  // value columns of a lane (register-state kernel)
 
 // Register-state form for key sizes D = 16 * kQ (<= 128). One wave per block
-// owns 16 kCols columns of one head's state over one segment of one run: lane
-// (r, c) keeps rows [r D/4, (r+1) D/4) of columns kCols c .. in registers, so
-// what a token brings (k, q, decays) is read from LDS once for all of them, a
-// token costs two passes over the registers, and the sums over the four lanes
-// of a column (the dot with k before the write, the one with q after it) are
-// lane swaps. q, k of kTile tokens are staged through LDS, normalised once per
+// owns 32 columns of one head's state over one segment of one run: lane (r, c)
+// of 8 x 8 keeps rows [r D/8, (r+1) D/8) of columns 4c..4c+3 in registers, so
+// what a token brings (k, q, decays) is read from LDS once for four columns. A
+// token costs two passes over the registers; the sums over a column's eight
+// lanes (the dot with k before the write, the one with q after it) are lane
+// swaps that leave one column's total to every lane. q, k of kTile tokens are staged through LDS, normalised once per
 // token (and per-channel decays, activated once per token); the next tile is
 // fetched into registers while the current one is walked.
 //
 // mode 0 (walk): columns are value columns; the segment starts from the
 //   slot's state (first segment), or from seg_state[seg] (later ones);
 //   writes o, and the slot's state after the run's last segment.
-// mode 1 (compose): the first ceil(D / 16 kCols) column blocks are columns of
+// mode 1 (compose): the first ceil(D / 32) column blocks are columns of
 //   the identity walked with zero values (-> seg_p, stored transposed), the
 //   rest value columns walked from zero (-> seg_b); the run's last segment is
 //   skipped.
@@ -181,7 +216,7 @@ __global__ __launch_bounds__(WAVE, 2) void gated_delta_scan_reg_kernel(
     int Dv, int ncb, float norm_eps, int nseg, int seg_len, int mode,
     float* __restrict__ seg_p, float* __restrict__ seg_b,
     const float* __restrict__ seg_state) {
-  constexpr int R = 4 * kQ, D = 4 * R, W = 16 * kCols;
+  constexpr int D = 16 * kQ, R = D / 8, QR = D / 4, W = 8 * kCols;
   const int cb = blockIdx.x % ncb;
   const int h = (blockIdx.x / ncb) % H;
   const int seg = (blockIdx.x / (ncb * H)) % nseg;
@@ -198,45 +233,43 @@ __global__ __launch_bounds__(WAVE, 2) void gated_delta_scan_reg_kernel(
   __shared__ __attribute__((aligned(16))) float gs[kChannel ? kTile * D : 4];
   __shared__ __attribute__((aligned(16))) float vs[kTile * W];
   __shared__ float gb[kTile * 2];
-  const int lane = threadIdx.x, r = lane >> 4, c = lane & 15;
+  const int lane = threadIdx.x, r = lane >> 3, c = lane & 7;
   // compose: the first column blocks walk the identity
   const int pcb = compose ? (D + W - 1) / W : 0;
   const bool ident = cb < pcb;
   const int vc0 = (cb - pcb) * W;       // the block's first value column (when not ident)
   const int j0 = vc0 + kCols * c;       // the lane's
-  const bool even = Dv % kCols == 0;    // whole pairs: aligned, all or none valid
+  const bool whole = Dv % kCols == 0;   // a lane's columns are aligned, all or none valid
   float S[kCols][R];
   auto load_cols = [&](const float* base) {
-    const float* p = base + (size_t)r * R * Dv + min(j0, Dv - 1);
-    if (even && j0 < Dv) {
+    const float* p = base + (size_t)r * R * Dv;
+    if (whole && j0 < Dv) {
 #pragma unroll
       for (int i = 0; i < R; ++i) {
-        const float2 x = *(const float2*)(p + (size_t)i * Dv);
-        S[0][i] = x.x;
-        S[1][i] = x.y;
+        const float4 x = *(const float4*)(p + (size_t)i * Dv + j0);
+        S[0][i] = x.x; S[1][i] = x.y; S[2][i] = x.z; S[3][i] = x.w;
       }
-    } else {
-      const int step = j0 + 1 < Dv ? 1 : 0;  // columns past the end are never stored
+    } else {  // columns past the end repeat the last one and are never stored
 #pragma unroll
-      for (int i = 0; i < R; ++i) {
-        S[0][i] = p[(size_t)i * Dv];
-        S[1][i] = p[(size_t)i * Dv + step];
-      }
+      for (int i = 0; i < R; ++i)
+#pragma unroll
+        for (int e = 0; e < kCols; ++e) S[e][i] = p[(size_t)i * Dv + min(j0 + e, Dv - 1)];
     }
   };
   auto store_cols = [&](float* base) {
     float* p = base + (size_t)r * R * Dv + j0;
     if (j0 >= Dv) return;
-    if (even) {
+    if (whole) {
 #pragma unroll
-      for (int i = 0; i < R; ++i) *(float2*)(p + (size_t)i * Dv) = make_float2(S[0][i], S[1][i]);
+      for (int i = 0; i < R; ++i)
+        *(float4*)(p + (size_t)i * Dv) = make_float4(S[0][i], S[1][i], S[2][i], S[3][i]);
     } else {
 #pragma unroll
-      for (int i = 0; i < R; ++i) p[(size_t)i * Dv] = S[0][i];
-      if (j0 + 1 < Dv) {
+      for (int e = 0; e < kCols; ++e)
+        if (j0 + e < Dv) {
 #pragma unroll
-        for (int i = 0; i < R; ++i) p[(size_t)i * Dv + 1] = S[1][i];
-      }
+          for (int i = 0; i < R; ++i) p[(size_t)i * Dv + e] = S[e][i];
+        }
     }
   };
   const size_t head_at = ((size_t)(slot < 0 ? 0 : slot) * H + h) * D * Dv;
@@ -262,8 +295,8 @@ __global__ __launch_bounds__(WAVE, 2) void gated_delta_scan_reg_kernel(
   // they stage is never used)
   auto prefetch = [&](int tile0) {
     const int t = min(tile0 + st_tt, s1 - 1);
-    const T* qp = q + (size_t)t * q_stride + hk * D + st_part * R;
-    const T* kp = k + (size_t)t * k_stride + hk * D + st_part * R;
+    const T* qp = q + (size_t)t * q_stride + hk * D + st_part * QR;
+    const T* kp = k + (size_t)t * k_stride + hk * D + st_part * QR;
 #pragma unroll
     for (int b = 0; b < kQ; ++b) {
       pq[b] = *(const raw4*)(qp + 4 * b);
@@ -280,9 +313,9 @@ __global__ __launch_bounds__(WAVE, 2) void gated_delta_scan_reg_kernel(
       // decode token is activated by many lanes
 #pragma unroll
       for (int b = 0; b < kQ; ++b) {
-        const int w = b * WAVE + lane, d = w % R * 4;
-        if (tile0 + b * WAVE / R < s1)  // wave-uniform
-          pg[b] = *(const raw4*)(decay_pre + (size_t)min(tile0 + w / R, s1 - 1) * a_stride +
+        const int w = b * WAVE + lane, d = w % QR * 4;
+        if (tile0 + b * WAVE / QR < s1)  // wave-uniform
+          pg[b] = *(const raw4*)(decay_pre + (size_t)min(tile0 + w / QR, s1 - 1) * a_stride +
                                  h * D + d);
       }
     }
@@ -292,7 +325,7 @@ __global__ __launch_bounds__(WAVE, 2) void gated_delta_scan_reg_kernel(
     const int nt = min(kTile, s1 - t0);
     __syncthreads();
     {
-      float qa[R], ka[R];
+      float qa[QR], ka[QR];
       float sq = 0.f, sk = 0.f;
 #pragma unroll
       for (int b = 0; b < kQ; ++b) {
@@ -300,7 +333,7 @@ __global__ __launch_bounds__(WAVE, 2) void gated_delta_scan_reg_kernel(
         cvt4(pk[b], ka + 4 * b);
       }
 #pragma unroll
-      for (int i = 0; i < R; ++i) {
+      for (int i = 0; i < QR; ++i) {
         sq += qa[i] * qa[i];
         sk += ka[i] * ka[i];
       }
@@ -310,7 +343,7 @@ __global__ __launch_bounds__(WAVE, 2) void gated_delta_scan_reg_kernel(
       sk += __shfl_xor(sk, 1, WAVE);
       sk += __shfl_xor(sk, 2, WAVE);
       const float rq = qscale / sqrtf(sq + norm_eps), rk = 1.0f / sqrtf(sk + norm_eps);
-      const int at = st_tt * D + st_part * R;
+      const int at = st_tt * D + st_part * QR;
 #pragma unroll
       for (int b = 0; b < kQ; ++b) {
         *(float4*)(qs + at + 4 * b) = make_float4(qa[4 * b] * rq, qa[4 * b + 1] * rq,
@@ -328,8 +361,8 @@ __global__ __launch_bounds__(WAVE, 2) void gated_delta_scan_reg_kernel(
       if constexpr (kChannel) {
 #pragma unroll
         for (int b = 0; b < kQ; ++b) {
-          const int w = b * WAVE + lane, d = w % R * 4;
-          if (b * WAVE / R < nt) {  // wave-uniform
+          const int w = b * WAVE + lane, d = w % QR * 4;
+          if (b * WAVE / QR < nt) {  // wave-uniform
             float x[4];
             cvt4(pg[b], x);
             const float4 db = *(const float4*)(dt_bias + (size_t)h * D + d);
@@ -343,71 +376,34 @@ __global__ __launch_bounds__(WAVE, 2) void gated_delta_scan_reg_kernel(
     __syncthreads();
     if (t0 + kTile < s1) prefetch(t0 + kTile);
     for (int tt = 0; tt < nt; ++tt) {
-      const float2 vj = *(const float2*)(vs + tt * W + kCols * c);
+      const float vj = vs[tt * W + kCols * c + (lane >> 4)];  // the lane's total's column
       const float beta = gb[2 * tt + 1];
-      const float4* q4 = (const float4*)(qs + tt * D + r * R);
-      const float4* k4 = (const float4*)(ks + tt * D + r * R);
-      float ka[R];
+      float ka[R], ga[kChannel ? R : 1], qa[R];
+      lds_read_n<R>(ks + tt * D + r * R, ka);
+      if constexpr (kChannel) lds_read_n<R>(gs + tt * D + r * R, ga);
+      lds_read_n<R>(qs + tt * D + r * R, qa);
+      const float g = kChannel ? 1.f : gb[2 * tt];
+      float dot[kCols] = {0.f, 0.f, 0.f, 0.f}, u[kCols];
 #pragma unroll
-      for (int b = 0; b < kQ; ++b) {
-        const float4 kk = k4[b];
-        ka[4 * b] = kk.x; ka[4 * b + 1] = kk.y; ka[4 * b + 2] = kk.z; ka[4 * b + 3] = kk.w;
-      }
-      // two partial sums per column: shorter dependence chains
-      float dot[kCols][2] = {};
-      if constexpr (kChannel) {
-        const float4* g4 = (const float4*)(gs + tt * D + r * R);
+      for (int i = 0; i < R; ++i)
 #pragma unroll
-        for (int b = 0; b < kQ; ++b) {
-          const float4 gg = g4[b];
-          const float ga[4] = {gg.x, gg.y, gg.z, gg.w};
-#pragma unroll
-          for (int x = 0; x < 4; ++x)
-#pragma unroll
-            for (int e = 0; e < kCols; ++e) {
-              S[e][4 * b + x] *= ga[x];
-              dot[e][x & 1] += S[e][4 * b + x] * ka[4 * b + x];
-            }
+        for (int e = 0; e < kCols; ++e) {
+          S[e][i] *= kChannel ? ga[kChannel ? i : 0] : g;
+          dot[e] += S[e][i] * ka[i];
         }
-      } else {
-        const float g = gb[2 * tt];
+      rows_to_all(beta * (vj - sum_to_rows(dot)), u);
+      float acc[kCols] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int i = 0; i < R; ++i)
+      for (int i = 0; i < R; ++i)
 #pragma unroll
-          for (int e = 0; e < kCols; ++e) {
-            S[e][i] *= g;
-            dot[e][i & 1] += S[e][i] * ka[i];
-          }
-      }
-      const float u[kCols] = {beta * (vj.x - quad_sum(dot[0][0] + dot[0][1])),
-                              beta * (vj.y - quad_sum(dot[1][0] + dot[1][1]))};
-      float acc[kCols][2] = {};
-#pragma unroll
-      for (int b = 0; b < kQ; ++b) {
-        const float4 qq = q4[b];
-        const float qa[4] = {qq.x, qq.y, qq.z, qq.w};
-#pragma unroll
-        for (int x = 0; x < 4; ++x) {
-          const int i = 4 * b + x;
-#pragma unroll
-          for (int e = 0; e < kCols; ++e) {
-            S[e][i] += ka[i] * u[e];
-            acc[e][x & 1] += qa[x] * S[e][i];
-          }
+        for (int e = 0; e < kCols; ++e) {
+          S[e][i] += ka[i] * u[e];
+          acc[e] += qa[i] * S[e][i];
         }
-      }
       if (!compose) {
-        const float a0 = quad_sum(acc[0][0] + acc[0][1]);
-        const float a1 = quad_sum(acc[1][0] + acc[1][1]);
-        if (r == 0) {
-          float* op = o + ((size_t)(t0 + tt) * H + h) * Dv + j0;
-          if (even) {
-            if (j0 < Dv) *(float2*)op = make_float2(a0, a1);
-          } else {
-            if (j0 < Dv) op[0] = a0;
-            if (j0 + 1 < Dv) op[1] = a1;
-          }
-        }
+        const float total = sum_to_rows(acc);
+        const int col = j0 + (lane >> 4);
+        if ((lane & 8) == 0 && col < Dv) o[((size_t)(t0 + tt) * H + h) * Dv + col] = total;
       }
     }
   }
@@ -420,9 +416,7 @@ __global__ __launch_bounds__(WAVE, 2) void gated_delta_scan_reg_kernel(
         float* pp = seg_p + sh * D * D + (size_t)col * D + r * R;  // P^T
         if (col < D) {
 #pragma unroll
-          for (int b = 0; b < kQ; ++b)
-            *(float4*)(pp + 4 * b) = make_float4(S[e][4 * b], S[e][4 * b + 1], S[e][4 * b + 2],
-                                                 S[e][4 * b + 3]);
+          for (int i = 0; i < R; i += 2) *(float2*)(pp + i) = make_float2(S[e][i], S[e][i + 1]);
         }
       }
     } else {
@@ -485,7 +479,7 @@ void gated_delta_scan(torch::Tensor o, torch::Tensor q, torch::Tensor k,
     return ((size_t)t.data_ptr()) % bytes == 0 && t.stride(0) % 4 == 0;
   };
   if (D % 16 == 0 && D <= 128 && vec_ok(q) && vec_ok(k) && (!channel || vec_ok(decay_pre))) {
-    constexpr int W = 16 * kCols;
+    constexpr int W = 8 * kCols;
     const int ncb = (Dv + W - 1) / W;
     int seg_len, nseg;
     delta_segments(max_len, n_seq, H, D, Dv, &seg_len, &nseg);
