@@ -169,7 +169,30 @@ DEV_INLINE void rows_to_all(float x, float* u) {
   u[3] = __builtin_bit_cast(float, (unsigned)odd[1]);
 }
 
-// kN floats from LDS in the widest pieces that kN allows
+// the raw pieces of a row: four activations, or two where rows only divide so
+template <typename T, int kN> struct RawN { typedef typename Raw4<T>::type type; };
+template <> struct RawN<float, 2> { typedef float2 type; };
+template <> struct RawN<bf16raw, 2> { typedef ushort2 type; };
+DEV_INLINE void cvt_n(const float4& v, float* o) { cvt4(v, o); }
+DEV_INLINE void cvt_n(const ushort4& v, float* o) { cvt4(v, o); }
+DEV_INLINE void cvt_n(const float2& v, float* o) { o[0] = v.x; o[1] = v.y; }
+DEV_INLINE void cvt_n(const ushort2& v, float* o) {
+  o[0] = bf16_to_f32(v.x);
+  o[1] = bf16_to_f32(v.y);
+}
+
+// kN floats to LDS, or from it, in the widest pieces that kN allows
+template <int kN>
+DEV_INLINE void lds_write_n(float* p, const float* x) {
+  if constexpr (kN % 4 == 0) {
+#pragma unroll
+    for (int b = 0; b < kN; b += 4) st4(p + b, x + b);
+  } else {
+#pragma unroll
+    for (int b = 0; b < kN; b += 2) *(float2*)(p + b) = make_float2(x[b], x[b + 1]);
+  }
+}
+
 template <int kN>
 DEV_INLINE void lds_read_n(const float* p, float* x) {
   if constexpr (kN % 4 == 0) {
@@ -193,7 +216,7 @@ constexpr int kCols = 4;  // value columns of a lane (register-state kernel)
 // what a token brings (k, q, decays) is read from LDS once for four columns. A
 // token costs two passes over the registers; the sums over a column's eight
 // lanes (the dot with k before the write, the one with q after it) are lane
-// swaps that leave one column's total to every lane. q, k of kTile tokens are staged through LDS, normalised once per
+// swaps that leave one column's total to every lane. q, k of kTok tokens are staged through LDS, normalised once per
 // token (and per-channel decays, activated once per token); the next tile is
 // fetched into registers while the current one is walked.
 //
@@ -216,7 +239,11 @@ __global__ __launch_bounds__(WAVE, 2) void gated_delta_scan_reg_kernel(
     int Dv, int ncb, float norm_eps, int nseg, int seg_len, int mode,
     float* __restrict__ seg_p, float* __restrict__ seg_b,
     const float* __restrict__ seg_state) {
-  constexpr int D = 16 * kQ, R = D / 8, QR = D / 4, W = 8 * kCols;
+  constexpr int D = 16 * kQ, R = D / 8, W = 8 * kCols;
+  // tokens staged per barrier: with per-channel decays in LDS too, fewer, so that
+  // LDS holds as many blocks as the registers do
+  constexpr int kTok = kChannel ? 8 : 16;
+  constexpr int kPart = WAVE / kTok, SR = D / kPart;  // lanes of a token, rows of a lane
   const int cb = blockIdx.x % ncb;
   const int h = (blockIdx.x / ncb) % H;
   const int seg = (blockIdx.x / (ncb * H)) % nseg;
@@ -228,11 +255,12 @@ __global__ __launch_bounds__(WAVE, 2) void gated_delta_scan_reg_kernel(
   if (s0 >= s1_run) return;
   const bool compose = mode == 1;
   if (compose && s1 == s1_run) return;
-  __shared__ __attribute__((aligned(16))) float qs[kTile * D];
-  __shared__ __attribute__((aligned(16))) float ks[kTile * D];
-  __shared__ __attribute__((aligned(16))) float gs[kChannel ? kTile * D : 4];
-  __shared__ __attribute__((aligned(16))) float vs[kTile * W];
-  __shared__ float gb[kTile * 2];
+  __shared__ __attribute__((aligned(16))) float qs[kTok * D];
+  __shared__ __attribute__((aligned(16))) float ks[kTok * D];
+  __shared__ __attribute__((aligned(16))) float gs[kChannel ? kTok * D : 4];
+  __shared__ __attribute__((aligned(16))) float db[kChannel ? D : 4];  // the head's dt_bias
+  __shared__ __attribute__((aligned(16))) float vs[kTok * W];
+  __shared__ float gb[kTok * 2];
   const int lane = threadIdx.x, r = lane >> 3, c = lane & 7;
   // compose: the first column blocks walk the identity
   const int pcb = compose ? (D + W - 1) / W : 0;
@@ -286,95 +314,101 @@ __global__ __launch_bounds__(WAVE, 2) void gated_delta_scan_reg_kernel(
   }
   const float rate = -expf(a_log[h]), bias = kChannel ? 0.f : dt_bias[h];
   const float qscale = 1.0f / sqrtf((float)D);
-  // staging: lane (st_tt, st_part) owns a quarter row of one token of the tile
+  // staging: lane (st_tt, st_part) owns SR rows of one token of the tile, in
+  // pieces of VN elements
+  constexpr int VN = SR % 4 == 0 ? 4 : 2, NV = SR / VN;
+  typedef typename RawN<T, VN>::type rawn;
   typedef typename Raw4<T>::type raw4;
-  const int st_tt = lane >> 2, st_part = lane & 3;
-  raw4 pq[kQ], pk[kQ], pg[kChannel ? kQ : 1];
-  T pv[W / 4], pa, pb;
+  constexpr int kPieces = kTok * D / 4;  // of four decays, dealt over the wave
+  constexpr int NG = (kPieces + WAVE - 1) / WAVE;
+  const int st_tt = lane / kPart, st_part = lane % kPart;
+  rawn pq[NV], pk[NV];
+  raw4 pg[kChannel ? NG : 1];
+  T pv[W / kPart], pa, pb;
   // (tokens past the end repeat the last one, columns past the end too: what
   // they stage is never used)
   auto prefetch = [&](int tile0) {
     const int t = min(tile0 + st_tt, s1 - 1);
-    const T* qp = q + (size_t)t * q_stride + hk * D + st_part * QR;
-    const T* kp = k + (size_t)t * k_stride + hk * D + st_part * QR;
+    const T* qp = q + (size_t)t * q_stride + hk * D + st_part * SR;
+    const T* kp = k + (size_t)t * k_stride + hk * D + st_part * SR;
 #pragma unroll
-    for (int b = 0; b < kQ; ++b) {
-      pq[b] = *(const raw4*)(qp + 4 * b);
-      pk[b] = *(const raw4*)(kp + 4 * b);
+    for (int n = 0; n < NV; ++n) {
+      pq[n] = *(const rawn*)(qp + VN * n);
+      pk[n] = *(const rawn*)(kp + VN * n);
     }
     const T* vp = v + (size_t)t * v_stride + h * Dv;
 #pragma unroll
-    for (int e = 0; e < W / 4; ++e)
-      pv[e] = vp[max(0, min(vc0 + st_part * (W / 4) + e, Dv - 1))];
+    for (int e = 0; e < W / kPart; ++e)
+      pv[e] = vp[max(0, min(vc0 + st_part * (W / kPart) + e, Dv - 1))];
     if constexpr (!kChannel) pa = decay_pre[(size_t)t * a_stride + h];
     pb = beta_pre[(size_t)t * b_stride + h];
     if constexpr (kChannel) {
-      // decays: four channels a lane, dealt over the wave, so that a single
-      // decode token is activated by many lanes
 #pragma unroll
-      for (int b = 0; b < kQ; ++b) {
-        const int w = b * WAVE + lane, d = w % QR * 4;
-        if (tile0 + b * WAVE / QR < s1)  // wave-uniform
-          pg[b] = *(const raw4*)(decay_pre + (size_t)min(tile0 + w / QR, s1 - 1) * a_stride +
+      for (int n = 0; n < NG; ++n) {
+        const int w = n * WAVE + lane, tt = w / (D / 4), d = w % (D / 4) * 4;
+        if (tile0 + n * WAVE / (D / 4) < s1)  // wave-uniform
+          pg[n] = *(const raw4*)(decay_pre + (size_t)min(tile0 + tt, s1 - 1) * a_stride +
                                  h * D + d);
       }
     }
   };
   prefetch(s0);
-  for (int t0 = s0; t0 < s1; t0 += kTile) {
-    const int nt = min(kTile, s1 - t0);
+  if constexpr (kChannel)
+    for (int d = lane; d < D; d += WAVE) db[d] = dt_bias[(size_t)h * D + d];
+  for (int t0 = s0; t0 < s1; t0 += kTok) {
+    const int nt = min(kTok, s1 - t0);
     __syncthreads();
     {
-      float qa[QR], ka[QR];
+      float qa[SR], ka[SR];
       float sq = 0.f, sk = 0.f;
 #pragma unroll
-      for (int b = 0; b < kQ; ++b) {
-        cvt4(pq[b], qa + 4 * b);
-        cvt4(pk[b], ka + 4 * b);
+      for (int n = 0; n < NV; ++n) {
+        cvt_n(pq[n], qa + VN * n);
+        cvt_n(pk[n], ka + VN * n);
       }
 #pragma unroll
-      for (int i = 0; i < QR; ++i) {
+      for (int i = 0; i < SR; ++i) {
         sq += qa[i] * qa[i];
         sk += ka[i] * ka[i];
       }
-      // the four lanes of a token are neighbours
-      sq += __shfl_xor(sq, 1, WAVE);
-      sq += __shfl_xor(sq, 2, WAVE);
-      sk += __shfl_xor(sk, 1, WAVE);
-      sk += __shfl_xor(sk, 2, WAVE);
-      const float rq = qscale / sqrtf(sq + norm_eps), rk = 1.0f / sqrtf(sk + norm_eps);
-      const int at = st_tt * D + st_part * QR;
+      // the lanes of a token are neighbours
 #pragma unroll
-      for (int b = 0; b < kQ; ++b) {
-        *(float4*)(qs + at + 4 * b) = make_float4(qa[4 * b] * rq, qa[4 * b + 1] * rq,
-                                                  qa[4 * b + 2] * rq, qa[4 * b + 3] * rq);
-        *(float4*)(ks + at + 4 * b) = make_float4(ka[4 * b] * rk, ka[4 * b + 1] * rk,
-                                                  ka[4 * b + 2] * rk, ka[4 * b + 3] * rk);
+      for (int x = 1; x < kPart; x *= 2) {
+        sq += __shfl_xor(sq, x, WAVE);
+        sk += __shfl_xor(sk, x, WAVE);
       }
+      const float rq = qscale / sqrtf(sq + norm_eps), rk = 1.0f / sqrtf(sk + norm_eps);
 #pragma unroll
-      for (int e = 0; e < W / 4; ++e)
-        vs[st_tt * W + st_part * (W / 4) + e] = ident ? 0.f : ldf(&pv[e]);
+      for (int i = 0; i < SR; ++i) {
+        qa[i] *= rq;
+        ka[i] *= rk;
+      }
+      lds_write_n<SR>(qs + st_tt * D + st_part * SR, qa);
+      lds_write_n<SR>(ks + st_tt * D + st_part * SR, ka);
+#pragma unroll
+      for (int e = 0; e < W / kPart; ++e)
+        vs[st_tt * W + st_part * (W / kPart) + e] = ident ? 0.f : ldf(&pv[e]);
       if (st_part == 0) {
         if constexpr (!kChannel) gb[2 * st_tt] = expf(rate * softplus_f(ldf(&pa) + bias));
         gb[2 * st_tt + 1] = sigmoid_f(ldf(&pb));
       }
       if constexpr (kChannel) {
 #pragma unroll
-        for (int b = 0; b < kQ; ++b) {
-          const int w = b * WAVE + lane, d = w % QR * 4;
-          if (b * WAVE / QR < nt) {  // wave-uniform
+        for (int n = 0; n < NG; ++n) {
+          const int w = n * WAVE + lane, d = w % (D / 4) * 4;
+          if (n * WAVE / (D / 4) < nt && (kPieces % WAVE == 0 || w < kPieces)) {
             float x[4];
-            cvt4(pg[b], x);
-            const float4 db = *(const float4*)(dt_bias + (size_t)h * D + d);
+            cvt4(pg[n], x);
+            const float4 bd = *(const float4*)(db + d);
             *(float4*)(gs + 4 * w) =
-                make_float4(decay_f(rate, x[0] + db.x), decay_f(rate, x[1] + db.y),
-                            decay_f(rate, x[2] + db.z), decay_f(rate, x[3] + db.w));
+                make_float4(decay_f(rate, x[0] + bd.x), decay_f(rate, x[1] + bd.y),
+                            decay_f(rate, x[2] + bd.z), decay_f(rate, x[3] + bd.w));
           }
         }
       }
     }
     __syncthreads();
-    if (t0 + kTile < s1) prefetch(t0 + kTile);
+    if (t0 + kTok < s1) prefetch(t0 + kTok);
     for (int tt = 0; tt < nt; ++tt) {
       const float vj = vs[tt * W + kCols * c + (lane >> 4)];  // the lane's total's column
       const float beta = gb[2 * tt + 1];

@@ -1007,7 +1007,8 @@ def lipulorn_preset(width: int, layers: int, vocab: int = 32000, head_dim: int =
     feed-forward is a dense 3.5 x width gated layer (times ff_scale, for
     matching another model's size)."""
     heads = max(1, width // head_dim)
-    mlp = {"kind": "dense", "ff": max(16, int(3.5 * ff_scale * width) // 16 * 16)}
+    step = 256 if width >= 1024 else 16
+    mlp = {"kind": "dense", "ff": max(16, int(3.5 * ff_scale * width) // step * step)}
     att = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": head_dim,
            "vdim": head_dim, "scale": head_dim ** -0.5, "mask": {"size": window}}
     delta = {"heads": heads, "kv_heads": max(1, heads // 2), "dim": head_dim,
