@@ -7,6 +7,8 @@
 // and writes the token-major layout the attention kernels read.
 #include "seq_common.h"
 
+#include <algorithm>
+
 namespace {
 
 typedef __attribute__((ext_vector_type(4))) short bf16x4;
@@ -14,7 +16,8 @@ typedef __attribute__((ext_vector_type(4))) float f32x4;
 
 constexpr int kHlWaves = 4;
 
-// bf16 on the matrix cores. grid (ceil(T / 64), H), one wave per 16 tokens.
+// bf16 on the matrix cores. grid (ceil(T / 64), H, parts of b_per output
+// channels: several when there are few tokens), one wave per 16 tokens.
 // Y^T = W X^T per 16-channel tile: the wave keeps its tokens' inputs as
 // B-operand fragments in registers (kSteps * 16 >= A) and streams the rows of
 // W[h] as A-operand fragments; a lane ends up with 4 consecutive output
@@ -24,7 +27,7 @@ __global__ __launch_bounds__(kHlWaves * WAVE) void head_linear_mfma_kernel(
     bf16raw* __restrict__ y, int64_t y_stride, int64_t y_hs,
     const bf16raw* __restrict__ x, int64_t x_stride, int64_t x_hs,
     const bf16raw* __restrict__ w, const bf16raw* __restrict__ gate,
-    int64_t gate_stride, int gate_per_head, int T, int H, int A, int B) {
+    int64_t gate_stride, int gate_per_head, int T, int H, int A, int B, int b_per) {
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int col = lane & 15, grp = lane >> 4;
   const int t0 = (blockIdx.x * kHlWaves + wave) * 16;
@@ -42,7 +45,8 @@ __global__ __launch_bounds__(kHlWaves * WAVE) void head_linear_mfma_kernel(
   for (int ks = 0; ks < kSteps; ++ks)
     if (ks < nks) xf[ks] = *(const bf16x4*)(xr + ks * 16);
   const bf16raw* wh = w + (size_t)h * B * A;
-  for (int b0 = 0; b0 < B; b0 += 16) {
+  const int b_end = min(B, (int)(blockIdx.z + 1) * b_per);
+  for (int b0 = blockIdx.z * b_per; b0 < b_end; b0 += 16) {
     const bf16raw* wr = wh + (size_t)(b0 + col) * A + grp * 4;
     f32x4 acc = (f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -139,13 +143,16 @@ void head_linear(torch::Tensor y, torch::Tensor x, torch::Tensor w,
       al8(x.data_ptr(), x.stride(0)) && al8(y.data_ptr(), y.stride(0)) &&
       x_hs % 4 == 0 && y_hs % 4 == 0 && al8(w.data_ptr(), 4) &&
       (gp == nullptr || gph || al8(gp, gs))) {
-    const dim3 grid((T + 16 * kHlWaves - 1) / (16 * kHlWaves), H);
+    const int tb = (T + 16 * kHlWaves - 1) / (16 * kHlWaves), tiles = B / 16;
+    const int parts = std::max(1, std::min(tiles, 512 / (tb * H)));
+    const int b_per = (tiles + parts - 1) / parts * 16;
+    const dim3 grid(tb, H, (B + b_per - 1) / b_per);
     auto launch = [&](auto kern) {
       hipLaunchKernelGGL(kern, grid, dim3(kHlWaves * WAVE), 0, SEQ_STREAM(),
                          (bf16raw*)y.data_ptr(), y.stride(0), y_hs,
                          (const bf16raw*)x.data_ptr(), x.stride(0), x_hs,
                          (const bf16raw*)w.data_ptr(), (const bf16raw*)gp, gs, gph, T,
-                         H, A, B);
+                         H, A, B, b_per);
     };
     if (A <= 128) launch(head_linear_mfma_kernel<8>);
     else launch(head_linear_mfma_kernel<32>);
